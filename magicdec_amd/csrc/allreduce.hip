@@ -624,7 +624,8 @@ extern "C" int md_ar_destroy(md_ar_comm* c) {
     (void)hipDeviceSynchronize();
     for (int i = 0; i < c->n_opened; ++i) (void)hipIpcCloseMemHandle(c->opened[i]);
     (void)hipFree(c->my_data);
-    (void)hipFree(c->my_sig);
+    // my_sig is uncached device memory that kernels have read: it stays allocated until the process ends (allocations made
+    // after such a free have been seen to hold wrong values)
     (void)hipFree(c->my_ctrl);
     delete c;
     return MD_OK;

@@ -28,7 +28,8 @@ def main():
         base = f[:-4]
         with tempfile.TemporaryDirectory() as td:
             out = os.path.join(td, base + ".s")
-            cmd = ["/opt/rocm/bin/hipcc", "-O3", "-std=c++17", "--offload-arch=gfx950", "--cuda-device-only", "-S",
+            cmd = ["/opt/rocm/bin/hipcc", "-O3", "-std=c++17", "--offload-arch=gfx950", "-Xclang", "-target-feature", "-Xclang",
+                   "-packed-fp32-ops", "--cuda-device-only", "-S",
                    os.path.join(CSRC, f), "-o", out]
             if base in EXACT:
                 cmd.insert(3, "-ffp-contract=off")
