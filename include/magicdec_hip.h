@@ -370,6 +370,80 @@ int md_linear_fused_split_add_rmsnorm(const void* x, int64_t ldx, const void* w_
                                       md_stream_t stream);
 
 /* ------------------------------------------------------------------------
+ * K11  the layered decoder designs: fp32 residual stream, token shift, extended attention, xIELU
+ *     (no counterpart in the reference)
+ * md_embed_pos          out[row] = float(table[token]) * scale + float(pos_table[pos]) (pos_table may be NULL); row j of
+ *                       request b = qo_indptr[b] + j, its position pos0[b] + j.
+ * md_resid_norm         x_out = x + delta (or + the sum of n_planes fp32 planes [n_planes][rows][width]; neither: x is
+ *                       normalised as it is), y = x / sqrt(mean(x^2) + eps) * weight * out_scale, all in fp32, y rounded to
+ *                       `dtype` at the end.  x_out must not be x.
+ * md_resid_norm_shift   the same with h = the normalised row and y_t = h_t + (h_{t-1} - h_t) * shift.  The h of the last rows
+ *                       of every sequence live in `ring` [slots][ring_len][width] fp32, position p in entry p % ring_len
+ *                       (slots: ring row of request b; NULL = b); a sequence may be rolled back by ring_len - 2 positions.
+ * md_xielu              y = z > 0 ? softplus(act[0]) z^2 + z / 2 : (1/2 + softplus(act[1])) (e^z - 1 - z) + z / 2 (fp32, one
+ *                       rounding; in place allowed; act = two fp32 values on the device).
+ * md_qk_norm_append     qkv rows (q heads | k heads | v heads) -> q_out [rows][H][pad(D)] and the pages: q and k divided by
+ *                       their root mean square per head when qk_norm is set, rows zero-padded.
+ * md_xattn              softmax attention over the pages; position i sees j <= i in its chunk (chunk = 0: no chunks), score
+ *                       = (q.k) * scale - r1[h] ln(1 + r2[h] (i - j)) (r1 = r2 = NULL: none), sink: one more score of 0
+ *                       without a value.  With q = NULL and qkv given (md_xattn_fused_supported: decode / verify steps of at
+ *                       most 32 rows per kv head) the normalisation and the append happen in the same launch.
+ *                       score_bound > 0: no score exceeds it (e.g. D * scale with qk_norm and r1 >= 0); needed by the
+ *                       matrix-core kernels, 0 = unknown.
+ * pages: k_cache [pages][KH][page_size][pad(D)], v_cache [pages][KH][page_size][pad(DV)], pad = md_xattn_head_pad; the page
+ * list of a request maps every position it may reach (position p: entry p / page_size); rows beyond it are dropped and
+ * counted (md_page_overflow_count).
+ * ---------------------------------------------------------------------- */
+#define MD_T_BF16 0
+#define MD_T_F32 1
+typedef struct md_resid_norm_args {
+    const float* x;
+    const void* delta;         /* dtype [rows][width], or NULL */
+    const float* planes;       /* fp32 [n_planes][rows][width], or NULL */
+    float* x_out;
+    const void* weight;        /* dtype [width] */
+    const void* shift;         /* dtype [width]; md_resid_norm_shift only */
+    void* y;                   /* dtype [rows][width] */
+    const int32_t* qo_indptr;  /* the rest: md_resid_norm_shift only */
+    const int32_t* pos0;
+    const int32_t* slots;
+    float* ring;
+    float eps, out_scale;
+    int rows, width, dtype, n_planes, B, n_max, ring_len;
+} md_resid_norm_args;
+int md_embed_pos(const int64_t* tokens, const void* table, const void* pos_table, int dtype, const int32_t* qo_indptr,
+                 const int32_t* pos0, int B, int n_max, int width, int vocab, int max_pos, float scale, float* out,
+                 md_stream_t stream);
+int md_resid_norm(const md_resid_norm_args* args, md_stream_t stream);
+int md_resid_norm_shift(const md_resid_norm_args* args, md_stream_t stream);
+int md_xielu(const void* z, int64_t z_row_stride, const float* act, void* y, int rows, int dim, int dtype, md_stream_t stream);
+
+typedef struct md_xattn_args {
+    const void* q;             /* [rows][H][pad(D)], or NULL: normalise + append in the attention launch */
+    const void* qkv;           /* raw projection rows */
+    void* k_cache;
+    void* v_cache;
+    void* out;                 /* [rows][H][DV] */
+    const int32_t* qo_indptr;
+    const int32_t* pos0;
+    const int32_t* page_indices;
+    const int32_t* page_indptr;
+    const float* r1;
+    const float* r2;
+    void* workspace;
+    size_t workspace_bytes;
+    int64_t ld_qkv;
+    float eps, scale, score_bound;
+    int B, n_max, H, KH, D, DV, page_size, max_pages, chunk, sink, qk_norm, dtype;
+    int force_plain;           /* 1: the plain kernel (comparison) */
+} md_xattn_args;
+int md_xattn_head_pad(int head_size);
+int md_xattn_fused_supported(const md_xattn_args* args);
+size_t md_xattn_workspace_bytes(const md_xattn_args* args);
+int md_qk_norm_append(const md_xattn_args* args, void* q_out, md_stream_t stream);
+int md_xattn(const md_xattn_args* args, md_stream_t stream);
+
+/* ------------------------------------------------------------------------
  * K10  argmax over a vocab shard / TP merge
  *     reference: Engine/SnapKV/model.py:175-188
  * argmax: per row, max bf16 logit and its lowest index (+index_offset).
@@ -383,6 +457,7 @@ int md_linear_fused_split_add_rmsnorm(const void* x, int64_t ldx, const void* w_
 int md_argmax(const void* logits, int64_t row_stride, int rows, int vocab, int64_t index_offset,
               void* max_val_out /* bf16 [rows], may be NULL */, int64_t* idx_out,
               md_stream_t stream);
+int md_argmax_f32(const float* logits, int64_t row_stride, int rows, int vocab, int64_t* idx_out, md_stream_t stream);
 int md_argmax_tp_slots(const void* logits, int64_t row_stride, int rows, int vocab, int64_t index_offset,
                        int tp_rank, int tp_world, void* vals_out /* bf16 [rows,tp_world] */,
                        int64_t* idx_out /* [rows,tp_world] */, md_stream_t stream);

@@ -24,6 +24,7 @@ from .model_core import PageTable
 
 PAGE_SIZE = 128    # Engine/SnapKV/backend.py:31
 CHUNK = 128        # Engine/SnapKV/backend.py:236
+PREFILL_ROWS = 16384   # rows of one prefill step where the portion is free to choose (models addressed by position, `step`)
 
 
 def default_kv_layout():
@@ -49,11 +50,57 @@ def _pages_per_request(max_batch_size, max_seq_length, page_size=PAGE_SIZE):
     return n, n // max_batch_size
 
 
+def _mapped_pages_per_request(max_seq_length, page_size=PAGE_SIZE):
+    """Pages that hold every position of a request (models that address pages by position)."""
+    return -(-max_seq_length // page_size)
+
+
+class SequencePool:
+    """Slots and pages of an engine whose sequences have unequal lengths and come and go on their own
+    (SnapKVTargetBackend.step): host bookkeeping only.  A sequence owns one slot (its entry in per-sequence state) and as many
+    pages as its tokens need; both go back to the pool when it ends and are handed out again, most recently freed first."""
+
+    def __init__(self, slots, pages, page_size):
+        self.page_size = page_size
+        self.free_slots = list(range(slots))[::-1]
+        self.free_pages = list(range(pages))[::-1]
+        self.seqs = {}                                     # id -> [slot, pages, tokens]
+
+    def pages_for(self, n):
+        return -(-n // self.page_size)
+
+    def fits(self, n_tokens):
+        """Could one more sequence of n_tokens be admitted now?"""
+        return bool(self.free_slots) and self.pages_for(n_tokens) <= len(self.free_pages)
+
+    def length(self, sid):
+        return self.seqs[sid][2] if sid in self.seqs else 0
+
+    def grow(self, sid, n):
+        """n more tokens of sequence `sid` (admitted here if it is new)."""
+        if sid not in self.seqs:
+            if not self.free_slots:
+                raise RuntimeError(f"sequence {sid!r}: every slot is taken ({len(self.seqs)} live sequences)")
+            self.seqs[sid] = [self.free_slots.pop(), [], 0]
+        e = self.seqs[sid]
+        need = self.pages_for(e[2] + n) - len(e[1])
+        if need > len(self.free_pages):
+            raise RuntimeError(f"sequence {sid!r}: {need} more pages needed, {len(self.free_pages)} free")
+        e[1].extend(self.free_pages.pop() for _ in range(need))
+        e[2] += n
+
+    def release(self, sid):
+        slot, pages, _ = self.seqs.pop(sid)
+        self.free_slots.append(slot)
+        self.free_pages.extend(reversed(pages))
+
+
 class _PagedState:
     """One paged cache's bookkeeping under a name prefix ('' or 'draft_') on the owning back-end."""
 
-    def __init__(self, owner, prefix, ppr):
-        self.o, self.p, self.ppr = owner, prefix, ppr
+    def __init__(self, owner, prefix, ppr, mapped=False):
+        """mapped: every request's whole page list is mapped from the start (models that address pages by position)."""
+        self.o, self.p, self.ppr, self.mapped = owner, prefix, ppr, mapped
 
     def _get(self, name):
         return getattr(self.o, self.p + name)
@@ -66,7 +113,7 @@ class _PagedState:
         ppr = self.ppr
         self._set("num_pages_per_request", torch.zeros(B, dtype=torch.int32, device=dev))
         self.host_pages = 0
-        if full_table:   # SnapKV draft cache: all pages mapped from the start (backend.py:87-90)
+        if full_table or self.mapped:   # SnapKV draft cache: all pages mapped from the start (backend.py:87-90)
             self._set("paged_kv_indptr", torch.arange(B + 1, dtype=torch.int32, device=dev) * ppr)
             self._set("paged_kv_indices", torch.arange(B * ppr, dtype=torch.int32, device=dev))
             self.host_pages = ppr
@@ -78,6 +125,8 @@ class _PagedState:
     def map_pages(self, n_pages, last_page_len):
         """Request b maps pages b*ppr .. b*ppr+n_pages-1; last page holds `last_page_len` rows
         (pre_encode, Engine/SnapKV/backend.py:270-275)."""
+        if self.mapped:
+            return
         o, B, dev = self.o, self.o.batch_size, self.o.device
         self.host_pages = n_pages
         self._get("num_pages_per_request").fill_(n_pages)
@@ -87,6 +136,7 @@ class _PagedState:
         self._set("paged_kv_last_page_len", torch.full((B,), last_page_len, dtype=torch.int32, device=dev))
 
     def table(self):
+        # (no slots: request b of a fixed batch is entry b of per-sequence state)
         return PageTable(self._get("paged_kv_indices"), self._get("paged_kv_indptr"),
                          self._get("paged_kv_last_page_len"), max(self.host_pages, 1))
 
@@ -112,6 +162,27 @@ class _BackendBase:
         """The reference compiles with Inductor/Triton + CUDA graphs (Engine/SnapKV/backend.py:116-125); here the
         decode steps are captured into hipGraphs on first use (see Engine/graph.py)."""
         self._use_graphs = True
+
+    def _geometry(self, max_batch_size, max_seq_length):
+        """Page counts and the prefill portion for this batch geometry."""
+        self.mapped = bool(getattr(self.model, "position_addressed", False))
+        if hasattr(self.model, "check_length"):
+            self.model.check_length(max_seq_length)
+        self.page_size = PAGE_SIZE
+        self.max_num_pages, self.max_num_pages_per_request = _pages_per_request(max_batch_size, max_seq_length)
+        self.prefill_chunk = CHUNK
+        if self.mapped:
+            self.max_num_pages_per_request = _mapped_pages_per_request(max_seq_length)
+            self.max_num_pages = max_batch_size * self.max_num_pages_per_request
+            self.prefill_chunk = max(CHUNK, min(4096, PREFILL_ROWS // max_batch_size // CHUNK * CHUNK))
+
+    def _sequence_state(self, dec_len):
+        """Extra setup_caches arguments of models with per-sequence state: one entry per request, deep enough for rejecting
+        every draft token of a verify step."""
+        if not self.mapped:
+            return {}
+        from .model_layers import STATE_RING
+        return dict(slots=self.batch_size, state_ring=max(STATE_RING, int(dec_len) + 2))
 
     def _qo(self, n):
         return self.qo_indptr * n
@@ -161,8 +232,10 @@ class SnapKVTargetBackend(_BackendBase):
 
     @torch.no_grad()
     def setup_caches(self, max_batch_size: int = 1, max_seq_length: int = 2048, draft_budget=0, window_size=32,
-                     kv_dtype="bf16", kv_layout=None):
-        """kv_dtype="fp8": the full-context cache is OCP e4m3fn with static per-head scales calibrated on the
+                     kv_dtype="bf16", kv_layout=None, num_pages=None):
+        """num_pages: pages of the pool that `step` serves unequal sequences from, when it is not to be a whole page list per
+        request (encode / inference are then unavailable).
+        kv_dtype="fp8": the full-context cache is OCP e4m3fn with static per-head scales calibrated on the
         first prefill chunk (not in the reference).  The compressed draft cache stays bf16.
         kv_layout="HND": the full-context cache keeps the rows of one kv head contiguous inside a page (the
         reference's flashinfer wrappers are planned "NHD": Engine/SnapKV/backend.py:30); same results, longer
@@ -170,11 +243,14 @@ class SnapKVTargetBackend(_BackendBase):
         kv_layout = default_kv_layout() if kv_layout is None else kv_layout
         self.max_length, self.batch_size = max_seq_length, max_batch_size
         dev = self.device
-        self.page_size = PAGE_SIZE
-        self.max_num_pages, self.max_num_pages_per_request = _pages_per_request(max_batch_size, max_seq_length)
+        self._geometry(max_batch_size, max_seq_length)
+        self.pool_only = num_pages is not None
+        if self.pool_only:
+            self.max_num_pages = num_pages
+        self.pool = SequencePool(max_batch_size, self.max_num_pages, PAGE_SIZE)
         self.cachelens = torch.zeros(max_batch_size, dtype=torch.int32, device=dev)
         self.qo_indptr = torch.arange(max_batch_size + 1, dtype=torch.int32, device=dev)
-        self._t = _PagedState(self, "", self.max_num_pages_per_request)
+        self._t = _PagedState(self, "", self.max_num_pages_per_request, self.mapped)
         self._t.reset()
         if self.is_spec:
             self.draft_budget, self.window_size = draft_budget, window_size
@@ -192,14 +268,15 @@ class SnapKVTargetBackend(_BackendBase):
         else:
             self.model.setup_caches(num_pages=self.max_num_pages, page_size=PAGE_SIZE,
                                     max_positions=max_seq_length + 256, kv_dtype=kv_dtype, kv_layout=kv_layout,
-                                    decode_rows=self._decode_rows(self.dec_len, two_token_step=False))
+                                    # (a pool's steps have any number of rows: every weight stays in both layouts)
+                                    decode_rows=None if self.pool_only else self._decode_rows(self.dec_len,
+                                                                                              two_token_step=False),
+                                    **self._sequence_state(self.dec_len))
 
     @torch.no_grad()
     def clear_kv(self):
         for b in self.model.layers:
-            b.attention.kv_cache.kv_cache.zero_()
-            if self.is_spec:
-                b.attention.kv_cache.draft_cache.zero_()
+            b.attention.kv_cache.clear()
         self._reset_kv_calibration()
         self.cachelens.zero_()
         self.qo_indptr = torch.arange(self.batch_size + 1, dtype=torch.int32, device=self.device)
@@ -211,17 +288,20 @@ class SnapKVTargetBackend(_BackendBase):
     @torch.no_grad()
     def encode(self, input_ids: torch.LongTensor, benchmark=False):
         """Chunked prefill (backend.py:232-268)."""
+        if self.pool_only or self.pool.seqs:
+            raise RuntimeError("encode: the pages belong to the sequences of step()")
         self.clear_kv()
         self._prefill_begin()
         seq_len = input_ids.shape[1]
         tokens = None
-        num_chunks = (seq_len + CHUNK - 1) // CHUNK
+        chunk = self.prefill_chunk
+        num_chunks = (seq_len + chunk - 1) // chunk
         is_last = False
         done = 0
         for i in range(num_chunks):
-            ids = input_ids[:, i * CHUNK:min((i + 1) * CHUNK, seq_len)]
+            ids = input_ids[:, i * chunk:min((i + 1) * chunk, seq_len)]
             n = ids.shape[1]
-            if n != CHUNK:
+            if n != chunk:
                 is_last = True
             self._t.map_pages(i + 1, n)                       # pre_encode
             self.model.skip_head = i != num_chunks - 1
@@ -238,6 +318,88 @@ class SnapKVTargetBackend(_BackendBase):
             self.draft_cachelens.copy_(self.cachelens)
         self._prefill_end()
         return tokens
+
+    # ------------------------------------------------------------------ sequences of unequal lengths
+    @torch.no_grad()
+    def step(self, entries, want=None, sample=True):
+        """One step of a ragged batch: entries = [(sequence id, its next tokens)]; an id that is not live yet starts a new
+        sequence (slot and pages from the pool), the others go on from what earlier steps left.  Long entries are processed in
+        portions.  want: per entry the places among its tokens whose logits are asked for (None: none).
+        Returns (tokens, logits): with `sample`, the greedy token after every entry's last one (int64 [entries], on the
+        device); the wanted rows in the order of the entries (float or bf16 [wanted, vocab], or None)."""
+        if not entries:
+            return None, None
+        ids = [torch.as_tensor(t, dtype=torch.long).reshape(-1).cpu() for _, t in entries]
+        if len({sid for sid, _ in entries}) != len(entries) or any(t.numel() == 0 for t in ids):
+            raise ValueError("step: every entry names another sequence and brings at least one token")
+        vocab = self.model.tok_embeddings.weight.shape[0]
+        if any(int(t.min()) < 0 or int(t.max()) >= vocab for t in ids):
+            raise ValueError(f"step: token ids must lie in [0, {vocab})")
+        if hasattr(self.model, "check_length"):
+            self.model.check_length(max(self.pool.length(sid) + t.numel() for (sid, _), t in zip(entries, ids)))
+        want = [sorted(set(w)) for w in want] if want is not None else [[]] * len(entries)
+        done = [0] * len(entries)
+        got = [{} for _ in entries]                        # per entry: place -> logits row
+        last = [None] * len(entries)
+        prefill = any(t.numel() > 1 for t in ids)
+        if prefill:
+            self._prefill_begin()
+        while any(d < t.numel() for d, t in zip(done, ids)):
+            live = [k for k, t in enumerate(ids) if done[k] < t.numel()]
+            portion = max(1, PREFILL_ROWS // len(live))
+            take = {k: min(portion, ids[k].numel() - done[k]) for k in live}
+            rows, row0 = [], 0                             # (entry, place | None = sampled only, flat row)
+            for k in live:
+                lo, hi = done[k], done[k] + take[k]
+                places = set(w for w in want[k] if lo <= w < hi)
+                if sample and hi == ids[k].numel():
+                    places.add(hi - 1)
+                rows += [(k, w, row0 + w - lo) for w in sorted(places)]
+                row0 += take[k]
+            tokens, logits = self._ragged_step([(entries[k][0], ids[k][done[k]:done[k] + take[k]]) for k in live],
+                                               [r for _, _, r in rows])
+            for j, (k, w, _) in enumerate(rows):
+                if w in want[k]:
+                    got[k][w] = logits[j]
+                if sample and w == ids[k].numel() - 1:
+                    last[k] = tokens[j]
+            for k in live:
+                done[k] += take[k]
+        if prefill:
+            self._prefill_end()
+        out = [got[k][w] for k in range(len(entries)) for w in want[k]]
+        return (torch.stack(last) if sample else None), (torch.stack(out) if out else None)
+
+    def _ragged_step(self, parts, head_rows):
+        """One model step over parts = [(sequence id, tokens)] (host tensors); logits and greedy tokens of head_rows."""
+        dev, B = self.device, len(parts)
+        n = [t.numel() for _, t in parts]
+        pos, slots, pages, indptr, last = [], [], [], [0], []
+        for sid, t in parts:
+            pos.append(self.pool.length(sid))
+            self.pool.grow(sid, t.numel())
+            slot, pg, length = self.pool.seqs[sid]
+            slots.append(slot)
+            pages += pg
+            indptr.append(len(pages))
+            last.append(length - (len(pg) - 1) * PAGE_SIZE)
+        qo = [0]
+        for v in n:
+            qo.append(qo[-1] + v)
+        # one upload for all the integers of the step
+        flat = torch.tensor(pos + slots + pages + indptr + last + qo, dtype=torch.int32).to(dev)
+        cut = torch.split(flat, [B, B, len(pages), B + 1, B, B + 1])
+        tab = PageTable(cut[2], cut[3], cut[4], max(indptr[i + 1] - indptr[i] for i in range(B)), slots=cut[1])
+        ids = torch.cat([t for _, t in parts]).to(dev)
+        self.model.skip_head = not head_rows
+        rows = torch.tensor(head_rows, dtype=torch.long).to(dev) if head_rows else None
+        tokens = self.model.forward(ids, cut[0], cut[5], tab, n_max=max(n), head_rows=rows)
+        self.model.skip_head = False
+        return (tokens, self.model._last_logits) if head_rows else (None, None)
+
+    def end(self, sid):
+        """Sequence `sid` is finished: its slot and pages go back to the pool."""
+        self.pool.release(sid)
 
     @torch.no_grad()
     def inference(self, input_ids: torch.LongTensor, benchmark=False):
@@ -296,11 +458,10 @@ class SnapKVDraftBackend(_BackendBase):
     def setup_caches(self, max_batch_size: int = 1, max_seq_length: int = 2048, draft_budget=0, window_size=32):
         self.batch_size = max_batch_size
         dev = self.device
-        self.page_size = PAGE_SIZE
-        self.max_num_pages, self.max_num_pages_per_request = _pages_per_request(max_batch_size, max_seq_length)
+        self._geometry(max_batch_size, max_seq_length)
         self.cachelens = torch.zeros(max_batch_size, dtype=torch.int32, device=dev)
         self.qo_indptr = torch.arange(max_batch_size + 1, dtype=torch.int32, device=dev)
-        self._t = _PagedState(self, "", self.max_num_pages_per_request)
+        self._t = _PagedState(self, "", self.max_num_pages_per_request, self.mapped)
         self._t.reset()
         if self.is_compress:
             self.draft_budget, self.window_size = draft_budget, window_size
@@ -314,14 +475,13 @@ class SnapKVDraftBackend(_BackendBase):
                                     decode_rows=self._decode_rows())
         else:
             self.model.setup_caches(num_pages=self.max_num_pages, page_size=PAGE_SIZE,
-                                    max_positions=max_seq_length + 256, decode_rows=self._decode_rows())
+                                    max_positions=max_seq_length + 256, decode_rows=self._decode_rows(),
+                                    **self._sequence_state(2))
 
     @torch.no_grad()
     def clear_kv(self):
         for b in self.model.layers:
-            b.attention.kv_cache.kv_cache.zero_()
-            if self.is_compress:
-                b.attention.kv_cache.draft_cache.zero_()
+            b.attention.kv_cache.clear()
         self._reset_kv_calibration()
         self.cachelens.zero_()
         self.qo_indptr = torch.arange(self.batch_size + 1, dtype=torch.int32, device=self.device)
@@ -336,13 +496,14 @@ class SnapKVDraftBackend(_BackendBase):
         self._prefill_begin()
         seq_len = input_ids.shape[1]
         tokens = None
-        num_chunks = (seq_len + CHUNK - 1) // CHUNK
+        chunk = self.prefill_chunk
+        num_chunks = (seq_len + chunk - 1) // chunk
         is_last = False
         done = 0
         for i in range(num_chunks):
-            ids = input_ids[:, i * CHUNK:min((i + 1) * CHUNK, seq_len)]
+            ids = input_ids[:, i * chunk:min((i + 1) * chunk, seq_len)]
             n = ids.shape[1]
-            if n != CHUNK:
+            if n != chunk:
                 is_last = True
             self._t.map_pages(i + 1, n)
             self.model.skip_head = i != num_chunks - 1
@@ -443,7 +604,7 @@ class StreamingDraftBackend(_BackendBase, _StreamingMixin):
     @torch.no_grad()
     def clear_kv(self):
         for b in self.model.layers:
-            b.attention.kv_cache.kv_cache.zero_()
+            b.attention.kv_cache.clear()
         self._reset_kv_calibration()
         self.cachelens.zero_()
         self.qo_indptr = torch.arange(self.batch_size + 1, dtype=torch.int32, device=self.device)
@@ -507,8 +668,7 @@ class StreamingSelfSpecBackend(_BackendBase, _StreamingMixin):
     @torch.no_grad()
     def clear_kv(self):
         for b in self.model.layers:
-            b.attention.kv_cache.kv_cache.zero_()
-            b.attention.kv_cache.draft_cache.zero_()
+            b.attention.kv_cache.clear()
         self._reset_kv_calibration()
         self.cachelens.zero_()
         self.draft_cachelens.zero_()

@@ -171,6 +171,11 @@ class KVCache(nn.Module):
         self.kv_len = kv_len
         self.page_size = page_size
 
+    def clear(self):
+        self.kv_cache.zero_()
+        if hasattr(self, "draft_cache"):
+            self.draft_cache.zero_()
+
     def scales(self, which="kv_cache"):
         return (self.k_scale, self.v_scale) if (self.fp8 and which == "kv_cache") else None
 
@@ -239,9 +244,12 @@ class PageTable:
     indptr: torch.Tensor
     last_page_len: torch.Tensor
     max_pages: int  # host upper bound of pages per request
+    slots: Optional[torch.Tensor] = None   # entry of request b in per-sequence state (int32); None: b
 
 
 class Transformer(nn.Module):
+    position_addressed = False   # True: the page list maps every position a request may reach (no last-page length)
+
     def __init__(self, config: ModelArgs):
         super().__init__()
         self.config = config
@@ -263,6 +271,13 @@ class Transformer(nn.Module):
         return cls(ModelArgs.from_name(name))
 
     # ------------------------------------------------------------------ setup
+    def check_length(self, max_seq_length):
+        """Raises if sequences of this length cannot be served (models with a fixed number of positions)."""
+
+    def rollback_depth(self):
+        """Tokens a sequence may be rolled back by (None: any number)."""
+        return None
+
     def setup_caches(self, num_pages, page_size=128, spec=False, draft_num_pages=0, draft_budget=0, window_size=32,
                      max_positions=None, streaming=False, kv_dtype="bf16", kv_layout="NHD", decode_rows=None):
         """Allocates the per-layer KV slabs and the device-side constants of the step
@@ -316,6 +331,15 @@ class Transformer(nn.Module):
             self._w13.append(w13)
         self._pack_weights()
 
+    def _streamed_weights(self):
+        """(weight, packed for SwiGLU, role, layer index | None) of every linear a decode step may stream."""
+        for i, b in enumerate(self.layers):
+            yield self._w13[i], True, "w13", i
+            yield b.attention.wqkv.weight, False, "wqkv", i
+            yield b.attention.wo.weight, False, "wo", i
+            yield b.feed_forward.w2.weight, False, "w2", i
+        yield self.output.weight, False, "head", None
+
     def _pack_weights(self, force=False):
         """Streaming-layout copies (ops.PackedWeight) of the weights the hand-written GEMMs serve in decode / verify
         steps -- md_linear for the long weight streams, md_linear_fused for the launch-bound small products
@@ -329,13 +353,9 @@ class Transformer(nn.Module):
 
         todo = []
         self._roles = {}                                # id(weight) -> (role, layer index | None)
-        for i, b in enumerate(self.layers):
-            for w, sw, role in ((self._w13[i], True, "w13"), (b.attention.wqkv.weight, False, "wqkv"),
-                                (b.attention.wo.weight, False, "wo"), (b.feed_forward.w2.weight, False, "w2")):
-                todo.append((w, sw))
-                self._roles[id(w)] = (role, i)
-        todo.append((self.output.weight, False))
-        self._roles[id(self.output.weight)] = ("head", None)
+        for w, sw, role, i in self._streamed_weights():
+            todo.append((w, sw))
+            self._roles[id(w)] = (role, i)
         todo = [(w, sw) for w, sw in todo if w.shape[1] % 16 == 0 and self._wants_packed(self._roles[id(w)][0], w)]
         # headroom check: the copies double the served weights' footprint (17 GB for the 8B + 1B pair)
         # and are made AFTER the KV slabs exist; if they do not fit beside them with a margin for the step's workspaces,
@@ -658,15 +678,17 @@ class Transformer(nn.Module):
         v = qkv[:, (H + KH) * D:].unflatten(1, (KH, D))
         return q, k, v, rows
 
-    def _run(self, idx, attn_fn):
+    def _run(self, idx, attn_fn, n_max=None, head_rows=None):
         """embed -> L x (norm, attention, +res, norm, mlp, +res) -> norm -> head -> argmax.
         attn_fn(i, layer, y, n) -> attention output [rows, H, D]: the qkv projection, RoPE, the KV append and the
         attention of layer i over the normalised hidden states y [rows, dim].
         With self.skip_head set (non-final prefill chunks, whose tokens the reference computes and discards,
-        Engine/SnapKV/backend.py:239-263) the lm head is skipped and None is returned."""
+        Engine/SnapKV/backend.py:239-263) the lm head is skipped and None is returned.
+        idx is [B, n], or flat (requests of unequal rows; n_max bounds them): then head_rows may name the flat rows whose
+        logits and tokens are wanted."""
         assert self._ready, "call setup_caches first"
-        B, n = idx.shape
-        x = self.tok_embeddings(idx).view(B * n, -1)
+        n = idx.shape[1] if idx.dim() == 2 else n_max
+        x = self.tok_embeddings(idx).view(idx.numel(), -1)
         layers = self.layers
         y = ops.rmsnorm(x, layers[0].attention_norm.weight, layers[0].attention_norm.eps)
         for i, layer in enumerate(layers):
@@ -678,9 +700,11 @@ class Transformer(nn.Module):
             x, y = self._proj_add_norm(act, layer.feed_forward.w2, x, nxt, layer.feed_forward.process_group)
         if self.skip_head:
             return None
+        if head_rows is not None:
+            y = (y.materialize() if isinstance(y, ops.DeferredNorm) else y).index_select(0, head_rows)
         logits = self._linear(y, self.output)                         # [rows, vocab / tp]; materialises a deferred norm
         self._last_logits = logits
-        return self._argmax(logits).view(B, n)
+        return self._argmax(logits).view(idx.shape) if head_rows is None else self._argmax(logits)
 
     def _argmax(self, logits):
         """argmax, or the TP merge of per-rank maxima (Engine/SnapKV/model.py:178-188): two sum-all-reduces of
@@ -700,7 +724,7 @@ class Transformer(nn.Module):
 
     # ------------------------------------------------------------------ step variants
     def _std_step(self, idx, offsets, qo_indptr, tab: PageTable, which="kv_cache", tab2: PageTable = None,
-                  snap_tab: PageTable = None, calibrate=False):
+                  snap_tab: PageTable = None, calibrate=False, n_max=None, head_rows=None):
         """rope(offsets) -> append (-> 2nd cache) -> attention (-> SnapKV select): Attention.forward / verify /
         draft_forward / prefill of Engine/SnapKV/model.py:322-387."""
         c = self.config
@@ -718,7 +742,7 @@ class Transformer(nn.Module):
             # the fused kernel derives (request, row-in-request) from the row index: every request must own exactly n
             # consecutive rows (what every back-end passes: qo_indptr = arange * n); anything else takes rope_append, which
             # honours qo_indptr
-            uniform_rows = yin.shape[0] == (qo_indptr.numel() - 1) * n
+            uniform_rows = idx.dim() == 2 and yin.shape[0] == (qo_indptr.numel() - 1) * n
             if (not need_calib and uniform_rows and self._fused_here(yin, att.wqkv.weight, "qkv", pro is not None)
                     and c.head_dim in (64, 128)):
                 # (deferred RMSNorm +) wqkv + bias + RoPE + paged append (both caches of a self-speculation verify):
@@ -749,10 +773,10 @@ class Transformer(nn.Module):
                                   self.draft_budget, POOL_KERNEL, kvc.draft_cache, snap_tab.indices, snap_tab.indptr,
                                   snap_tab.last_page_len, self.workspace, kv_scales=scales, kv_layout=layout)
             return o
-        return self._run(idx, fn)
+        return self._run(idx, fn, n_max, head_rows)
 
-    def forward(self, idx, input_pos, kv_append_indptr, tab: PageTable):
-        return self._std_step(idx, input_pos, kv_append_indptr, tab)
+    def forward(self, idx, input_pos, kv_append_indptr, tab: PageTable, n_max=None, head_rows=None):
+        return self._std_step(idx, input_pos, kv_append_indptr, tab, n_max=n_max, head_rows=head_rows)
 
     def verify(self, idx, input_pos, kv_append_indptr, tab: PageTable, draft_tab: PageTable = None):
         """Self-spec SnapKV verify also appends the gamma+1 rows to the draft cache (model.py:338-353)."""

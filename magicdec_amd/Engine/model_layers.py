@@ -1,0 +1,257 @@
+"""The layered decoder: one model class for every design of Engine/designs.py.
+
+It is a `Transformer` whose layers follow a `DecoderSpec`: the same step interface (prefill / forward over a page table and
+device-side positions, token ids out), weight packing, GEMM policy, graph capture and back-ends; what differs is what a layer
+computes:
+
+* the residual stream is float32; the residual add, the RMS norm behind it and the token shift are one launch
+  (ops.resid_norm), fed by the projection's 16-bit rows or directly by a split-K product's float32 planes;
+* attention is ops.extended_attention: separate query/key and value head sizes, query/key norm, distance bias, chunk mask and
+  sink, over `SplitKVCache` pages that are addressed by position; decode steps normalise, append and attend in one launch;
+* the last unshifted rows of every sequence live in a small float32 ring per layer, indexed by position (ops.resid_norm), so a
+  step may be repeated (graph capture) or rolled back (rejected draft tokens) without saving state.
+
+With float32 weights every kernel runs in 32-bit (plain attention kernel, library GEMMs without reduced-precision modes).
+"""
+from __future__ import annotations
+
+import math
+
+import torch
+import torch.nn as nn
+from torch.nn import functional as F
+
+from .. import ops
+from .designs import DecoderSpec, LayerSpec
+from .model_core import PageTable, RMSNorm, Transformer
+
+STATE_RING = 16        # unshifted rows kept per sequence and layer: rollbacks of up to STATE_RING - 2 tokens
+
+
+class SplitKVCache(nn.Module):
+    """Paged keys [pages, KH, page_size, pad(D)] and values [pages, KH, page_size, pad(DV)] of one layer.  A page list maps
+    every position of its sequence, so stale rows are never read and nothing has to be cleared between sequences."""
+
+    def __init__(self, num_pages, page_size, kv_heads, dim, vdim, dtype):
+        super().__init__()
+        self.register_buffer("k_cache", torch.zeros((num_pages, kv_heads, page_size, ops.head_pad(dim)), dtype=dtype),
+                             persistent=False)
+        self.register_buffer("v_cache", torch.zeros((num_pages, kv_heads, page_size, ops.head_pad(vdim)), dtype=dtype),
+                             persistent=False)
+        self.calibrated = False
+
+    def clear(self):
+        pass
+
+
+class ExtendedAttention(nn.Module):
+    def __init__(self, dim, spec):
+        super().__init__()
+        self.spec = spec
+        self.wqkv = nn.Linear(dim, (spec.heads + spec.kv_heads) * spec.dim + spec.kv_heads * spec.vdim, bias=False)
+        self.wo = nn.Linear(spec.heads * spec.vdim, dim, bias=False)
+        if spec.distance_bias:
+            self.r1 = nn.Parameter(torch.empty(spec.heads))
+            self.r2 = nn.Parameter(torch.empty(spec.heads))
+        self.kv_cache = None
+
+    def kernel_spec(self, eps, max_positions) -> ops.XattnSpec:
+        """The layer's constants for the kernels, with the bound on its scores that the matrix-core kernels rely on:
+        normalised queries and keys have |q.k| <= D, and a bias with r1 < 0 adds at most |r1| ln(1 + r2 * distance)."""
+        s = self.spec
+        r1 = r2 = None
+        bound = 1.02 * s.dim * abs(s.scale) if s.qk_norm else 0.0        # 2 %: the 16-bit rounding of q and k
+        if s.distance_bias:
+            r1, r2 = self.r1.detach().float().contiguous(), self.r2.detach().float().contiguous()
+            reach = (min(s.chunk, max_positions) if s.chunk else max_positions) - 1
+            a, b = r1.double().cpu(), r2.double().cpu()
+            if bool((b < 0).any()) or not bool(torch.isfinite(a).all() and torch.isfinite(b).all()):
+                bound = 0.0
+            elif bound > 0:
+                bound += float(((-a).clamp(min=0) * torch.log1p(b * reach)).max())
+        return ops.XattnSpec(s.heads, s.kv_heads, s.dim, s.vdim, s.scale, eps, s.chunk, s.sink, s.qk_norm, r1, r2, bound)
+
+
+class DenseMLP(nn.Module):
+    """down . act(up . h)"""
+
+    def __init__(self, dim, spec):
+        super().__init__()
+        if spec.act != "xielu":
+            raise ValueError(f"unknown activation {spec.act!r}")
+        self.up = nn.Linear(dim, spec.ff, bias=False)
+        self.down = nn.Linear(spec.ff, dim, bias=False)
+        self.act = nn.Parameter(torch.empty(2))
+
+
+class DecoderLayer(nn.Module):
+    def __init__(self, dim, eps, spec: LayerSpec):
+        super().__init__()
+        self.attention_norm = RMSNorm(dim, eps)
+        self.attention = ExtendedAttention(dim, spec.attention)
+        if spec.token_shift:
+            self.shift = nn.Parameter(torch.empty(dim))
+        self.feed_forward = None
+        if spec.mlp is not None:
+            self.ffn_norm = RMSNorm(dim, eps)
+            self.feed_forward = DenseMLP(dim, spec.mlp)
+
+
+class LayeredTransformer(Transformer):
+    position_addressed = True        # pages are found by position: the back-end maps a request's whole page list at once
+
+    def __init__(self, spec: DecoderSpec):
+        nn.Module.__init__(self)
+        self.config = self.spec = spec
+        self.tok_embeddings = nn.Embedding(spec.vocab_size, spec.dim)
+        self.pos_embeddings = nn.Embedding(spec.max_positions, spec.dim) if spec.max_positions else None
+        self.layers = nn.ModuleList(DecoderLayer(spec.dim, spec.norm_eps, s) for s in spec.layers)
+        self.norm = RMSNorm(spec.dim, spec.norm_eps)
+        self.output = nn.Linear(spec.dim, spec.vocab_size, bias=False)
+        self.world_size = self.rank = self.process_group = None
+        self._ready, self.skip_head = False, False
+
+    # ------------------------------------------------------------------ weights
+    def state_from_tensors(self, t):
+        """state_dict of this model from the tensors of a model.safetensors file (embed, pos, l<i>.norm1, l<i>.mix.q, ...)."""
+        used = set()
+
+        def take(name):
+            used.add(name)
+            if name not in t:
+                raise KeyError(f"model.safetensors has no tensor '{name}'")
+            return t[name]
+        sd = {"tok_embeddings.weight": take("embed"), "norm.weight": take("final.norm"), "output.weight": take("head")}
+        if self.pos_embeddings is not None:
+            sd["pos_embeddings.weight"] = take("pos")
+        for i, s in enumerate(self.spec.layers):
+            p, m = f"layers.{i}.", f"l{i}."
+            sd[p + "attention_norm.weight"] = take(m + "norm1")
+            if s.token_shift:
+                sd[p + "shift"] = take(m + "shift")
+            sd[p + "attention.wqkv.weight"] = torch.cat([take(m + "mix.q"), take(m + "mix.k"), take(m + "mix.v")])
+            sd[p + "attention.wo.weight"] = take(m + "mix.o")
+            if s.attention.distance_bias:
+                sd[p + "attention.r1"], sd[p + "attention.r2"] = take(m + "mix.r1"), take(m + "mix.r2")
+            if s.mlp is not None:
+                sd[p + "ffn_norm.weight"] = take(m + "norm2")
+                sd[p + "feed_forward.up.weight"], sd[p + "feed_forward.down.weight"] = take(m + "mlp.up"), take(m + "mlp.down")
+                sd[p + "feed_forward.act"] = take(m + "mlp.act")
+        extra = sorted(set(t) - used)
+        if extra:
+            raise KeyError(f"model.safetensors holds tensors this design does not have: {extra[:8]}")
+        want = dict(self.named_parameters())
+        for k, v in sd.items():
+            if tuple(v.shape) != tuple(want[k].shape):
+                raise ValueError(f"model.safetensors: {k} is {tuple(v.shape)}, config.json says {tuple(want[k].shape)}")
+        return sd
+
+    # ------------------------------------------------------------------ setup
+    def check_length(self, max_seq_length):
+        if self.spec.max_positions and max_seq_length > self.spec.max_positions:
+            raise ValueError(f"sequences of {max_seq_length} tokens: the model has {self.spec.max_positions} position vectors")
+
+    def setup_caches(self, num_pages, page_size=128, spec=False, draft_num_pages=0, draft_budget=0, window_size=32,
+                     max_positions=None, streaming=False, kv_dtype="bf16", kv_layout=None, decode_rows=None, slots=1,
+                     state_ring=STATE_RING):
+        """Per-layer pages and state rings for `slots` sequences.  kv_layout is ignored (there is one layout)."""
+        if spec or streaming:
+            raise NotImplementedError(f"{self.spec.design}: its cache already holds one chunk per sequence of interest; the "
+                                      "compressed draft caches (SnapKV, StreamingLLM) do not apply to it")
+        if kv_dtype != "bf16":
+            raise NotImplementedError(f"{self.spec.design}: the fp8 cache is not available for this design")
+        w = self.output.weight
+        if w.dtype not in (torch.bfloat16, torch.float32):
+            raise NotImplementedError("the layered decoder runs in bfloat16 or float32")
+        dev, c = w.device, self.spec
+        self.page_size, self.slots = page_size, slots
+        self.state_ring = max(int(state_ring), 2)
+        longest = max_positions or num_pages * page_size
+        self._xspec, self._rings, self._act = [], [], []
+        for i, (layer, s) in enumerate(zip(self.layers, c.layers)):
+            a = s.attention
+            layer.attention.kv_cache = SplitKVCache(num_pages, page_size, a.kv_heads, a.dim, a.vdim, w.dtype).to(dev)
+            self._xspec.append(layer.attention.kernel_spec(c.norm_eps, longest))
+            self._rings.append(torch.zeros((slots, self.state_ring, c.dim), dtype=torch.float32, device=dev)
+                               if s.token_shift else None)
+            self._act.append(layer.feed_forward.act.detach().float().contiguous() if s.mlp is not None else None)
+        self.workspace = ops.AttnWorkspace(dev)
+        self.decode_rows = tuple(sorted(set(int(r) for r in decode_rows))) if decode_rows else None
+        self._pack_weights()
+        self._ready = True
+
+    def rollback_depth(self):
+        """Tokens a sequence may be rolled back by (None: any number)."""
+        return self.state_ring - 2 if any(r is not None for r in self._rings) else None
+
+    def _streamed_weights(self):
+        if self.output.weight.dtype != torch.bfloat16:
+            return
+        for i, b in enumerate(self.layers):
+            yield b.attention.wqkv.weight, False, "wqkv", i
+            yield b.attention.wo.weight, False, "wo", i
+            if b.feed_forward is not None:
+                yield b.feed_forward.up.weight, False, "up", i
+                yield b.feed_forward.down.weight, False, "down", i
+        yield self.output.weight, False, "head", None
+
+    def _decode_hows(self, role, N, K, int8, M, packed=True):
+        return {self._linear_how(M, N, K, False, int8, True if packed else None, "plain", False)}
+
+    # ------------------------------------------------------------------ the step
+    def _linear(self, x2d, lin, **kw):
+        if x2d.dtype == torch.float32:
+            return F.linear(x2d, lin.weight)
+        return super()._linear(x2d, lin, **kw)
+
+    def _project(self, inp, lin):
+        """Output projection of a sub-layer, in a form ops.resid_norm adds to the residual."""
+        return self._linear(inp, lin)
+
+    def _step(self, idx, offsets, qo_indptr, tab: PageTable, n_max=None, head_rows=None):
+        """One step over `idx` ([B, n], or flat with n_max): embed -> layers -> norm -> head -> argmax.  head_rows: the flat
+        rows whose logits are wanted (None: all)."""
+        assert self._ready, "call setup_caches first"
+        c = self.spec
+        flat = idx.reshape(-1)
+        rows = ops.StepRows(qo_indptr, offsets, idx.shape[1] if idx.dim() == 2 else n_max, tab.slots)
+        x = ops.embed_pos(flat, self.tok_embeddings.weight,
+                          self.pos_embeddings.weight if self.pos_embeddings is not None else None, rows, c.embed_scale)
+        delta = None
+        for i, layer in enumerate(self.layers):
+            att, kvc = layer.attention, layer.attention.kv_cache
+            x, y = ops.resid_norm(x, delta, layer.attention_norm.weight, c.norm_eps,
+                                  shift=getattr(layer, "shift", None), ring=self._rings[i], rows=rows)
+            qkv = self._linear(y, att.wqkv)
+            o = ops.extended_attention(qkv, self._xspec[i], kvc.k_cache, kvc.v_cache, rows, tab.indices, tab.indptr,
+                                       tab.max_pages, self.workspace)
+            delta = self._project(o, att.wo)
+            if layer.feed_forward is not None:
+                x, y = ops.resid_norm(x, delta, layer.ffn_norm.weight, c.norm_eps)
+                z = self._linear(y, layer.feed_forward.up)
+                delta = self._project(ops.xielu(z, self._act[i], out=z), layer.feed_forward.down)
+            if self._layer_hook is not None:
+                self._layer_hook(i, x, delta)
+        if self.skip_head:
+            return None
+        x, y = ops.resid_norm(x, delta, self.norm.weight, c.norm_eps, out_scale=c.logit_scale)
+        if head_rows is not None:
+            y = y.index_select(0, head_rows)
+        logits = self._linear(y, self.output)
+        self._last_logits = logits
+        tokens = self._argmax(logits)
+        return tokens.view(idx.shape) if head_rows is None else tokens
+
+    _layer_hook = None       # called as (layer index, residual, pending delta): diagnostics
+
+    def forward(self, idx, input_pos, kv_append_indptr, tab: PageTable, n_max=None, head_rows=None):
+        return self._step(idx, input_pos, kv_append_indptr, tab, n_max, head_rows)
+
+    def prefill(self, idx, input_pos, kv_append_indptr, tab: PageTable, is_last=False, draft_tab=None, ctx_len=None,
+                n_max=None, head_rows=None):
+        return self._step(idx, input_pos, kv_append_indptr, tab, n_max, head_rows)
+
+    def verify(self, *a, **k):
+        raise NotImplementedError(f"{self.spec.design}: no self-speculation cache")
+
+    draft_forward = stream_prefill = verify

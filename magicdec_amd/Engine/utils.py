@@ -153,8 +153,40 @@ def repeak_head_(model, miss):
         raise RuntimeError("repeak_head_: the head's row-major tensor is released and it has no streaming copy")
 
 
+def _design_weights_(model, seed, device, dtype):
+    """Seeded weights of a layered design where no checkpoint exists: norms 1, small bias slopes, a moderate shift."""
+    _random_init_(model, seed, device, dtype)
+    for name, p in model.named_parameters():
+        leaf = name.rsplit(".", 1)[-1]
+        fill = {"r1": 1.0, "r2": 0.25, "shift": 0.25, "act": 0.0}.get(leaf)
+        if fill is not None:
+            p.data.fill_(fill)
+
+
+def _load_design(spec, checkpoint_path, device, precision, use_tp, seed=1234):
+    """A layered design (Engine/designs.py): config.json + model.safetensors, or seeded weights of a named configuration."""
+    from .model_layers import LayeredTransformer
+    if use_tp:
+        raise NotImplementedError(f"{spec.design}: tensor parallelism is not available for this design")
+    with torch.device("meta"):
+        model = LayeredTransformer(spec)
+    folder = checkpoint_path if checkpoint_path.is_dir() else checkpoint_path.parent
+    weights = folder / "model.safetensors"
+    if weights.exists():
+        from safetensors.torch import load_file
+        model.load_state_dict(model.state_from_tensors(load_file(str(weights))), assign=True)
+    else:
+        print(f"[magicdec_amd] {weights} not found: seeded random weights for this {spec.design} configuration")
+        _design_weights_(model, seed, device, precision)
+    return model.requires_grad_(False).to(device=device, dtype=precision).eval()
+
+
 def _load(transformer_cls, checkpoint_path, device, precision, use_tp, rank_group, group, seed=1234, is_draft=False):
     checkpoint_path = Path(checkpoint_path)
+    from .designs import find_design
+    spec = find_design(checkpoint_path)
+    if spec is not None:
+        return _load_design(spec, checkpoint_path, device, precision, use_tp, seed)
     with torch.device("meta"):
         model = transformer_cls.from_name(checkpoint_path.parent.name)
     int8 = "int8" in str(checkpoint_path)          # Engine/utils.py:201-205 of the reference

@@ -12,7 +12,7 @@ from ctypes import c_char_p, c_double, c_float, c_int, c_int64, c_size_t, c_void
 _HERE = os.path.dirname(os.path.abspath(__file__))
 # MAGICDEC_HIP_LIB: development only -- another build of the same sources (e.g. `make TIMING=1`'s instrumented library)
 LIB_PATH = os.environ.get("MAGICDEC_HIP_LIB") or os.path.join(_HERE, "libmagicdec_hip.so")
-ABI_VERSION = 10
+ABI_VERSION = 11
 
 _lib = None
 _err = None
@@ -32,6 +32,22 @@ class FusedLinearArgs(ctypes.Structure):
                 ("cache2", P), ("page_indices2", P), ("page_indptr2", P), ("last_page_len2", P),
                 ("k_scale", P), ("v_scale", P),
                 ("ssq_out", P), ("pro_ssq", P), ("pro_norm_w", P), ("pro_eps", c_float), ("pro_tiles", I)]
+
+class ResidNormArgs(ctypes.Structure):
+    """md_resid_norm_args of include/magicdec_hip.h."""
+    _fields_ = [("x", P), ("delta", P), ("planes", P), ("x_out", P), ("weight", P), ("shift", P), ("y", P),
+                ("qo_indptr", P), ("pos0", P), ("slots", P), ("ring", P), ("eps", c_float), ("out_scale", c_float),
+                ("rows", I), ("width", I), ("dtype", I), ("n_planes", I), ("B", I), ("n_max", I), ("ring_len", I)]
+
+
+class XattnArgs(ctypes.Structure):
+    """md_xattn_args of include/magicdec_hip.h."""
+    _fields_ = [("q", P), ("qkv", P), ("k_cache", P), ("v_cache", P), ("out", P), ("qo_indptr", P), ("pos0", P),
+                ("page_indices", P), ("page_indptr", P), ("r1", P), ("r2", P), ("workspace", P),
+                ("workspace_bytes", c_size_t), ("ld_qkv", L), ("eps", c_float), ("scale", c_float),
+                ("score_bound", c_float), ("B", I), ("n_max", I), ("H", I), ("KH", I), ("D", I), ("DV", I),
+                ("page_size", I), ("max_pages", I), ("chunk", I), ("sink", I), ("qk_norm", I), ("dtype", I),
+                ("force_plain", I)]
 
 
 _SIGNATURES = {
@@ -80,7 +96,17 @@ _SIGNATURES = {
     "md_rmsnorm": (c_int, [P, P, P, I, I, c_float, P]),
     "md_add_rmsnorm": (c_int, [P, P, P, P, P, I, I, c_float, P]),
     "md_silu_mul": (c_int, [P, P, L, L, P, I, I, P]),
+    "md_embed_pos": (c_int, [P, P, P, I, P, P, I, I, I, I, I, c_float, P, P]),
+    "md_resid_norm": (c_int, [ctypes.POINTER(ResidNormArgs), P]),
+    "md_resid_norm_shift": (c_int, [ctypes.POINTER(ResidNormArgs), P]),
+    "md_xielu": (c_int, [P, L, P, P, I, I, I, P]),
+    "md_xattn_head_pad": (c_int, [I]),
+    "md_xattn_fused_supported": (c_int, [ctypes.POINTER(XattnArgs)]),
+    "md_xattn_workspace_bytes": (c_size_t, [ctypes.POINTER(XattnArgs)]),
+    "md_qk_norm_append": (c_int, [ctypes.POINTER(XattnArgs), P, P]),
+    "md_xattn": (c_int, [ctypes.POINTER(XattnArgs), P]),
     "md_argmax": (c_int, [P, L, I, I, L, P, P, P]),
+    "md_argmax_f32": (c_int, [P, L, I, I, P, P]),
     "md_argmax_tp_slots": (c_int, [P, L, I, I, L, I, I, P, P, P]),
     "md_tp_argmax_merge": (c_int, [P, P, I, I, P, P]),
     "md_accept_rollback": (c_int, [P, P, P, I, P, P, P, P, P, I, I, I, I, L, L, L, P, P, P, P, P, P]),

@@ -32,7 +32,7 @@
 //     K/V tile through LDS); workgroups sharing a (request, kv head) are placed on one XCD (block id mod 8).
 #include <type_traits>
 
-#include "md_common.h"
+#include "attn_common.h"
 
 #include <hip/hip_ext.h>
 
@@ -63,7 +63,6 @@ struct AttnParams {
     const float* v_scale;
 };
 
-constexpr int kVSub = 1056;  // bytes per [32 keys][16 d] V sub-tile (+32 B pad: conflict-free ds_write_b128)
 
 template <int D, int QT>
 __host__ __device__ constexpr int attn_wave_lds() {
@@ -76,14 +75,6 @@ __host__ __device__ constexpr int attn_wave_lds() {
 template <int D, int KT = 32>
 __host__ __device__ constexpr int prefill_stage_bytes() {
     return KT * (D * 2 + 16) + (KT / 32) * (D / 16) * kVSub;   // one shared KT-key K + V tile image (prefill kernel)
-}
-
-__device__ __forceinline__ bf16x8 lds_read_b128(const unsigned char* p) {
-    return *reinterpret_cast<const bf16x8*>(p);
-}
-__device__ __forceinline__ bf16x4 lds_read_tr(const unsigned char* p) {
-    return __builtin_amdgcn_ds_read_tr16_b64_v4bf16(
-        (__attribute__((address_space(3))) bf16x4*)(p));
 }
 
 // decode/verify reads every K/V byte exactly once: non-temporal loads (+5 % of HBM peak measured); the prefill

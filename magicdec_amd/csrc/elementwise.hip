@@ -163,28 +163,67 @@ __global__ __launch_bounds__(256) void silu_mul_kernel(const bf16_t* __restrict_
     }
 }
 
+// xIELU: a quadratic with slope 1/2 at 0 on the right, an exponential one on the left; the coefficients are softplus of two
+// learned numbers.  fp32 inside, one rounding; expm1 keeps e^z - 1 - z accurate near 0
+__device__ __forceinline__ float softplus_f(float x) { return log1pf(expf(-fabsf(x))) + fmaxf(x, 0.f); }
+
+template <typename T, int VEC>
+__global__ __launch_bounds__(256) void xielu_kernel(const T* __restrict__ z, int64_t zs, const float* __restrict__ act, T* y,
+                                                    int rows, int dim) {
+    const float ap = softplus_f(act[0]), an = 0.5f + softplus_f(act[1]);
+    const int nvec = dim / VEC;
+    const int64_t total = (int64_t)rows * nvec;
+    typedef T vec __attribute__((ext_vector_type(VEC)));
+    for (int64_t i = (int64_t)blockIdx.x * blockDim.x + threadIdx.x; i < total; i += (int64_t)gridDim.x * blockDim.x) {
+        const int64_t row = i / nvec;
+        const int c = (int)(i - row * nvec) * VEC;
+        float f[VEC];
+        if constexpr (VEC == 1) {
+            f[0] = (float)z[row * zs + c];
+        } else {
+            const vec v = *reinterpret_cast<const vec*>(z + row * zs + c);
+#pragma unroll
+            for (int e = 0; e < VEC; ++e) f[e] = (float)v[e];
+        }
+#pragma unroll
+        for (int e = 0; e < VEC; ++e) {
+            const float x = f[e];
+            f[e] = (x > 0.f ? ap * x * x : an * (expm1f(fminf(x, 0.f)) - x)) + 0.5f * x;
+        }
+        if constexpr (VEC == 1) {
+            y[row * dim + c] = (T)f[0];
+        } else {
+            vec v;
+#pragma unroll
+            for (int e = 0; e < VEC; ++e) v[e] = (T)f[e];
+            *reinterpret_cast<vec*>(y + row * dim + c) = v;
+        }
+    }
+}
+
 // one workgroup of NT threads per row; lowest index among equal maxima.  Decode steps have few rows (64..256) of a
 // 128K vocabulary: with NT = 1024 (16 waves, 4 loads in flight each) a row is limited by its CU's load issue rate
 // instead of by one wave's memory latency (49 -> ~15 us for 64 rows)
 // slots > 0 (md_argmax_tp_slots): the outputs are [rows, slots] and the row's result goes to column `slot`, zeros to the
 // others -- the one-hot-slot tensors the reference builds with torch.zeros + an index assignment before its two
 // all-reduces (Engine/SnapKV/model.py:178-184), in the argmax launch itself
-template <int NT>
-__global__ __launch_bounds__(NT) void argmax_kernel(const bf16_t* __restrict__ logits, int64_t row_stride, int vocab,
+template <int NT, typename T = bf16_t>
+__global__ __launch_bounds__(NT) void argmax_kernel(const T* __restrict__ logits, int64_t row_stride, int vocab,
                                                     int64_t index_offset, bf16_t* max_val_out, int64_t* idx_out,
                                                     int slots, int slot) {
     __shared__ float sv[NT / 64];
     __shared__ int si[NT / 64];
     const int64_t row = blockIdx.x;
-    const bf16_t* p = logits + row * row_stride;
+    typedef T vec8 __attribute__((ext_vector_type(8)));
+    const T* p = logits + row * row_stride;
     float best = -INFINITY;
     int bi = 0x7fffffff;
     const int nvec = vocab / 8;
-    const bool vec_ok = (((uintptr_t)p) & 15) == 0;
+    const bool vec_ok = (((uintptr_t)p) & (8 * sizeof(T) - 1)) == 0;
     if (vec_ok) {
 #pragma unroll 4
         for (int i = threadIdx.x; i < nvec; i += NT) {
-            const f32x8 f = __builtin_convertvector(reinterpret_cast<const bf16x8*>(p)[i], f32x8);
+            const f32x8 f = __builtin_convertvector(reinterpret_cast<const vec8*>(p)[i], f32x8);
 #pragma unroll
             for (int e = 0; e < 8; ++e) {
                 const float v = f[e];
@@ -196,7 +235,7 @@ __global__ __launch_bounds__(NT) void argmax_kernel(const bf16_t* __restrict__ l
             }
         }
         for (int id = nvec * 8 + threadIdx.x; id < vocab; id += NT) {
-            const float v = bf16_to_f32(p[id]);
+            const float v = (float)p[id];
             if (v > best || (v == best && id < bi)) {
                 best = v;
                 bi = id;
@@ -204,7 +243,7 @@ __global__ __launch_bounds__(NT) void argmax_kernel(const bf16_t* __restrict__ l
         }
     } else {
         for (int id = threadIdx.x; id < vocab; id += NT) {
-            const float v = bf16_to_f32(p[id]);
+            const float v = (float)p[id];
             if (v > best || (v == best && id < bi)) {
                 best = v;
                 bi = id;
@@ -317,6 +356,26 @@ extern "C" int md_silu_mul(const void* a, const void* b, int64_t a_row_stride, i
     return MD_OK;
 }
 
+extern "C" int md_xielu(const void* z, int64_t z_row_stride, const float* act, void* y, int rows, int dim, int dtype,
+                        md_stream_t stream) {
+    MD_CHECK_ARG(z && act && y, "md_xielu: null pointer argument");
+    MD_CHECK_ARG(rows > 0 && dim > 0 && z_row_stride >= dim, "md_xielu: bad shape rows=%d dim=%d", rows, dim);
+    MD_CHECK_ARG(dtype == MD_T_BF16 || dtype == MD_T_F32, "md_xielu: dtype must be MD_T_BF16 or MD_T_F32");
+    const bool vec = dim % 8 == 0 && z_row_stride % 8 == 0 && (((uintptr_t)z | (uintptr_t)y) & 15) == 0;
+    const int64_t total = (int64_t)rows * (vec ? dim / (dtype == MD_T_F32 ? 4 : 8) : dim);
+    const int grid = (int)(total + 255 > 4096 * 256 ? 4096 : (total + 255) / 256);
+    hipStream_t st = (hipStream_t)stream;
+    if (dtype == MD_T_F32) {
+        if (vec) hipLaunchKernelGGL((xielu_kernel<float, 4>), dim3(grid), dim3(256), 0, st, (const float*)z, z_row_stride, act, (float*)y, rows, dim);
+        else hipLaunchKernelGGL((xielu_kernel<float, 1>), dim3(grid), dim3(256), 0, st, (const float*)z, z_row_stride, act, (float*)y, rows, dim);
+    } else {
+        if (vec) hipLaunchKernelGGL((xielu_kernel<bf16_t, 8>), dim3(grid), dim3(256), 0, st, (const bf16_t*)z, z_row_stride, act, (bf16_t*)y, rows, dim);
+        else hipLaunchKernelGGL((xielu_kernel<bf16_t, 1>), dim3(grid), dim3(256), 0, st, (const bf16_t*)z, z_row_stride, act, (bf16_t*)y, rows, dim);
+    }
+    MD_CHECK_LAUNCH("md_xielu");
+    return MD_OK;
+}
+
 extern "C" int md_argmax(const void* logits, int64_t row_stride, int rows, int vocab, int64_t index_offset,
                          void* max_val_out, int64_t* idx_out, md_stream_t stream) {
     MD_CHECK_ARG(logits && idx_out, "md_argmax: null pointer argument");
@@ -328,6 +387,16 @@ extern "C" int md_argmax(const void* logits, int64_t row_stride, int rows, int v
         hipLaunchKernelGGL((argmax_kernel<256>), dim3(rows), dim3(256), 0, (hipStream_t)stream, (const bf16_t*)logits,
                            row_stride, vocab, index_offset, (bf16_t*)max_val_out, idx_out, 0, 0);
     MD_CHECK_LAUNCH("md_argmax");
+    return MD_OK;
+}
+
+extern "C" int md_argmax_f32(const float* logits, int64_t row_stride, int rows, int vocab, int64_t* idx_out,
+                             md_stream_t stream) {
+    MD_CHECK_ARG(logits && idx_out, "md_argmax_f32: null pointer argument");
+    MD_CHECK_ARG(rows > 0 && vocab > 0, "md_argmax_f32: bad shape rows=%d vocab=%d", rows, vocab);
+    hipLaunchKernelGGL((argmax_kernel<256, float>), dim3(rows), dim3(256), 0, (hipStream_t)stream, logits, row_stride, vocab,
+                       (int64_t)0, (bf16_t*)nullptr, idx_out, 0, 0);
+    MD_CHECK_LAUNCH("md_argmax_f32");
     return MD_OK;
 }
 

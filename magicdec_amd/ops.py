@@ -709,14 +709,197 @@ def silu_mul(a, b):
     return y
 
 
+# ----------------------------------------------------------------------------- K11
+MD_T_BF16, MD_T_F32 = 0, 1
+_MODEL_DTYPES = {torch.bfloat16: MD_T_BF16, torch.float32: MD_T_F32}
+
+
+def _model_dtype(t):
+    if t.dtype not in _MODEL_DTYPES:
+        raise TypeError(f"the layered decoder kernels take bfloat16 or float32 tensors, got {t.dtype}")
+    return _MODEL_DTYPES[t.dtype]
+
+
+def _dense(*ts):
+    for t in ts:
+        if t is not None and not t.is_contiguous():
+            raise ValueError("expected contiguous tensors")
+
+
+class StepRows:
+    """Which rows a step runs: request b owns rows qo_indptr[b] .. qo_indptr[b+1]-1 at positions pos0[b] + 0, 1, ...;
+    `slots[b]` is its entry in per-sequence state (None: b); n_max bounds the rows of one request (host)."""
+
+    def __init__(self, qo_indptr, pos0, n_max, slots=None):
+        self.qo_indptr, self.pos0, self.n_max, self.slots = _i32(qo_indptr), _i32(pos0), int(n_max), slots
+        self.B = qo_indptr.numel() - 1
+        if pos0.numel() < self.B or (slots is not None and slots.numel() < self.B):
+            raise ValueError("StepRows: one position and one slot per request expected")
+        if slots is not None:
+            _i32(slots)
+
+
+def embed_pos(tokens, table, pos_table, rows: StepRows, scale=1.0):
+    """float32 residual rows E[token] * scale + P[pos] (pos_table may be None)."""
+    _gpu(tokens, table, pos_table)
+    _dense(tokens, table, pos_table)
+    vocab, width = table.shape
+    if tokens.dtype != torch.int64:
+        raise TypeError("embed_pos: token ids are int64")
+    if pos_table is not None and (pos_table.dtype != table.dtype or pos_table.shape[1] != width):
+        raise ValueError("embed_pos: the position table must match the embedding table")
+    out = torch.empty((tokens.numel(), width), dtype=torch.float32, device=table.device)
+    check(_lib.load().md_embed_pos(_p(tokens), _p(table), _p(pos_table), _model_dtype(table), _p(rows.qo_indptr),
+                                   _p(rows.pos0), rows.B, rows.n_max, width, vocab,
+                                   pos_table.shape[0] if pos_table is not None else 1, float(scale), _p(out), _stream()),
+          "md_embed_pos")
+    return out
+
+
+class Planes:
+    """A projection as n fp32 partial planes [n, rows, width] in a workspace (a split-K product before its combine)."""
+
+    def __init__(self, ptr, n, rows, width):
+        self.ptr, self.n, self.shape = ptr, n, (rows, width)
+
+
+def resid_norm(x, delta, weight, eps, out_scale=1.0, shift=None, ring=None, rows: StepRows = None):
+    """(x + delta, y): the fp32 residual add and the weighted RMS norm behind it, y in weight's dtype.  delta: rows of that
+    dtype, `Planes`, or None (x is returned as it is).  shift [width] + ring [slots, R, width] float32: the token shift
+    (md_resid_norm_shift); the ring is updated."""
+    _gpu(x, weight, shift, ring)
+    _dense(x, weight, shift, ring)
+    M, width = x.shape
+    if x.dtype != torch.float32 or weight.numel() != width:
+        raise ValueError("resid_norm: x must be float32 [rows, width], weight [width]")
+    a = _lib.ResidNormArgs()
+    a.x, a.weight, a.rows, a.width = x.data_ptr(), weight.data_ptr(), M, width
+    a.dtype, a.eps, a.out_scale = _model_dtype(weight), float(eps), float(out_scale)
+    x_out = x
+    if delta is not None:
+        if tuple(delta.shape) != (M, width):
+            raise ValueError(f"resid_norm: delta is {tuple(delta.shape)}, the residual {(M, width)}")
+        x_out = torch.empty_like(x)
+        a.x_out = x_out.data_ptr()
+        if isinstance(delta, Planes):
+            a.planes, a.n_planes = delta.ptr, delta.n
+        else:
+            _gpu(delta)
+            _dense(delta)
+            if delta.dtype != weight.dtype:
+                raise TypeError("resid_norm: delta must have the weight's dtype")
+            a.delta = delta.data_ptr()
+    y = torch.empty((M, width), dtype=weight.dtype, device=x.device)
+    a.y = y.data_ptr()
+    lib = _lib.load()
+    if shift is None:
+        check(lib.md_resid_norm(ctypes.byref(a), _stream()), "md_resid_norm")
+    else:
+        if ring.dtype != torch.float32 or ring.dim() != 3 or ring.shape[2] != width or shift.dtype != weight.dtype:
+            raise ValueError("resid_norm: ring must be float32 [slots, R, width], shift of the weight's dtype")
+        a.shift, a.ring, a.ring_len = shift.data_ptr(), ring.data_ptr(), ring.shape[1]
+        a.qo_indptr, a.pos0, a.B, a.n_max = rows.qo_indptr.data_ptr(), rows.pos0.data_ptr(), rows.B, rows.n_max
+        a.slots = rows.slots.data_ptr() if rows.slots is not None else None
+        check(lib.md_resid_norm_shift(ctypes.byref(a), _stream()), "md_resid_norm_shift")
+    return x_out, y
+
+
+def xielu(z, act, out=None):
+    """xIELU of 2-D rows; act = float32 [2] on the device (the numbers in front of the softplus)."""
+    _gpu(z, act)
+    if z.dim() != 2 or z.stride(1) != 1 or act.dtype != torch.float32 or act.numel() != 2:
+        raise ValueError("xielu expects 2-D rows with unit inner stride and float32 act[2]")
+    y = torch.empty(z.shape, dtype=z.dtype, device=z.device) if out is None else out
+    check(_lib.load().md_xielu(_p(z), z.stride(0), _p(act), _p(y), z.shape[0], z.shape[1], _model_dtype(z), _stream()),
+          "md_xielu")
+    return y
+
+
+def head_pad(head_size):
+    """Width the extended attention's pages and queries are padded to."""
+    n = int(_lib.load().md_xattn_head_pad(int(head_size)))
+    if n == 0:
+        raise ValueError(f"head size {head_size} unsupported")
+    return n
+
+
+class XattnSpec:
+    """The constants of one extended-attention layer (md_xattn_args): heads, sizes, score scale, chunk (0: none), softmax
+    sink, query/key norm, and the per-head distance bias r1, r2 (float32 [H] or None).  score_bound: see magicdec_hip.h."""
+
+    def __init__(self, H, KH, D, DV, scale, eps, chunk=0, sink=False, qk_norm=False, r1=None, r2=None, score_bound=0.0):
+        self.H, self.KH, self.D, self.DV = int(H), int(KH), int(D), int(DV)
+        self.scale, self.eps, self.chunk = float(scale), float(eps), int(chunk)
+        self.sink, self.qk_norm, self.score_bound = bool(sink), bool(qk_norm), float(score_bound)
+        for r in (r1, r2):
+            if r is not None and (r.dtype != torch.float32 or r.numel() != self.H or not r.is_contiguous()):
+                raise ValueError("distance bias: float32 [H] expected")
+        self.r1, self.r2 = r1, r2
+
+
+def _xattn_args(s: XattnSpec, k_cache, v_cache, rows: StepRows, page_indices, page_indptr, max_pages, dtype):
+    _gpu(k_cache, v_cache)
+    _dense(k_cache, v_cache)
+    if k_cache.dim() != 4 or k_cache.shape[:3] != v_cache.shape[:3] or k_cache.shape[1] != s.KH:
+        raise ValueError("extended attention: pages must be [pages, KH, page_size, width]")
+    if k_cache.shape[3] != head_pad(s.D) or v_cache.shape[3] != head_pad(s.DV) or k_cache.dtype != dtype:
+        raise ValueError("extended attention: pages of another head size or dtype")
+    if page_indptr.numel() != rows.B + 1:
+        raise ValueError("extended attention: page table of another batch")
+    a = _lib.XattnArgs()
+    a.k_cache, a.v_cache = k_cache.data_ptr(), v_cache.data_ptr()
+    a.qo_indptr, a.pos0, a.B, a.n_max = rows.qo_indptr.data_ptr(), rows.pos0.data_ptr(), rows.B, rows.n_max
+    a.page_indices, a.page_indptr = _i32(page_indices).data_ptr(), _i32(page_indptr).data_ptr()
+    a.page_size, a.max_pages = k_cache.shape[2], int(max_pages)
+    a.H, a.KH, a.D, a.DV, a.scale, a.eps = s.H, s.KH, s.D, s.DV, s.scale, s.eps
+    a.chunk, a.sink, a.qk_norm, a.score_bound = s.chunk, int(s.sink), int(s.qk_norm), s.score_bound
+    a.r1 = s.r1.data_ptr() if s.r1 is not None else None
+    a.r2 = s.r2.data_ptr() if s.r2 is not None else None
+    a.dtype = _MODEL_DTYPES[dtype]
+    return a
+
+
+def extended_attention(qkv, s: XattnSpec, k_cache, v_cache, rows: StepRows, page_indices, page_indptr, max_pages,
+                       workspace: AttnWorkspace, fuse=True, plain=False):
+    """One attention layer over the raw projection rows qkv [M, H*D + KH*D + KH*DV]: normalise q and k, append k and v,
+    attend.  Returns [M, H * DV].  Decode / verify steps are one launch where md_xattn_fused_supported (fuse=False: the
+    separate normalise + append launch); plain=True forces the plain attention kernel (comparison)."""
+    _gpu(qkv)
+    M = qkv.shape[0]
+    if qkv.dim() != 2 or qkv.stride(1) != 1 or qkv.shape[1] != (s.H + s.KH) * s.D + s.KH * s.DV:
+        raise ValueError("extended attention: qkv rows must be q | k | v heads")
+    lib = _lib.load()
+    a = _xattn_args(s, k_cache, v_cache, rows, page_indices, page_indptr, max_pages, qkv.dtype)
+    a.qkv, a.ld_qkv = qkv.data_ptr(), qkv.stride(0)
+    out = torch.empty((M, s.H * s.DV), dtype=qkv.dtype, device=qkv.device)
+    a.out, a.force_plain = out.data_ptr(), int(plain)
+    q = None
+    if (plain or not fuse or qkv.stride(0) % 8 or qkv.data_ptr() % 16 or not lib.md_xattn_fused_supported(ctypes.byref(a))):
+        q = torch.empty((M, s.H, k_cache.shape[3]), dtype=qkv.dtype, device=qkv.device)
+        check(lib.md_qk_norm_append(ctypes.byref(a), _p(q), _stream()), "md_qk_norm_append")
+        a.q = q.data_ptr()
+    nbytes = lib.md_xattn_workspace_bytes(ctypes.byref(a))
+    if nbytes and not plain:
+        ws = workspace.get(nbytes + 256)
+        off = (-ws.data_ptr()) % 256
+        a.workspace, a.workspace_bytes = ws.data_ptr() + off, nbytes
+    check(lib.md_xattn(ctypes.byref(a), _stream()), "md_xattn")
+    return out
+
+
 # ----------------------------------------------------------------------------- K10
 def argmax(logits, index_offset=0, return_values=False):
-    """Row-wise argmax of bf16 logits [rows, vocab] (lowest index among equal maxima)."""
+    """Row-wise argmax of bf16 (or float32) logits [rows, vocab] (lowest index among equal maxima)."""
     _gpu(logits)
     if logits.dim() != 2 or logits.stride(1) != 1:
         raise ValueError("argmax expects [rows, vocab] with unit inner stride")
     rows, vocab = logits.shape
     idx = torch.empty(rows, dtype=torch.int64, device=logits.device)
+    if logits.dtype == torch.float32:
+        if return_values or index_offset:
+            raise ValueError("argmax: values and index offsets exist for bf16 logits")
+        check(_lib.load().md_argmax_f32(_p(logits), logits.stride(0), rows, vocab, _p(idx), _stream()), "md_argmax_f32")
+        return idx
     vals = torch.empty(rows, dtype=logits.dtype, device=logits.device) if return_values else None
     lib = _lib.load()
     check(lib.md_argmax(_p(logits), logits.stride(0), rows, vocab, int(index_offset), _p(vals), _p(idx), _stream()),
