@@ -105,6 +105,11 @@ def parse(argv=None):
                          "Default (round 6): peaked with miss = 0.2, so that the driver's line carries a MEASURED "
                          "acceptance next to the replay that defines `value`; timings are weight-value independent "
                          "(ms_per_step of the two agree to 0.1 %%: profiles/r06_bench_cfg3_peaked_miss_sweep_c7.json)")
+    ap.add_argument("--design", default=None, metavar="furitar",
+                    help="instead of a workload: prefill and decode throughput of a layered decoder design at a few sizes, beside "
+                         "the Llama-style model of equal size (magicdec_amd/design_bench.py)")
+    ap.add_argument("--design-sizes", nargs="*", default=None, help="sizes of --design (default: all)")
+    ap.add_argument("--design-only", default=None, choices=["design", "zoo_llama"], help="one side only (profiling)")
     return ap.parse_args(argv)
 
 
@@ -192,6 +197,9 @@ def main(device=None):
     """`device` is None in production (one cuda device per rank); tests/test_bench_cpu.py passes "cpu" from a wrapper
     that first installs its device-op stand-ins, to drive the launcher + rendezvous + JSON contract without a GPU."""
     args = parse()
+    if args.design:
+        from magicdec_amd import design_bench
+        return design_bench.main(args)
     if "WORLD_SIZE" not in os.environ and args.gpus > 1:
         sys.exit(self_launch(args.gpus))
     world = int(os.environ.get("WORLD_SIZE", "1"))

@@ -301,6 +301,7 @@ int md_linear_block_add_rmsnorm(const void* x, int64_t ldx, const void* w_packed
  *   MD_FL_NONE         out[M][N]   = bf16(acc + bias)
  *   MD_FL_SWIGLU       out[M][N/2] = bf16(bf16(silu(bf16(h1))) * bf16(h3)); W packed for MD_EPI_SWIGLU, no bias
  *   MD_FL_RESID        out[M][N]   = bf16(resid + bf16(acc + bias))                 (the bf16 residual add)
+ *   MD_FL_XIELU        out[M][N]   = bf16(xielu(acc)), no bias (md_xielu)
  *   MD_FL_ROPE_APPEND  N = (H + 2 KH) * D fused qkv rows [q; k; v]: q columns -> interleaved RoPE -> out = q_rot
  *                      [M][H*D] (contiguous); k columns -> RoPE -> paged cache; v columns -> paged cache.  Request b
  *                      owns rows [b * rows_per_req, (b+1) * rows_per_req) (uniform append, what a decode step has);
@@ -313,6 +314,7 @@ int md_linear_block_add_rmsnorm(const void* x, int64_t ldx, const void* w_packed
 #define MD_FL_SWIGLU 1
 #define MD_FL_RESID 2
 #define MD_FL_ROPE_APPEND 3
+#define MD_FL_XIELU 4
 typedef struct md_fused_linear_args {
     const void* x;            /* [M][K] bf16, row stride ldx (elements) */
     const void* w_packed;     /* streaming layout (md_linear, w_packed = 1) */
@@ -345,6 +347,7 @@ typedef struct md_fused_linear_args {
     const void* pro_norm_w;   /* bf16 [K] */
     float pro_eps;
     int pro_tiles;
+    const float* act;         /* MD_FL_XIELU: the two fp32 numbers of the activation (md_xielu) */
 } md_fused_linear_args;
 int md_linear_fused_supported(int M, int N, int K, int epilogue);
 int md_linear_fused(const md_fused_linear_args* args, md_stream_t stream);
@@ -382,6 +385,10 @@ int md_linear_fused_split_add_rmsnorm(const void* x, int64_t ldx, const void* w_
  *                       (slots: ring row of request b; NULL = b); a sequence may be rolled back by ring_len - 2 positions.
  * md_xielu              y = z > 0 ? softplus(act[0]) z^2 + z / 2 : (1/2 + softplus(act[1])) (e^z - 1 - z) + z / 2 (fp32, one
  *                       rounding; in place allowed; act = two fp32 values on the device).
+ * md_linear_planes      x [M][K] . W^T as md_linear_planes_count fp32 partial planes [n][M][N] (0: unsupported) -- one of the
+ *                       split-K GEMMs (W in the streaming layout) without its combine launch: md_resid_norm[_shift] adds the
+ *                       planes to the residual.
+ * md_linear_xielu, md_linear_block_xielu, MD_FL_XIELU (md_linear_fused): the linear with the activation as its epilogue.
  * md_qk_norm_append     qkv rows (q heads | k heads | v heads) -> q_out [rows][H][pad(D)] and the pages: q and k divided by
  *                       their root mean square per head when qk_norm is set, rows zero-padded.
  * md_xattn              softmax attention over the pages; position i sees j <= i in its chunk (chunk = 0: no chunks), score
@@ -414,6 +421,16 @@ typedef struct md_resid_norm_args {
 int md_embed_pos(const int64_t* tokens, const void* table, const void* pos_table, int dtype, const int32_t* qo_indptr,
                  const int32_t* pos0, int B, int n_max, int width, int vocab, int max_pos, float scale, float* out,
                  md_stream_t stream);
+#define MD_PLANES_SKINNY 0
+#define MD_PLANES_TILE 1
+#define MD_PLANES_BLOCK 2
+int md_linear_planes_count(int kind, int M, int N, int K);
+int md_linear_planes(int kind, const void* x, int64_t ldx, const void* w_packed, int M, int N, int K, float* planes,
+                     size_t planes_bytes, md_stream_t stream);
+int md_linear_xielu(const void* x, int64_t ldx, const void* w, int w_packed, const float* act, void* out, int64_t ldo, int M,
+                    int N, int K, void* workspace, size_t workspace_bytes, md_stream_t stream);
+int md_linear_block_xielu(const void* x, int64_t ldx, const void* w_packed, const float* act, void* out, int64_t ldo, int M,
+                          int N, int K, void* workspace, size_t workspace_bytes, md_stream_t stream);
 int md_resid_norm(const md_resid_norm_args* args, md_stream_t stream);
 int md_resid_norm_shift(const md_resid_norm_args* args, md_stream_t stream);
 int md_xielu(const void* z, int64_t z_row_stride, const float* act, void* y, int rows, int dim, int dtype, md_stream_t stream);

@@ -23,6 +23,7 @@ from torch.nn import functional as F
 
 from .. import ops
 from .designs import DecoderSpec, LayerSpec
+from .gemm_policy import choose, use_split
 from .model_core import PageTable, RMSNorm, Transformer
 
 STATE_RING = 16        # unshifted rows kept per sequence and layer: rollbacks of up to STATE_RING - 2 tokens
@@ -196,6 +197,8 @@ class LayeredTransformer(Transformer):
         yield self.output.weight, False, "head", None
 
     def _decode_hows(self, role, N, K, int8, M, packed=True):
+        if role in ("wo", "down"):
+            return {self._project_how(M, N, K, packed)}
         return {self._linear_how(M, N, K, False, int8, True if packed else None, "plain", False)}
 
     # ------------------------------------------------------------------ the step
@@ -204,16 +207,49 @@ class LayeredTransformer(Transformer):
             return F.linear(x2d, lin.weight)
         return super()._linear(x2d, lin, **kw)
 
+    def _project_how(self, M, N, K, packed):
+        """Where an output projection runs: a split-K GEMM up to its float32 planes ("skinny" | "tile" | "block"; the residual
+        add + norm launch that follows is its combine), the skinny GEMM with 16-bit rows ("rows"), or the library."""
+        how = choose(M, N, K, False, False, packed, "resid") if packed else "lib"
+        if packed and how != "block" and (how == "fused" or use_split(M, N, K, "resid")):
+            how = "tile"                     # the tile kernel's residual epilogue is 16-bit: take its K-split form instead
+        if how in ("tile", "block", "skinny") and ops.linear_planes_count(how, M, N, K):
+            return how
+        return "rows" if how == "skinny" and ops.linear_supported(M, N, K) else "lib"
+
     def _project(self, inp, lin):
         """Output projection of a sub-layer, in a form ops.resid_norm adds to the residual."""
-        return self._linear(inp, lin)
+        pk = self._packed.get(id(lin.weight))
+        M, K = inp.shape
+        how = self._project_how(M, lin.weight.shape[0], K, pk is not None) if M <= 256 else "lib"
+        if how in ops.PLANES_KINDS:
+            return ops.linear_planes(inp, pk, how, self.workspace)
+        if how == "rows":
+            return ops.linear(inp, pk, workspace=self.workspace)
+        self._last_M = M
+        return F.linear(inp, self._resident(lin.weight))
+
+    def _up_act(self, y, lin, act):
+        """act(up . y): the activation is the GEMM's epilogue wherever a hand-written kernel runs it."""
+        pk = self._packed.get(id(lin.weight))
+        (M, K), N = y.shape, lin.weight.shape[0]
+        how = self._linear_how(M, N, K, False, False, pk, "plain", False) if pk is not None and M <= 256 else "lib"
+        if how == "fused":
+            return ops.fused_linear(y, pk, xielu=act)
+        if how == "block":
+            return ops.linear_block(y, pk, workspace=self.workspace, xielu=act)
+        if how == "skinny":
+            return ops.linear(y, pk, workspace=self.workspace, xielu=act)
+        self._last_M = M
+        z = F.linear(y, self._resident(lin.weight))
+        return ops.xielu(z, act, out=z)
 
     def _step(self, idx, offsets, qo_indptr, tab: PageTable, n_max=None, head_rows=None):
         """One step over `idx` ([B, n], or flat with n_max): embed -> layers -> norm -> head -> argmax.  head_rows: the flat
         rows whose logits are wanted (None: all)."""
         assert self._ready, "call setup_caches first"
         c = self.spec
-        flat = idx.reshape(-1)
+        flat = idx.reshape(-1).contiguous()
         rows = ops.StepRows(qo_indptr, offsets, idx.shape[1] if idx.dim() == 2 else n_max, tab.slots)
         x = ops.embed_pos(flat, self.tok_embeddings.weight,
                           self.pos_embeddings.weight if self.pos_embeddings is not None else None, rows, c.embed_scale)
@@ -228,8 +264,7 @@ class LayeredTransformer(Transformer):
             delta = self._project(o, att.wo)
             if layer.feed_forward is not None:
                 x, y = ops.resid_norm(x, delta, layer.ffn_norm.weight, c.norm_eps)
-                z = self._linear(y, layer.feed_forward.up)
-                delta = self._project(ops.xielu(z, self._act[i], out=z), layer.feed_forward.down)
+                delta = self._project(self._up_act(y, layer.feed_forward.up, self._act[i]), layer.feed_forward.down)
             if self._layer_hook is not None:
                 self._layer_hook(i, x, delta)
         if self.skip_head:

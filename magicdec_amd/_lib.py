@@ -31,7 +31,7 @@ class FusedLinearArgs(ctypes.Structure):
                 ("cache", P), ("page_indices", P), ("page_indptr", P), ("last_page_len", P),
                 ("cache2", P), ("page_indices2", P), ("page_indptr2", P), ("last_page_len2", P),
                 ("k_scale", P), ("v_scale", P),
-                ("ssq_out", P), ("pro_ssq", P), ("pro_norm_w", P), ("pro_eps", c_float), ("pro_tiles", I)]
+                ("ssq_out", P), ("pro_ssq", P), ("pro_norm_w", P), ("pro_eps", c_float), ("pro_tiles", I), ("act", P)]
 
 class ResidNormArgs(ctypes.Structure):
     """md_resid_norm_args of include/magicdec_hip.h."""
@@ -97,6 +97,10 @@ _SIGNATURES = {
     "md_add_rmsnorm": (c_int, [P, P, P, P, P, I, I, c_float, P]),
     "md_silu_mul": (c_int, [P, P, L, L, P, I, I, P]),
     "md_embed_pos": (c_int, [P, P, P, I, P, P, I, I, I, I, I, c_float, P, P]),
+    "md_linear_planes_count": (c_int, [I, I, I, I]),
+    "md_linear_planes": (c_int, [I, P, L, P, I, I, I, P, c_size_t, P]),
+    "md_linear_xielu": (c_int, [P, L, P, I, P, P, L, I, I, I, P, c_size_t, P]),
+    "md_linear_block_xielu": (c_int, [P, L, P, P, P, L, I, I, I, P, c_size_t, P]),
     "md_resid_norm": (c_int, [ctypes.POINTER(ResidNormArgs), P]),
     "md_resid_norm_shift": (c_int, [ctypes.POINTER(ResidNormArgs), P]),
     "md_xielu": (c_int, [P, L, P, P, I, I, I, P]),

@@ -82,6 +82,11 @@ def baseline_parser():
     """The flags and defaults of tests/baseline_benchmark.py (+ --dataset / --benchmark / --kv_dtype / --kv_layout)."""
     parser = argparse.ArgumentParser(description='Process model configuration and partitions.')
     _common(parser, "baseline")
+    parser.add_argument('--dtype', type=str, default="bfloat16", choices=["bfloat16", "float32"],
+                        help='Compute type (float32: the layered decoder designs only).')
+    parser.add_argument('--ragged', action='store_true',
+                        help='Prompts of unequal lengths (half of --prefix_len and up), served with continuous batching: '
+                             '--B sequences at a time, --max_len - --prefix_len new tokens each.')
     return parser
 
 
@@ -308,7 +313,7 @@ def baseline_main(argv=None):
     setup_seed(args.seed)
     print_(f"Using device={DEVICE}")
     from .Engine.SnapKV.backend import LMBackend
-    engine = LMBackend(dtype=torch.bfloat16, device=DEVICE)
+    engine = LMBackend(dtype=getattr(torch, args.dtype), device=DEVICE)
     engine.load_model(args.model, use_tp=use_tp, rank_group=args.rank_group, group=global_group)
     if args.compile:
         engine.compile()
@@ -320,6 +325,20 @@ def baseline_main(argv=None):
     dataset = _dataset(args, tokenizer, engine.model.tok_embeddings.weight.shape[0])
     dataloader = DataLoader(dataset, batch_size=args.B, shuffle=False, drop_last=True)
     num_eval_steps = min(10, len(dataloader))
+    if args.ragged:
+        g = torch.Generator().manual_seed(args.seed)
+        prompts = []
+        for batch, _ in zip(dataloader, range(num_eval_steps)):
+            n = torch.randint(args.prefix_len // 2, args.prefix_len + 1, (args.B,), generator=g)
+            prompts += [row[:k].tolist() for row, k in zip(batch[0], n.tolist())]
+        out, steps, dt = harness.run_sequences(engine, prompts, args.max_len - args.prefix_len, eot=(eot_1, eot_2))
+        if args.printoutput:
+            for tokens in out:
+                print_(tokenizer.decode(tokens))
+        n_tokens = sum(len(t) for t in out)
+        print_(f"sequences :{len(prompts)}, tokens :{n_tokens}, decode steps :{steps}, total time :{dt:.5f}s")
+        print_(f"Final tokens per second :{n_tokens / dt}")
+        return n_tokens / dt
     total_time, model_steps = 0.0, 0
     for step, batch in enumerate(dataloader):
         if step >= num_eval_steps:

@@ -49,11 +49,12 @@ constexpr int kStageB = BN * BK * 2;            // 16 KiB: [4 column tiles][4 k-
 constexpr int kEpiPitch = BN + 4;               // fp32 epilogue tile [256][132]: 135 168 B inside the rings
 constexpr int lds_bytes(int XS, int WS) { return XS * kStageA + WS * kStageB; }
 
-enum { BE_NONE = 0, BE_SWIGLU = 1 };
+enum { BE_NONE = 0, BE_SWIGLU = 1, BE_XIELU = 2 };
 
 struct BlockParams {
     const bf16_t* x;
     const bf16_t* w;        // streaming layout [N/32][K/16][64][8]
+    const float* act;       // BE_XIELU: the two numbers of the activation
     const bf16_t* bias;     // [N] or null (un-split BE_NONE only; split products get it in the combine launch)
     bf16_t* out;            // un-split: [M][N] (BE_NONE) or [M][N/2] (BE_SWIGLU), row stride ldo
     float* partial;         // split: [S][M][N] fp32, GEMM-column order ([w1; w3] for BE_SWIGLU)
@@ -296,13 +297,21 @@ __global__ __launch_bounds__(512) void block_gemm_kernel(const BlockParams p) {
     } else {
         const int c8 = (tid & 15) * 8;                                        // the thread's 8 columns: the same for every q
         f32x8 bv = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
-        if (p.bias) bv = __builtin_convertvector(*reinterpret_cast<const bf16x8*>(p.bias + tn * BN + c8), f32x8);
+        if (EPI == BE_NONE && p.bias) bv = __builtin_convertvector(*reinterpret_cast<const bf16x8*>(p.bias + tn * BN + c8), f32x8);
 #pragma unroll 4
         for (int q = 0; q < 8; ++q) {
             const int row = (tid + 512 * q) >> 4;
             if (row >= p.M) continue;
             const float* src = tile + row * kEpiPitch + c8;
-            const f32x4 va = *reinterpret_cast<const f32x4*>(src), vb = *reinterpret_cast<const f32x4*>(src + 4);
+            f32x4 va = *reinterpret_cast<const f32x4*>(src), vb = *reinterpret_cast<const f32x4*>(src + 4);
+            if constexpr (EPI == BE_XIELU) {
+                const Xielu f_act(p.act);
+#pragma unroll
+                for (int e = 0; e < 4; ++e) {
+                    va[e] = f_act(va[e]);
+                    vb[e] = f_act(vb[e]);
+                }
+            }
             bf16x8 o;
 #pragma unroll
             for (int e = 0; e < 4; ++e) {
@@ -374,6 +383,7 @@ int setup(BlockParams& p, const void* x, int64_t ldx, const void* w, int M, int 
     p.x = (const bf16_t*)x;
     p.w = (const bf16_t*)w;
     p.bias = nullptr;
+    p.act = nullptr;
     p.out = nullptr;
     p.ldx = ldx;
     p.ldo = 0;
@@ -436,6 +446,35 @@ extern "C" int md_linear_block(const void* x, int64_t ldx, const void* w_packed,
     }
     MD_CHECK_LAUNCH("md_linear_block");
     return MD_OK;
+}
+
+extern "C" int md_linear_block_xielu(const void* x, int64_t ldx, const void* w_packed, const float* act, void* out, int64_t ldo,
+                                     int M, int N, int K, void* workspace, size_t workspace_bytes, md_stream_t stream) {
+    MD_CHECK_ARG(act && out && (((uintptr_t)out) & 15) == 0 && ldo % 8 == 0,
+                 "md_linear_block_xielu: act; out must be 16-byte aligned, ldo %% 8 == 0");
+    BlockParams p;
+    int rc = setup(p, x, ldx, w_packed, M, N, K, false, workspace, workspace_bytes, "md_linear_block_xielu");
+    if (rc != MD_OK) return rc;
+    p.out = (bf16_t*)out;
+    p.ldo = ldo;
+    p.act = act;
+    hipStream_t st = (hipStream_t)stream;
+    rc = launch_epi<BE_XIELU>(p, (N / BN) * p.S, st);
+    if (rc == MD_OK && p.S > 1) rc = md_internal_launch_skinny_reduce(p.partial, p.S, M, N, BE_XIELU, act, out, ldo, st);
+    if (rc != MD_OK) return rc;
+    MD_CHECK_LAUNCH("md_linear_block_xielu");
+    return MD_OK;
+}
+
+// md_linear_planes (residual.hip): the partial planes without a combine launch
+int md_internal_planes_block_count(int M, int N, int K) { return shape_ok(M, N, K) ? pick_splits(N / BN, K / BK) : 0; }
+int md_internal_planes_block(const void* x, int64_t ldx, const void* w, int M, int N, int K, void* ws, size_t ws_bytes, int* S,
+                             hipStream_t st) {
+    BlockParams p;
+    const int rc = setup(p, x, ldx, w, M, N, K, true, ws, ws_bytes, "md_linear_planes");
+    if (rc != MD_OK) return rc;
+    *S = p.S;
+    return launch_epi<BE_NONE>(p, (N / BN) * p.S, st);
 }
 
 extern "C" int md_linear_block_add_rmsnorm(const void* x, int64_t ldx, const void* w_packed, const void* bias,

@@ -163,14 +163,10 @@ __global__ __launch_bounds__(256) void silu_mul_kernel(const bf16_t* __restrict_
     }
 }
 
-// xIELU: a quadratic with slope 1/2 at 0 on the right, an exponential one on the left; the coefficients are softplus of two
-// learned numbers.  fp32 inside, one rounding; expm1 keeps e^z - 1 - z accurate near 0
-__device__ __forceinline__ float softplus_f(float x) { return log1pf(expf(-fabsf(x))) + fmaxf(x, 0.f); }
-
 template <typename T, int VEC>
 __global__ __launch_bounds__(256) void xielu_kernel(const T* __restrict__ z, int64_t zs, const float* __restrict__ act, T* y,
                                                     int rows, int dim) {
-    const float ap = softplus_f(act[0]), an = 0.5f + softplus_f(act[1]);
+    const Xielu f_act(act);
     const int nvec = dim / VEC;
     const int64_t total = (int64_t)rows * nvec;
     typedef T vec __attribute__((ext_vector_type(VEC)));
@@ -186,10 +182,7 @@ __global__ __launch_bounds__(256) void xielu_kernel(const T* __restrict__ z, int
             for (int e = 0; e < VEC; ++e) f[e] = (float)v[e];
         }
 #pragma unroll
-        for (int e = 0; e < VEC; ++e) {
-            const float x = f[e];
-            f[e] = (x > 0.f ? ap * x * x : an * (expm1f(fminf(x, 0.f)) - x)) + 0.5f * x;
-        }
+        for (int e = 0; e < VEC; ++e) f[e] = f_act(f[e]);
         if constexpr (VEC == 1) {
             y[row * dim + c] = (T)f[0];
         } else {

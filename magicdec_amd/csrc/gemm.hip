@@ -36,7 +36,7 @@ constexpr int kSlabK = 128;                 // k depth of one LDS activation sla
 constexpr int kStepsPerSlab = kSlabK / 16;  // 8 MFMA k-steps (32x32x16) per slab
 constexpr int kPitch = kSlabK * 2 + 16;     // LDS row pitch in bytes (272: rows start 4 banks apart)
 
-enum { EPI_NONE = 0, EPI_SWIGLU = 1 };
+enum { EPI_NONE = 0, EPI_SWIGLU = 1, EPI_XIELU = 2 };
 
 struct GemmParams {
     const bf16_t* x;      // [M][K], row stride ldx (elements)
@@ -54,6 +54,7 @@ struct GemmParams {
     const bf16_t* pro_w;  // RMSNorm weight [K]
     float pro_eps;
     int pro_tiles;
+    const float* act;     // EPI_XIELU: the two numbers of the activation
 };
 
 __device__ __forceinline__ f32x2 unpack2(unsigned int v) {          // the two bf16 of a dword as fp32 (low half first)
@@ -337,6 +338,8 @@ __global__ __launch_bounds__(64 * NW) void skinny_gemm_kernel(const GemmParams p
                 if (W8) h = bf16_to_f32(f32_to_bf16(h * bf16_to_f32(p.scales[col])));
                 const float h3 = __shfl_xor(h, 16);                 // lanes j and j^16 hold w1 / w3 of one column
                 v = silu_bf16(h) * h3;
+            } else if constexpr (EPI == EPI_XIELU) {
+                v = Xielu(p.act)(v);
             } else {
                 v += bias;
                 if (W8) v = bf16_to_f32(f32_to_bf16(v)) * scale;
@@ -386,6 +389,8 @@ __global__ __launch_bounds__(256) void skinny_reduce_kernel(const GemmParams p) 
                 h3 = bf16_to_f32(f32_to_bf16(h3 * bf16_to_f32(p.scales[(p.N >> 1) + c0 + e])));
             }
             v = silu_bf16(h1) * h3;
+        } else if constexpr (EPI == EPI_XIELU) {
+            v = Xielu(p.act)(v);
         } else {
             if (p.bias) v += bf16_to_f32(p.bias[c0 + e]);
             if (W8) v = bf16_to_f32(f32_to_bf16(v)) * bf16_to_f32(p.scales[c0 + e]);
@@ -525,6 +530,7 @@ int wave_tiles(int N, int epilogue) { return epilogue == EPI_SWIGLU ? ((N >> 1) 
 }  // namespace
 
 // blockgemm.hip: the fixed-order combine of fp32 partial slabs [S][M][N] (+ bias / SwiGLU) for md_linear_block
+// (epilogue EPI_XIELU: `bias` is the activation's two fp32 numbers)
 int md_internal_launch_skinny_reduce(const float* partial, int S, int M, int N, int epilogue, const void* bias, void* out,
                                      int64_t ldo, hipStream_t st) {
     GemmParams p = {};
@@ -533,13 +539,16 @@ int md_internal_launch_skinny_reduce(const float* partial, int S, int M, int N, 
     p.M = M;
     p.N = N;
     p.Nout = epilogue == EPI_SWIGLU ? N / 2 : N;
-    p.bias = (const bf16_t*)bias;
+    p.bias = epilogue == EPI_XIELU ? nullptr : (const bf16_t*)bias;
+    p.act = epilogue == EPI_XIELU ? (const float*)bias : nullptr;
     p.out = (bf16_t*)out;
     p.ldo = ldo;
     const int64_t threads = (int64_t)M * (p.Nout / 4);
     const dim3 grid((unsigned)((threads + 255) / 256));
     if (epilogue == EPI_SWIGLU)
         hipLaunchKernelGGL((skinny_reduce_kernel<EPI_SWIGLU, false>), grid, dim3(256), 0, st, p);
+    else if (epilogue == EPI_XIELU)
+        hipLaunchKernelGGL((skinny_reduce_kernel<EPI_XIELU, false>), grid, dim3(256), 0, st, p);
     else
         hipLaunchKernelGGL((skinny_reduce_kernel<EPI_NONE, false>), grid, dim3(256), 0, st, p);
     return MD_OK;
@@ -567,11 +576,13 @@ namespace {
 int linear_impl(const void* x, int64_t ldx, const void* w, int w_dtype, int w_packed, const void* scales,
                 const void* bias, void* out, int64_t ldo, int M, int N, int K, int epilogue, void* workspace,
                 size_t workspace_bytes, md_stream_t stream, const float* pro_ssq, int pro_tiles, const void* pro_w,
-                float pro_eps) {
+                float pro_eps, const float* act = nullptr) {
     MD_CHECK_ARG(x && w && out, "md_linear: null pointer argument");
     MD_CHECK_ARG(md_linear_supported(M, N, K, epilogue), "md_linear: unsupported shape M=%d N=%d K=%d epilogue=%d "
                  "(need 1 <= M <= 256, K %% 128 == 0, N %% 4 == 0)", M, N, K, epilogue);
-    MD_CHECK_ARG(epilogue == EPI_NONE || epilogue == EPI_SWIGLU, "md_linear: unknown epilogue %d", epilogue);
+    MD_CHECK_ARG(epilogue == EPI_NONE || epilogue == EPI_SWIGLU || (epilogue == EPI_XIELU && act && !pro_ssq &&
+                                                                          w_dtype == MD_W_BF16 && !bias),
+                 "md_linear: unknown epilogue %d", epilogue);
     MD_CHECK_ARG(w_dtype == MD_W_BF16 || (w_dtype == MD_W_INT8 && scales), "md_linear: w_dtype must be MD_W_BF16 or "
                  "MD_W_INT8 (with per-channel scales)");
     MD_CHECK_ARG(!(epilogue == EPI_SWIGLU && bias), "md_linear: SwiGLU epilogue takes no bias");
@@ -591,6 +602,7 @@ int linear_impl(const void* x, int64_t ldx, const void* w, int w_dtype, int w_pa
     p.Nout = epilogue == EPI_SWIGLU ? N / 2 : N;
     p.packed = w_packed ? 1 : 0;
     p.skip_reduce = 0;
+    p.act = act;
     const bool pro = pro_ssq != nullptr;
     if (pro) {
         MD_CHECK_ARG(w_dtype == MD_W_BF16, "md_linear_normed: bf16 weights only");
@@ -619,6 +631,8 @@ int linear_impl(const void* x, int64_t ldx, const void* w, int w_dtype, int w_pa
     if (pro)
         rc = epilogue == EPI_SWIGLU ? launch_mt<EPI_SWIGLU, false, true>(p, pl.nw, n_blocks, st)
                                     : launch_mt<EPI_NONE, false, true>(p, pl.nw, n_blocks, st);
+    else if (epilogue == EPI_XIELU)
+        rc = launch_mt<EPI_XIELU, false>(p, pl.nw, n_blocks, st);
     else if (epilogue == EPI_SWIGLU)
         rc = w8 ? launch_mt<EPI_SWIGLU, true>(p, pl.nw, n_blocks, st) : launch_mt<EPI_SWIGLU, false>(p, pl.nw, n_blocks, st);
     else
@@ -634,6 +648,42 @@ extern "C" int md_linear(const void* x, int64_t ldx, const void* w, int w_dtype,
                          size_t workspace_bytes, md_stream_t stream) {
     return linear_impl(x, ldx, w, w_dtype, w_packed, scales, bias, out, ldo, M, N, K, epilogue, workspace, workspace_bytes,
                        stream, nullptr, 0, nullptr, 0.f);
+}
+
+extern "C" int md_linear_xielu(const void* x, int64_t ldx, const void* w, int w_packed, const float* act, void* out, int64_t ldo,
+                               int M, int N, int K, void* workspace, size_t workspace_bytes, md_stream_t stream) {
+    MD_CHECK_ARG(act, "md_linear_xielu: null pointer argument");
+    return linear_impl(x, ldx, w, MD_W_BF16, w_packed, nullptr, nullptr, out, ldo, M, N, K, EPI_XIELU, workspace,
+                       workspace_bytes, stream, nullptr, 0, nullptr, 0.f, act);
+}
+
+// md_linear_planes (residual.hip): the split-K partial planes without a combine launch; a product with one K slice has none
+int md_internal_planes_skinny_count(int M, int N, int K) {
+    if (!md_linear_supported(M, N, K, EPI_NONE)) return 0;
+    const int S = plan_of(wave_tiles(N, EPI_NONE), K, false).S;
+    return S > 1 ? S : 0;
+}
+int md_internal_planes_skinny(const void* x, int64_t ldx, const void* w, int M, int N, int K, void* ws, size_t ws_bytes, int* S,
+                              hipStream_t st) {
+    MD_CHECK_ARG(md_internal_planes_skinny_count(M, N, K), "md_linear_planes: unsupported shape M=%d N=%d K=%d", M, N, K);
+    MD_CHECK_ARG((((uintptr_t)x | (uintptr_t)w) & 15) == 0 && ldx % 8 == 0, "md_linear_planes: x / w must be 16-byte aligned");
+    GemmParams p = {};
+    p.x = (const bf16_t*)x;
+    p.w = w;
+    p.ldx = ldx;
+    p.M = M;
+    p.N = p.Nout = N;
+    p.K = K;
+    p.ldo = N;
+    p.packed = 1;
+    p.skip_reduce = 1;
+    const int ntiles = wave_tiles(N, EPI_NONE);
+    const SkinnyPlan pl = plan_of(ntiles, K, nw_allowed(M, false));
+    p.S = *S = pl.S;
+    p.kblk = K / p.S;
+    p.partial = (float*)ws;
+    MD_CHECK_ARG(ws && ws_bytes >= (size_t)p.S * M * N * 4 && ((uintptr_t)ws & 15) == 0, "md_linear_planes: workspace too small");
+    return launch_mt<EPI_NONE, false>(p, pl.nw, (ntiles + pl.nw - 1) / pl.nw, st);
 }
 
 extern "C" int md_linear_normed(const void* h, int64_t ldh, const float* ssq, int ssq_tiles, const void* norm_weight,

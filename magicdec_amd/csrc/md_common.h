@@ -66,6 +66,20 @@ __device__ __forceinline__ float bf16_bits_to_f32(unsigned short b) {
 __device__ __forceinline__ bf16_t f32_to_bf16(float x) { return (bf16_t)x; }
 __device__ __forceinline__ float bf16_to_f32(bf16_t x) { return (float)x; }
 
+// xIELU: a quadratic with slope 1/2 at 0 on the right, an exponential one on the left; the coefficients are softplus of two
+// learned numbers.  fp32; expm1 keeps e^z - 1 - z accurate near 0
+struct Xielu {
+    float ap, an;
+    __device__ __forceinline__ explicit Xielu(const float* act) {
+        const float a = act[0], b = act[1];
+        ap = log1pf(expf(-fabsf(a))) + fmaxf(a, 0.f);
+        an = 0.5f + log1pf(expf(-fabsf(b))) + fmaxf(b, 0.f);
+    }
+    __device__ __forceinline__ float operator()(float z) const {
+        return (z > 0.f ? ap * z * z : an * (expm1f(fminf(z, 0.f)) - z)) + 0.5f * z;
+    }
+};
+
 __device__ __forceinline__ float wave_reduce_sum(float v) {
 #pragma unroll
     for (int o = 32; o > 0; o >>= 1) v += __shfl_xor(v, o);

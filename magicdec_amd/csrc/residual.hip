@@ -311,6 +311,36 @@ bool resid_vec(const md_resid_norm_args* a) {
 
 }  // namespace
 
+// the split-K GEMMs (gemm.hip, tilegemm.hip, blockgemm.hip) up to their partial planes
+#define MD_PLANES_DECL(kind)                                                                                              \
+    int md_internal_planes_##kind##_count(int M, int N, int K);                                                            \
+    int md_internal_planes_##kind(const void* x, int64_t ldx, const void* w, int M, int N, int K, void* ws, size_t ws_bytes, \
+                                  int* S, hipStream_t st);
+MD_PLANES_DECL(skinny)
+MD_PLANES_DECL(tile)
+MD_PLANES_DECL(block)
+#undef MD_PLANES_DECL
+
+extern "C" int md_linear_planes_count(int kind, int M, int N, int K) {
+    return kind == MD_PLANES_SKINNY ? md_internal_planes_skinny_count(M, N, K)
+         : kind == MD_PLANES_TILE   ? md_internal_planes_tile_count(M, N, K)
+         : kind == MD_PLANES_BLOCK  ? md_internal_planes_block_count(M, N, K) : 0;
+}
+
+extern "C" int md_linear_planes(int kind, const void* x, int64_t ldx, const void* w_packed, int M, int N, int K, float* planes,
+                                size_t planes_bytes, md_stream_t stream) {
+    MD_CHECK_ARG(md_linear_planes_count(kind, M, N, K) > 0, "md_linear_planes: unsupported shape kind=%d M=%d N=%d K=%d", kind, M,
+                 N, K);
+    int S = 0, rc;
+    hipStream_t st = (hipStream_t)stream;
+    if (kind == MD_PLANES_SKINNY) rc = md_internal_planes_skinny(x, ldx, w_packed, M, N, K, planes, planes_bytes, &S, st);
+    else if (kind == MD_PLANES_TILE) rc = md_internal_planes_tile(x, ldx, w_packed, M, N, K, planes, planes_bytes, &S, st);
+    else rc = md_internal_planes_block(x, ldx, w_packed, M, N, K, planes, planes_bytes, &S, st);
+    if (rc != MD_OK) return rc;
+    MD_CHECK_LAUNCH("md_linear_planes");
+    return MD_OK;
+}
+
 extern "C" int md_embed_pos(const int64_t* tokens, const void* table, const void* pos_table, int dtype,
                             const int32_t* qo_indptr, const int32_t* pos0, int B, int n_max, int width, int vocab, int max_pos,
                             float scale, float* out, md_stream_t stream) {

@@ -61,7 +61,8 @@ constexpr int kPitch = kKC * 2 + 16;     // LDS row pitch (272 B: consecutive ro
 constexpr int kWaveLds = 32 * kPitch;    // wave-private activation image (8704 B >= the 4 KiB partial tile)
 
 enum { FL_NONE = 0, FL_SWIGLU = 1, FL_RESID = 2, FL_ROPE_APPEND = 3,
-       FL_PARTIAL = 4 };      // internal: the K range is ALSO split over workgroups; fp32 partial tiles -> workspace
+       FL_XIELU = 4,
+       FL_PARTIAL = 5 };      // internal: the K range is ALSO split over workgroups; fp32 partial tiles -> workspace
 
 struct KvTable {
     void* cache;
@@ -85,6 +86,7 @@ struct TileParams {
     KvTable t1, t2;
     const float* k_scale;
     const float* v_scale;
+    const float* act;         // XIELU: the two numbers of the activation
     unsigned int* overflow;   // dropped-row counter (md_page_overflow_count)
     // deferred RMSNorm (see the kernel header): producer side (RESID) / consumer side (PRO)
     float* ssq_out;           // RESID: [M][n_tiles] sum of squares of the tile's 32 output columns per row, or null
@@ -494,6 +496,11 @@ __global__ __launch_bounds__(64 * NW, MT * NT > 1 ? 2 : 4) void tile_gemm_kernel
                 s[1] += bf16_to_f32(p.bias[n + 1]);
             }
             if (gm >= p.M) continue;
+            if constexpr (EPI == FL_XIELU) {                  // fp32 accumulator -> activation -> one rounding
+                const Xielu f_act(p.act);
+                *reinterpret_cast<unsigned int*>(p.out + (int64_t)gm * p.ldo + n) = pack2(f_act(s[0]), f_act(s[1]));
+                continue;
+            }
             // the linear's own output, rounded to bf16 as nn.Linear returns it
             const float o0 = bf16_to_f32(f32_to_bf16(s[0])), o1 = bf16_to_f32(f32_to_bf16(s[1]));
             if constexpr (EPI == FL_NONE) {
@@ -594,7 +601,7 @@ int launch_tile_pro(const TileParams& p, hipStream_t st) {
     // chunk, and measured 25.9 us in the cfg3 iteration against 24.5 for the 1 x 1 form -- profiles/r04_bench_cfg3_iter_breakdown.csv)
     // round 6: also WITH the deferred-RMSNorm prologue (SwiGLU consumer), now that that instantiation has a four-deep W
     // ring, no spills, and its own prologue (kNewPro in the kernel)
-    if constexpr ((EPI == FL_SWIGLU || EPI == FL_NONE || EPI == FL_RESID) && (!PRO || EPI == FL_SWIGLU)) {
+    if constexpr ((EPI == FL_SWIGLU || EPI == FL_NONE || EPI == FL_RESID || EPI == FL_XIELU) && (!PRO || EPI == FL_SWIGLU)) {
         const int groups = (p.n_tiles / 2) * ((p.m_tiles + 1) / 2);
         bool t22 = p.m_tiles >= 2 && p.n_tiles % 2 == 0 && p.K % 128 == 0 && groups >= 192;
         if (g_force_tile == 11) t22 = false;
@@ -720,6 +727,16 @@ int md_internal_launch_reduce_add_rmsnorm(const float* partial, int S, int M, in
                                           const void* x, int64_t ldx, const void* w, void* h_out, void* y, float eps,
                                           hipStream_t st);
 
+// md_linear_planes (residual.hip): the fp32 planes without a combine launch
+int md_internal_planes_tile(const void* x, int64_t ldx, const void* w, int M, int N, int K, void* ws, size_t ws_bytes, int* S,
+                            hipStream_t st) {
+    const int rc = split_check("md_linear_planes", x, ldx, w, M, N, K, ws, ws_bytes);
+    return rc != MD_OK ? rc : split_main(x, ldx, w, M, N, K, ws, st, S);
+}
+int md_internal_planes_tile_count(int M, int N, int K) {
+    return (M < 1 || M > 256 || K < 128 || K % 128 || N < 32 || N % 32) ? 0 : split_plan(M, N, K).S;
+}
+
 #ifdef MD_DEV_KNOBS
 extern "C" void md_debug_set_fused_split(int S) { g_force_split = S > 0 ? S : 0; }
 extern "C" void md_debug_set_tile_timing(void* buf) { g_tile_dbg = (unsigned long long*)buf; }
@@ -777,7 +794,7 @@ extern "C" void md_debug_set_fused_nw(int nw) {
 
 extern "C" int md_linear_fused_supported(int M, int N, int K, int epilogue) {
     if (M < 1 || M > 256 || K < 128 || K % 128 || N < 32 || N % 32) return 0;
-    return (epilogue >= FL_NONE && epilogue <= FL_ROPE_APPEND) ? 1 : 0;
+    return (epilogue >= FL_NONE && epilogue <= FL_XIELU) ? 1 : 0;
 }
 
 extern "C" int md_linear_fused(const md_fused_linear_args* a, md_stream_t stream) {
@@ -827,6 +844,11 @@ extern "C" int md_linear_fused(const md_fused_linear_args* a, md_stream_t stream
         break;
     case FL_SWIGLU:
         rc = launch_tile<FL_SWIGLU, false>(p, st);
+        break;
+    case FL_XIELU:
+        MD_CHECK_ARG(a->act && !a->bias, "md_linear_fused: the xIELU epilogue needs `act` and takes no bias");
+        p.act = a->act;
+        rc = launch_tile<FL_XIELU, false>(p, st);
         break;
     case FL_RESID:
         MD_CHECK_ARG(a->resid && ((uintptr_t)a->resid & 3) == 0 && a->ldr % 2 == 0,

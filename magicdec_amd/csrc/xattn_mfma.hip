@@ -44,15 +44,26 @@ constexpr int decode_wave_lds() {
     return ((stage > merge ? stage : merge) + 255) / 256 * 256;
 }
 
+// 16-byte loads in flight per wavefront: two tiles where the register budget allows it (256 registers at two workgroups per
+// CU, 512 where the LDS images leave room for one anyway), else one
+template <int DV, int QT>
+constexpr int decode_wgs() { return 4 * decode_wave_lds<DV, QT>() > 80 * 1024 ? 1 : 2; }
+template <int DV, int QT>
+constexpr int decode_tiles_in_flight() {
+    const int regs = 2 * (DK + DV) / 4 + QT * (DV / 4 + DK / 8);
+    return regs <= (decode_wgs<DV, QT>() == 1 ? 400 : 176) ? 2 : 1;
+}
+
 // Four wavefronts share one (request, kv head, kv split); each owns a stream of 32-key tiles (two in flight in registers),
 // no barrier in the loop.  S^T = K Q^T and O^T = V^T P^T on 16x16x32; the S accumulator is the PV operand.
 // FUSED: q holds the RAW projection rows (q | k | v of the step's tokens): the q heads are normalised in registers, and the
 // wavefront that owns the tile a new key falls into normalises it, puts it into its LDS image and appends it to the pages.
 template <int DV, int QT, bool FUSED>
-__global__ __launch_bounds__(256, 2) void xattn_decode_kernel(const XattnParams p) {
+__global__ __launch_bounds__(256, (decode_wgs<DV, QT>())) void xattn_decode_kernel(const XattnParams p) {
     constexpr int KS = DK / 32, NB = DV / 16;
     constexpr int NK = DK / 16, NV = DV / 16;          // 16-byte pieces per lane of a 32-key K / V tile
     constexpr int WAVE_LDS = decode_wave_lds<DV, QT>();
+    constexpr int NS = decode_tiles_in_flight<DV, QT>(), PF = 4 * NS;      // prefetch distance in tiles
     extern __shared__ __attribute__((aligned(16))) unsigned char smem[];
     const int tid = threadIdx.x, lane = tid & 63, lq = lane & 15, lc = lane >> 4;
     const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
@@ -162,9 +173,9 @@ __global__ __launch_bounds__(256, 2) void xattn_decode_kernel(const XattnParams 
             *reinterpret_cast<u32x4*>(ldsV + v_addr(row, c % (DV / 8))) = vr[i];
         }
         if constexpr (decltype(steady)::value) {
-            issue(t + 8, kr, vr);
+            issue(t + PF, kr, vr);
         } else {
-            if (t + 8 < t_end) issue(t + 8, kr, vr);
+            if (t + PF < t_end) issue(t + PF, kr, vr);
         }
         if constexpr (FUSED) {
             if (tail >= pos_b) {                    // wave-uniform: this tile takes (some of) the step's own keys
@@ -241,7 +252,13 @@ __global__ __launch_bounds__(256, 2) void xattn_decode_kernel(const XattnParams 
         __builtin_amdgcn_wave_barrier();
     };
 
-    {
+    if constexpr (NS == 1) {
+        u32x4 ka[NK], va[NV];
+        int t = t_begin + wave;
+        if (t < t_end) issue(t, ka, va);
+        for (; t + 4 < t_end; t += 4) process(std::true_type{}, t, ka, va);
+        if (t < t_end) process(std::false_type{}, t, ka, va);
+    } else {
         u32x4 ka[NK], va[NV], kb[NK], vb[NV];
         int t = t_begin + wave;
         if (t < t_end) issue(t, ka, va);

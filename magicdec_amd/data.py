@@ -98,5 +98,6 @@ def convert_pg19_dataset(tokenizer=None, seq_len=4096, vocab_size=128256, num_se
     n = num_sequences if num_sequences is not None else 640
     g = torch.Generator().manual_seed(seed)
     ids = torch.randint(0, vocab_size, (n, seq_len), generator=g)
-    ids[:, 0] = getattr(tokenizer, "bos_token_id", None) or 1
+    bos = getattr(tokenizer, "bos_token_id", None) or 1
+    ids[:, 0] = bos if bos < vocab_size else min(1, vocab_size - 1)       # (the stand-in tokenizer's ids are Llama-3's)
     return TensorDataset(ids)

@@ -262,6 +262,7 @@ def run_longspec_batch(engine, draft, input_ids, gamma, max_len, eot_1, eot_2, f
                        trace_fn=None, bcast=None, barrier=None, timers: PhaseTimers = None):
     """A whole batch: prefill both models, loop until termination.  Returns (state, seconds in the loop)."""
     B, S = input_ids.shape
+    _check_rollback(gamma, engine, draft)
     st = new_state(B, gamma, max_len + 1, input_ids.device, input_ids)
     st.tokens_buffer[:, :1] = engine.encode(input_ids=input_ids)[:, -1:]
     if draft is not None:
@@ -305,6 +306,56 @@ def run_selfspec_batch(engine, input_ids, gamma, max_len, eot_1, eot_2, streamin
         warn_on_page_overflow("selfspec batch")
         check_collectives(engine)
     return st, dt
+
+
+def run_sequences(engine, prompts, max_new_tokens, eot=(), on_token=None):
+    """Greedy generation for prompts of unequal lengths with continuous batching: a prompt is admitted as soon as the engine's
+    pool (SequencePool) has a slot, and pages for it and everything it may generate, beside what the live sequences may still
+    need; a sequence that has ended gives both back.  Prompts admitted together are prefilled as one ragged step, live
+    sequences decode as one.  Returns (generated token lists, decode steps, seconds)."""
+    pool = engine.pool
+    total = [len(p) + max_new_tokens for p in prompts]
+    for n in total:
+        if pool.pages_for(n) > len(pool.free_pages) + sum(len(e[1]) for e in pool.seqs.values()):
+            raise ValueError(f"a sequence of {n} tokens does not fit the engine's pages")
+    out = [[] for _ in prompts]
+    waiting, live = list(range(len(prompts))), []
+    sid = lambda i: ("seq", i)                                      # noqa: E731
+    steps, t0 = 0, time.perf_counter()
+
+    def take(ids, tokens):
+        for i, t in zip(ids, tokens.tolist()):
+            out[i].append(t)
+            if on_token is not None:
+                on_token(i, t)
+            if t in eot or len(out[i]) == max_new_tokens:
+                engine.end(sid(i))
+                live.remove(i)
+    while waiting or live:
+        admit = []
+        owed = sum(pool.pages_for(total[i]) - len(pool.seqs[sid(i)][1]) for i in live)
+        while waiting and len(admit) < len(pool.free_slots):
+            need = pool.pages_for(total[waiting[0]])
+            if owed + need > len(pool.free_pages):
+                break
+            owed += need
+            admit.append(waiting.pop(0))
+        if admit:
+            live += admit
+            take(admit, engine.step([(sid(i), prompts[i]) for i in admit])[0])
+        elif live:
+            now = list(live)
+            steps += 1
+            take(now, engine.step([(sid(i), [out[i][-1]]) for i in now])[0])
+    return out, steps, time.perf_counter() - t0
+
+
+def _check_rollback(gamma, *engines):
+    """Models with per-sequence state take back a bounded number of tokens (Transformer.rollback_depth)."""
+    for e in engines:
+        depth = getattr(getattr(e, "model", None), "rollback_depth", lambda: None)() if e is not None else None
+        if depth is not None and gamma > depth:
+            raise ValueError(f"gamma={gamma}: the model can take back at most {depth} tokens")
 
 
 def run_baseline_batch(engine, input_ids, max_len, eot_1, eot_2, check_eot_every=1):

@@ -316,14 +316,21 @@ class PackedWeight:
         return out
 
 
+def _act_numbers(act):
+    if act.dtype != torch.float32 or act.numel() != 2 or not act.is_cuda or not act.is_contiguous():
+        raise ValueError("xielu: float32 act[2] on the GPU expected")
+    return _p(act)
+
+
 def linear(x, weight, bias=None, scales=None, swiglu=False, workspace: "AttnWorkspace" = None, out=None,
-           pro: "DeferredNorm" = None):
+           pro: "DeferredNorm" = None, xielu=None):
     """F.linear(x, weight, bias) for M = x.shape[0] <= 256 rows on the hand-written gfx950 skinny GEMM (md_linear).
     x [M, K] bf16 with unit inner stride (row stride free); weight: a contiguous [N, K] tensor or a PackedWeight
     (streaming layout), bf16 -- or int8 with bf16 per-row `scales` (WeightOnlyInt8Linear semantics:
     bf16(x.w^T) * scales).  swiglu=True: weight = [w1; w3] (N = 2*I rows) and the result is
     silu(x.w1^T) * (x.w3^T) [M, I] with the reference's bf16 rounding points.
-    pro (bf16 weights): x is pro.h, the un-normalised hidden state, and is normalised on the fly (md_linear_normed)."""
+    pro (bf16 weights): x is pro.h, the un-normalised hidden state, and is normalised on the fly (md_linear_normed).
+    xielu (bf16 weights): the two numbers of the activation applied to the result (md_linear_xielu)."""
     packed = isinstance(weight, PackedWeight)
     wt = weight.data if packed else weight
     _gpu(x, wt, bias, scales)
@@ -361,6 +368,12 @@ def linear(x, weight, bias=None, scales=None, swiglu=False, workspace: "AttnWork
         ws = workspace.get(nbytes + 256)
         off = (-ws.data_ptr()) % 256
     wsp = ctypes.c_void_p(ws.data_ptr() + off) if ws is not None else None
+    if xielu is not None:
+        if wd != MD_W_BF16 or swiglu or pro is not None or bias is not None:
+            raise ValueError("linear: the xIELU epilogue takes bf16 weights and nothing beside it")
+        check(lib.md_linear_xielu(_p(x), x.stride(0), _p(wt), 1 if packed else 0, _act_numbers(xielu), _p(out), out.stride(0),
+                                  M, N, K, wsp, nbytes, _stream()), "md_linear_xielu")
+        return out
     if pro is not None:
         if wd != MD_W_BF16:
             raise TypeError("linear: the deferred norm needs bf16 weights")
@@ -504,7 +517,8 @@ def _block_bias(bias, N):
         raise ValueError(f"linear_block: bias must be a contiguous, 16-byte aligned bf16 vector of {N} elements")
 
 
-def linear_block(x, weight: "PackedWeight", bias=None, swiglu=False, workspace: "AttnWorkspace" = None, out=None):
+def linear_block(x, weight: "PackedWeight", bias=None, swiglu=False, workspace: "AttnWorkspace" = None, out=None,
+                 xielu=None):
     """F.linear(x, W, bias) (or silu(x.w1^T) * (x.w3^T) for swiglu=True, weight = [w1; w3]) for 129..256 rows on the
     block-tile GEMM md_linear_block; same contract and rounding points as linear()."""
     M, N, K = _block_args(x, weight, swiglu)
@@ -518,6 +532,12 @@ def linear_block(x, weight: "PackedWeight", bias=None, swiglu=False, workspace: 
             raise ValueError("linear_block: out must be bf16 [M, N_out] with unit inner stride")
     lib = _lib.load()
     wsp, nbytes = _block_ws(lib, M, N, K, False, workspace)
+    if xielu is not None:
+        if swiglu or bias is not None:
+            raise ValueError("linear_block: the xIELU epilogue takes nothing beside it")
+        check(lib.md_linear_block_xielu(_p(x), x.stride(0), _p(weight.data), _act_numbers(xielu), _p(out), out.stride(0), M, N,
+                                        K, wsp, nbytes, _stream()), "md_linear_block_xielu")
+        return out
     check(lib.md_linear_block(_p(x), x.stride(0), _p(weight.data), _p(bias), _p(out), out.stride(0), M, N, K,
                               EPI_SWIGLU if swiglu else EPI_NONE, wsp, nbytes, _stream()), "md_linear_block")
     return out
@@ -543,7 +563,7 @@ def linear_block_add_rmsnorm(x, weight: "PackedWeight", resid, norm_weight, eps,
 
 
 # ----------------------------------------------------------------------------- K8b
-FL_NONE, FL_SWIGLU, FL_RESID, FL_ROPE_APPEND = 0, 1, 2, 3
+FL_NONE, FL_SWIGLU, FL_RESID, FL_ROPE_APPEND, FL_XIELU = 0, 1, 2, 3, 4
 
 
 def fused_linear_supported(M, N, K, epilogue=FL_NONE):
@@ -596,13 +616,17 @@ def _set_pro(a, x, pro: "DeferredNorm"):
 
 
 def fused_linear(x, weight: "PackedWeight", bias=None, swiglu=False, resid=None, out=None, want_ssq=False,
-                 pro: "DeferredNorm" = None):
+                 pro: "DeferredNorm" = None, xielu=None):
     """One launch (md_linear_fused): F.linear(x, W, bias) for M <= 256 rows over a PackedWeight, optionally followed by
     SiLU(h1) * h3 (swiglu=True, weight = [w1; w3]) or by the bf16 residual add `resid + linear` (resid [M, N]).
     want_ssq (with resid): also return the per-row partial sums of squares [M, N/32] of the result (the producer half of
     a deferred RMSNorm).  pro (with swiglu): x is pro.h and is normalised on the fly (the consumer half)."""
-    epi = FL_SWIGLU if swiglu else (FL_RESID if resid is not None else FL_NONE)
+    epi = FL_SWIGLU if swiglu else (FL_RESID if resid is not None else (FL_XIELU if xielu is not None else FL_NONE))
+    if xielu is not None and epi != FL_XIELU:
+        raise ValueError("fused linear: the xIELU epilogue takes nothing beside it")
     a = _fused_args(x, weight, bias, epi)
+    if xielu is not None:
+        a.act = _act_numbers(xielu).value
     n_out = weight.N // 2 if swiglu else weight.N
     if out is None:
         out = torch.empty((x.shape[0], n_out), dtype=x.dtype, device=x.device)
@@ -757,10 +781,42 @@ def embed_pos(tokens, table, pos_table, rows: StepRows, scale=1.0):
 
 
 class Planes:
-    """A projection as n fp32 partial planes [n, rows, width] in a workspace (a split-K product before its combine)."""
+    """A projection as n fp32 partial planes [n, rows, width] in a workspace (a split-K product before its combine); valid
+    until the next user of the workspace."""
 
-    def __init__(self, ptr, n, rows, width):
-        self.ptr, self.n, self.shape = ptr, n, (rows, width)
+    def __init__(self, planes):
+        self.planes, self.n, self.shape = planes, planes.shape[0], tuple(planes.shape[1:])
+
+    def sum(self):
+        return self.planes.sum(0)
+
+
+PLANES_KINDS = {"skinny": 0, "tile": 1, "block": 2}
+
+
+def linear_planes_count(kind, M, N, K):
+    """Partial planes of this product on the split-K GEMM `kind` (0: unsupported)."""
+    return int(_lib.load().md_linear_planes_count(PLANES_KINDS[kind], int(M), int(N), int(K)))
+
+
+def linear_planes(x, weight: "PackedWeight", kind, workspace: AttnWorkspace):
+    """x . W^T as `Planes` in the workspace: one launch; resid_norm is the combine."""
+    _gpu(x, weight.data)
+    if x.dim() != 2 or x.stride(1) != 1 or x.dtype != torch.bfloat16 or weight.swiglu or weight.dtype != torch.bfloat16:
+        raise ValueError("linear_planes expects bf16 x [M, K] with unit inner stride and a plain bf16 packed weight")
+    M, K = x.shape
+    if weight.K != K:
+        raise ValueError(f"linear_planes: x has K={K}, weight has K={weight.K}")
+    n = linear_planes_count(kind, M, weight.N, K)
+    if n == 0:
+        raise ValueError(f"linear_planes: {kind} does not take M={M} N={weight.N} K={K}")
+    nbytes = n * M * weight.N * 4
+    ws = workspace.get(nbytes + 256)
+    off = (-ws.data_ptr()) % 256
+    planes = ws[off:off + nbytes].view(torch.float32).view(n, M, weight.N)
+    check(_lib.load().md_linear_planes(PLANES_KINDS[kind], _p(x), x.stride(0), _p(weight.data), M, weight.N, K, _p(planes),
+                                       nbytes, _stream()), "md_linear_planes")
+    return Planes(planes)
 
 
 def resid_norm(x, delta, weight, eps, out_scale=1.0, shift=None, ring=None, rows: StepRows = None):
@@ -782,7 +838,7 @@ def resid_norm(x, delta, weight, eps, out_scale=1.0, shift=None, ring=None, rows
         x_out = torch.empty_like(x)
         a.x_out = x_out.data_ptr()
         if isinstance(delta, Planes):
-            a.planes, a.n_planes = delta.ptr, delta.n
+            a.planes, a.n_planes = delta.planes.data_ptr(), delta.n
         else:
             _gpu(delta)
             _dense(delta)

@@ -113,12 +113,17 @@ def test_every_entry_point_rejects_null_arguments():
     fa.M, fa.N, fa.K = 64, 100, 256
     assert lib.md_linear_fused(ctypes.byref(fa), None) < 0 and "unsupported shape" in lib.md_last_error_string().decode()
     skip.add("md_linear_fused")
+    # size and shape queries of the extended attention and the planes
+    assert lib.md_xattn_head_pad(0) == 0 and lib.md_xattn_head_pad(48) == 64 and lib.md_xattn_head_pad(2000) == 0
+    assert lib.md_xattn_fused_supported(None) == 0 and lib.md_linear_planes_count(3, 64, 2048, 1024) == 0
+    assert lib.md_linear_planes_count(1, 64, 2048, 1024) > 0 and lib.md_linear_planes_count(1, 64, 2040, 1024) == 0
+    skip |= {"md_xattn_head_pad", "md_xattn_fused_supported", "md_linear_planes_count"}
     for name, (restype, argtypes) in _lib._SIGNATURES.items():
         if name in skip:
             continue
         args = []
         for t in argtypes:
-            args.append(None if t is ctypes.c_void_p else (0.0 if t in (ctypes.c_float, ctypes.c_double) else 0))
+            args.append(None if t is ctypes.c_void_p or hasattr(t, "_type_") and hasattr(t, "contents") else (0.0 if t in (ctypes.c_float, ctypes.c_double) else 0))
         rc = getattr(lib, name)(*args)
         if restype is ctypes.c_size_t:
             assert rc == 0, name

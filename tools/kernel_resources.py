@@ -22,15 +22,14 @@ def demangle(names):
 
 def main():
     rows = []
-    for f in sorted(os.listdir(CSRC)):
-        if not f.endswith(".hip"):
-            continue
-        base = f[:-4]
+    units = [(f[:-4], f, []) for f in sorted(os.listdir(CSRC)) if f.endswith(".hip") and f != "xattn_mfma.hip"]
+    units += [(f"xattn_dk{dk}", "xattn_mfma.hip", [f"-DMD_XATTN_DK={dk}"]) for dk in (32, 64, 96, 128, 192, 256)]
+    for base, f, defs in units:
         with tempfile.TemporaryDirectory() as td:
             out = os.path.join(td, base + ".s")
             cmd = ["/opt/rocm/bin/hipcc", "-O3", "-std=c++17", "--offload-arch=gfx950", "-Xclang", "-target-feature", "-Xclang",
                    "-packed-fp32-ops", "--cuda-device-only", "-S",
-                   os.path.join(CSRC, f), "-o", out]
+                   os.path.join(CSRC, f), "-o", out] + defs
             if base in EXACT:
                 cmd.insert(3, "-ffp-contract=off")
             subprocess.run(cmd, check=True, capture_output=True)
