@@ -25,11 +25,6 @@
 
 namespace {
 
-template <typename T>
-__device__ __forceinline__ float ld1(const T* p, int64_t i) {
-    return (float)p[i];
-}
-
 template <int VEC>
 __device__ __forceinline__ void ld_vec(const float* p, float (&f)[VEC]) {
     if constexpr (VEC == 8) {
@@ -254,7 +249,7 @@ void launch_resid(const ResidParams& p, int dtype, bool vec, dim3 grid, hipStrea
     }
 }
 
-template <typename T>
+template <typename T, int VEC>
 __global__ __launch_bounds__(256) void embed_pos_kernel(const int64_t* __restrict__ tokens, const T* __restrict__ table,
                                                         const T* __restrict__ pos_table, const int32_t* __restrict__ qo_indptr,
                                                         const int32_t* __restrict__ pos0, int width, int vocab, int max_pos,
@@ -266,11 +261,24 @@ __global__ __launch_bounds__(256) void embed_pos_kernel(const int64_t* __restric
     tok = tok < 0 ? 0 : (tok >= vocab ? vocab - 1 : tok);            // the host refuses such ids; never index past the table
     int pos = pos0[b] + j;
     pos = pos < 0 ? 0 : (pos >= max_pos ? max_pos - 1 : pos);
-    for (int i = threadIdx.x; i < width; i += 256) {
-        float v = ld1(table, tok * width + i) * scale;
-        if (pos_table) v += ld1(pos_table, (int64_t)pos * width + i);
-        out[(int64_t)(q0 + j) * width + i] = v;
+    for (int i = threadIdx.x; i < width / VEC; i += 256) {
+        float v[VEC], q[VEC];
+        ld_vec<VEC>(table + tok * width + i * VEC, v);
+        if (pos_table) ld_vec<VEC>(pos_table + (int64_t)pos * width + i * VEC, q);
+#pragma unroll
+        for (int e = 0; e < VEC; ++e) {
+            v[e] *= scale;
+            if (pos_table) v[e] += q[e];
+        }
+        st_vec<VEC>(out + (int64_t)(q0 + j) * width + i * VEC, v);
     }
+}
+
+template <typename T, int VEC>
+void launch_embed(const int64_t* tokens, const void* table, const void* pos_table, const int32_t* qo_indptr, const int32_t* pos0,
+                  dim3 grid, int width, int vocab, int max_pos, float scale, float* out, hipStream_t st) {
+    hipLaunchKernelGGL((embed_pos_kernel<T, VEC>), grid, dim3(256), 0, st, tokens, (const T*)table, (const T*)pos_table,
+                       qo_indptr, pos0, width, vocab, max_pos, scale, out);
 }
 
 bool aligned16(const void* q) { return ((uintptr_t)q & 15) == 0; }
@@ -348,13 +356,10 @@ extern "C" int md_embed_pos(const int64_t* tokens, const void* table, const void
     MD_CHECK_ARG(B > 0 && B <= 65535 && n_max > 0 && width > 0 && vocab > 0 && max_pos > 0,
                  "md_embed_pos: bad shape B=%d n_max=%d width=%d", B, n_max, width);
     MD_CHECK_ARG(dtype == MD_T_BF16 || dtype == MD_T_F32, "md_embed_pos: dtype must be MD_T_BF16 or MD_T_F32");
-    const dim3 grid(n_max, B);
-    if (dtype == MD_T_F32)
-        hipLaunchKernelGGL((embed_pos_kernel<float>), grid, dim3(256), 0, (hipStream_t)stream, tokens, (const float*)table,
-                           (const float*)pos_table, qo_indptr, pos0, width, vocab, max_pos, scale, out);
-    else
-        hipLaunchKernelGGL((embed_pos_kernel<bf16_t>), grid, dim3(256), 0, (hipStream_t)stream, tokens, (const bf16_t*)table,
-                           (const bf16_t*)pos_table, qo_indptr, pos0, width, vocab, max_pos, scale, out);
+    const bool vec = width % 8 == 0 && aligned16(table) && aligned16(pos_table) && aligned16(out);
+    auto k = dtype == MD_T_F32 ? (vec ? launch_embed<float, 8> : launch_embed<float, 1>)
+                               : (vec ? launch_embed<bf16_t, 8> : launch_embed<bf16_t, 1>);
+    k(tokens, table, pos_table, qo_indptr, pos0, dim3(n_max, B), width, vocab, max_pos, scale, out, (hipStream_t)stream);
     MD_CHECK_LAUNCH("md_embed_pos");
     return MD_OK;
 }

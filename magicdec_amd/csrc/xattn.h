@@ -26,6 +26,7 @@ struct XattnParams {
 // one translation unit per padded query/key width; false: no kernel for (DKp, DVp)
 #define MD_XATTN_DECL(DK)                                                                                       \
     int md_internal_xattn_decode_##DK(const XattnParams& p, int qt, bool fused, int grid, hipStream_t st);       \
+    int md_internal_xattn_waves_##DK(int dv, int g, int rows);                                                    \
     int md_internal_xattn_prefill_##DK(const XattnParams& p, int nw, int grid, hipStream_t st);
 MD_XATTN_DECL(32)
 MD_XATTN_DECL(64)

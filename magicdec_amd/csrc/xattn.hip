@@ -59,6 +59,52 @@ __global__ __launch_bounds__(256) void qk_norm_append_kernel(const XattnParams p
     }
 }
 
+// the same with 8-element pieces (head sizes and rows that are multiples of 8): `lanes` = lanes per head vector (a power of two
+// that covers its padded width), several heads per wavefront; the sum of squares is a butterfly over them
+template <typename T>
+__global__ __launch_bounds__(256) void qk_norm_append_vec_kernel(const XattnParams p, T* __restrict__ q_out, int lanes_log2,
+                                                                 int vlanes_log2) {
+    typedef T vec8 __attribute__((ext_vector_type(8)));
+    const int b = blockIdx.y, j = blockIdx.x;
+    const int q0 = p.qo_indptr[b];
+    if (j >= p.qo_indptr[b + 1] - q0) return;
+    const int pos = p.pos0[b] + j;
+    const int pg0 = p.page_indptr[b], np = p.page_indptr[b + 1] - pg0;
+    const bool fits = pos >= 0 && pos < np * p.page_size;
+    if (!fits && threadIdx.x == 0) atomicAdd(p.overflow, 1u);
+    const int page = fits ? p.page_indices[pg0 + pos / p.page_size] : 0, slot = pos % p.page_size;
+    const T* row = reinterpret_cast<const T*>(p.qkv) + (int64_t)(q0 + j) * p.ld_qkv;
+    const int nqk = (p.H + p.KH) << lanes_log2, total = nqk + (p.KH << vlanes_log2);
+    for (int i = threadIdx.x; i < total; i += 256) {          // a head's lanes are aligned neighbours: active together
+        if (i < nqk) {
+            const int hv = i >> lanes_log2, d = (i - (hv << lanes_log2)) * 8;
+            f32x8 v = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
+            if (d < p.D) v = __builtin_convertvector(*reinterpret_cast<const vec8*>(row + hv * p.D + d), f32x8);
+            float ss = 0.f;
+#pragma unroll
+            for (int e = 0; e < 8; ++e) ss += v[e] * v[e];
+            for (int o = 1; o < (1 << lanes_log2); o <<= 1) ss += __shfl_xor(ss, o);
+            const float rs = p.qk_norm ? 1.0f / sqrtf(ss / (float)p.D + p.eps) : 1.f;
+            if (d >= p.DKp || (hv >= p.H && !fits)) continue;
+            T* dst = hv < p.H ? q_out + ((int64_t)(q0 + j) * p.H + hv) * p.DKp
+                              : reinterpret_cast<T*>(p.k_cache) + (((int64_t)page * p.KH + hv - p.H) * p.page_size + slot) * p.DKp;
+            *reinterpret_cast<vec8*>(dst + d) = __builtin_convertvector(v * rs, vec8);
+        } else {
+            const int h = (i - nqk) >> vlanes_log2, d = (i - nqk - (h << vlanes_log2)) * 8;
+            if (d >= p.DVp || !fits) continue;
+            vec8 v = {};
+            if (d < p.DV) v = *reinterpret_cast<const vec8*>(row + (p.H + p.KH) * p.D + h * p.DV + d);
+            *reinterpret_cast<vec8*>(reinterpret_cast<T*>(p.v_cache) + (((int64_t)page * p.KH + h) * p.page_size + slot) * p.DVp + d) = v;
+        }
+    }
+}
+
+int lanes_log2_of(int padded) {           // lanes of 8 elements each
+    int n = 0;
+    while ((8 << n) < padded) ++n;
+    return n;
+}
+
 // ------------------------------------------------------------------------------------------------ plain attention
 template <typename T>
 __device__ __forceinline__ float dot_row(const T* k, const float* q, int n);
@@ -294,6 +340,16 @@ extern "C" int md_qk_norm_append(const md_xattn_args* a, void* q_out, md_stream_
     const XattnParams p = make_params(a);
     MD_CHECK_ARG(p.overflow, "md_qk_norm_append: cannot resolve the page-overflow counter");
     const dim3 grid(a->n_max, a->B);
+    const int ll = lanes_log2_of(p.DKp), lv = lanes_log2_of(p.DVp);
+    if (a->D % 8 == 0 && a->DV % 8 == 0 && a->ld_qkv % 8 == 0 && ll <= 6 && lv <= 6 &&
+        (((uintptr_t)a->qkv | (uintptr_t)q_out) & 31) == 0) {
+        if (a->dtype == MD_T_F32)
+            hipLaunchKernelGGL((qk_norm_append_vec_kernel<float>), grid, dim3(256), 0, (hipStream_t)stream, p, (float*)q_out, ll, lv);
+        else
+            hipLaunchKernelGGL((qk_norm_append_vec_kernel<bf16_t>), grid, dim3(256), 0, (hipStream_t)stream, p, (bf16_t*)q_out, ll, lv);
+        MD_CHECK_LAUNCH("md_qk_norm_append");
+        return MD_OK;
+    }
     if (a->dtype == MD_T_F32)
         hipLaunchKernelGGL((qk_norm_append_kernel<float>), grid, dim3(256), 0, (hipStream_t)stream, p, (float*)q_out);
     else
@@ -315,7 +371,14 @@ extern "C" int md_xattn(const md_xattn_args* a, md_stream_t stream) {
         MD_CHECK_ARG(((uintptr_t)a->qkv & 15) == 0 && a->ld_qkv % 8 == 0 && p.overflow,
                      "md_xattn: projection rows must be 16-byte aligned");
     }
-    if (!mfma_ok(a) || a->force_plain) {
+    const int rows = decode_rows(a), pairs8 = (a->B * a->KH + 7) / 8 * 8;
+    int nw = 0;                                   // prefill: wavefronts per workgroup (0: its bias table does not fit)
+    if (mfma_ok(a) && rows > 32) {
+#define MD_XW(DK) case DK: nw = md_internal_xattn_waves_##DK(p.DVp, p.g, rows); break;
+        switch (p.DKp) { MD_XW(32) MD_XW(64) MD_XW(96) MD_XW(128) MD_XW(192) default: nw = md_internal_xattn_waves_256(p.DVp, p.g, rows); }
+#undef MD_XW
+    }
+    if (!mfma_ok(a) || a->force_plain || (rows > 32 && nw == 0)) {
         MD_CHECK_ARG(!fused, "md_xattn: the plain kernel takes normalised queries");
         const dim3 grid(a->n_max, a->H, a->B);
         if (a->dtype == MD_T_F32)
@@ -325,7 +388,6 @@ extern "C" int md_xattn(const md_xattn_args* a, md_stream_t stream) {
         MD_CHECK_LAUNCH("md_xattn(plain)");
         return MD_OK;
     }
-    const int rows = decode_rows(a), pairs8 = (a->B * a->KH + 7) / 8 * 8;
     int rc;
     if (rows <= 32) {
         p.nsplit = decode_splits(a);
@@ -345,7 +407,6 @@ extern "C" int md_xattn(const md_xattn_args* a, md_stream_t stream) {
             hipLaunchKernelGGL(xattn_merge_kernel, dim3((unsigned)((threads + 255) / 256)), dim3(256), 0, st, p);
         }
     } else {
-        const int nw = rows >= 256 ? 8 : 4;
         p.n_qgroups = (rows + 32 * nw - 1) / (32 * nw);
         const int grid = pairs8 * p.n_qgroups;
 #define MD_XP(DK) case DK: rc = md_internal_xattn_prefill_##DK(p, nw, grid, st); break;

@@ -8,7 +8,10 @@
 //   * there is no rescaling, no max reduction, and no second pass over a tile's scores: a 32-key block goes from its S
 //     accumulator to P to the PV product at once, 16 + 16 registers instead of a whole tile's worth;
 //   * partial sums of wavefronts and of kv splits simply add up.
-// The distance bias is one fma + v_log_f32 + fma per score (log2 domain: r1 ln(x) = (r1 log2 x) in the exp2 argument).
+// The distance bias is taken in the log2 domain (r1 ln(x) = (r1 log2 x) in the exp2 argument).  Decode evaluates it per score
+// (fma + v_log_f32 + fma: 8 scores per lane and tile); prefill looks it up: a workgroup's rows and a key tile meet at only
+// KT + tokens different distances, so the workgroup fills a small table per head and tile (a few logarithms per thread instead
+// of one per score) and every score is one fma with a table entry.  Negative distances hold -inf: the causal mask is the table.
 //
 // P is kept to 16 significant bits: the bf16 weight and the bf16 rest of it feed two PV products, so that the attention
 // weights reach the 32-bit accumulator with an error of 2^-17 instead of 2^-9.
@@ -325,13 +328,14 @@ __global__ __launch_bounds__(256, (decode_wgs<DV, QT>())) void xattn_decode_kern
 // NW wavefronts of 32 query rows (token-major: row = token * g + head of the group) share KT-key tiles through two LDS
 // images, one barrier per tile.  A workgroup visits the tiles from its first row's chunk start to its last row's position.
 template <int DV, int NW, int KT>
-__global__ __launch_bounds__(64 * NW, NW == 8 ? 2 : 1) void xattn_prefill_kernel(const XattnParams p) {
+__global__ __launch_bounds__(64 * NW, NW == 8 ? 2 : 1) void xattn_prefill_kernel(const XattnParams p, const int W) {
     constexpr int KS = DK / 16, NB = DV / 16, DB = DV / 32;
     constexpr int K_BYTES = KT * KROW, VG = NB * kVSub, STAGE = stage_bytes<DV>(KT);
     constexpr int CK = KT * DK / 8, CV = KT * DV / 8;            // 16-byte pieces of a tile
     constexpr int NK = (CK + 64 * NW - 1) / (64 * NW), NV = (CV + 64 * NW - 1) / (64 * NW);
-    extern __shared__ __attribute__((aligned(16))) unsigned char smem[];   // 2 x STAGE, then int[2 NW]
+    extern __shared__ __attribute__((aligned(16))) unsigned char smem[];   // 2 x STAGE, int[2 NW], 2 x float[g W]
     int* s_rng = reinterpret_cast<int*>(smem + 2 * STAGE);
+    float* s_bias = reinterpret_cast<float*>(smem + 2 * STAGE + 8 * NW);
     const int tid = threadIdx.x, lane = tid & 63, j = lane & 31, kh = lane >> 5;
     const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
     const int r0 = blockIdx.x >> 3;
@@ -348,17 +352,15 @@ __global__ __launch_bounds__(64 * NW, NW == 8 ? 2 : 1) void xattn_prefill_kernel
     const int qi = valid ? R / g : 0, qr = valid ? R - qi * g : 0, h = kvh * g + qr;
     const int pos = pos_b + qi;
     const int lim = valid ? min(pos, cap - 1) : -1, low = valid ? (pos / p.chunk) * p.chunk : 0x7fffffff;
-    int hi = lim, lim_min = valid ? lim : 0x7fffffff, lo = low, low_max = valid ? low : -1;
+    int hi = lim, lo = low, low_max = valid ? low : -1;
 #pragma unroll
     for (int o = 1; o < 32; o <<= 1) {
         hi = max(hi, __shfl_xor(hi, o));
-        lim_min = min(lim_min, __shfl_xor(lim_min, o));
         lo = min(lo, __shfl_xor(lo, o));
         low_max = max(low_max, __shfl_xor(low_max, o));
     }
     hi = __builtin_amdgcn_readfirstlane(hi);
     lo = __builtin_amdgcn_readfirstlane(lo);
-    lim_min = __builtin_amdgcn_readfirstlane(lim_min);
     low_max = __builtin_amdgcn_readfirstlane(low_max);
     if (lane == 0) {
         s_rng[wave] = hi;
@@ -381,8 +383,26 @@ __global__ __launch_bounds__(64 * NW, NW == 8 ? 2 : 1) void xattn_prefill_kernel
 #pragma unroll
         for (int ks = 0; ks < KS; ++ks) qf[ks] = valid ? *reinterpret_cast<const bf16x8*>(qp + ks * 16 + kh * 8) : z;
     }
-    const float r1 = p.r1 ? p.r1[h] : 0.f, r2 = p.r2 ? p.r2[h] : 0.f;
     const float sl2 = p.scale_log2, mref = -p.ref_log2;
+    // bias table of one tile: entry e of head r is the distance d = (position of the workgroup's first token) - (last key of
+    // the tile) + e.  A lane's entries have the same indexes in every tile.
+    const int tok0 = qg * NW * 32 / g, tsize = g * W;
+    const float* my_bias = s_bias + (valid ? qr * W + qi - tok0 : 0) + 4 - 4 * kh;
+    const int fill_r = tid / W, fill_e = tid - fill_r * W;
+    auto fill = [&](int t, float* tab) {
+        const int d0 = pos_b + tok0 - (t * KT + KT - 1);
+        int r = fill_r, e = fill_e;
+        for (int i = tid; i < tsize; i += 64 * NW) {
+            const float a = p.r1 ? p.r1[kvh * g + r] : 0.f, c = p.r1 ? p.r2[kvh * g + r] : 0.f;
+            const int d = d0 + e;
+            tab[i] = d < 0 ? -INFINITY : fmaf(-a, __builtin_amdgcn_logf(fmaf(c, (float)d, 1.0f)), mref);
+            e += 64 * NW;
+            while (e >= W) {
+                e -= W;
+                ++r;
+            }
+        }
+    };
     f32x16 o[DB];
 #pragma unroll
     for (int db = 0; db < DB; ++db)
@@ -407,15 +427,17 @@ __global__ __launch_bounds__(64 * NW, NW == 8 ? 2 : 1) void xattn_prefill_kernel
     auto stage = [&](int t, unsigned char* img) {
 #pragma unroll
         for (int i = 0; i < NK; ++i) {
-            const int c = i * 64 * NW + tid;
-            if (CK % (64 * NW) == 0 || c < CK)
-                *reinterpret_cast<u32x4*>(img + (c / (DK / 8)) * KROW + (c % (DK / 8)) * 16) = kreg[i];
+            const int c = i * 64 * NW + tid, row = c / (DK / 8);
+            if (CK % (64 * NW) == 0 || c < CK) {
+                if (t * KT + row > last) kreg[i] = u32x4{0u, 0u, 0u, 0u};     // rows not written yet may hold anything (NaN)
+                *reinterpret_cast<u32x4*>(img + row * KROW + (c % (DK / 8)) * 16) = kreg[i];
+            }
         }
 #pragma unroll
         for (int i = 0; i < NV; ++i) {
             const int c = i * 64 * NW + tid, row = c / (DV / 8), ch = c % (DV / 8);
             if (CV % (64 * NW) == 0 || c < CV) {
-                if (t * KT + row > last) vreg[i] = u32x4{0u, 0u, 0u, 0u};     // rows not written yet may hold anything
+                if (t * KT + row > last) vreg[i] = u32x4{0u, 0u, 0u, 0u};
                 *reinterpret_cast<u32x4*>(img + K_BYTES + (row >> 5) * VG + (ch >> 1) * kVSub + (row & 31) * 32 + (ch & 1) * 16) =
                     vreg[i];
             }
@@ -425,7 +447,7 @@ __global__ __launch_bounds__(64 * NW, NW == 8 ? 2 : 1) void xattn_prefill_kernel
     const int lq = lane & 15;
     // the two 16-d sub-tiles one transpose read pairs lie NB / 2 apart (disjoint LDS banks at the usual widths)
     const int vra0 = K_BYTES + ((lane >> 4) & 1) * (NB / 2) * kVSub + (kh * 4 + (lq >> 2)) * 32 + (lq & 3) * 8;
-    auto compute = [&](int t, const unsigned char* img, bool masked) {
+    auto compute = [&](int t, const unsigned char* img, const float* bias, bool masked) {
         constexpr int KGU = KT >= 64 ? 2 : 1;                      // 32-key blocks whose S products run interleaved
 #pragma unroll
         for (int kg0 = 0; kg0 < KT / 32; kg0 += KGU) {
@@ -444,18 +466,15 @@ __global__ __launch_bounds__(64 * NW, NW == 8 ? 2 : 1) void xattn_prefill_kernel
 #pragma unroll
             for (int u = 0; u < KGU; ++u) {
                 const int kbase = t * KT + (kg0 + u) * 32 + 4 * kh;
-                const float c0 = fmaf(r2, (float)(pos - kbase), 1.0f);
 #pragma unroll
-                for (int r = 0; r < 16; ++r) {
-                    const float lg = __builtin_amdgcn_logf(fmaf(r2, -(float)((r & 3) + 8 * (r >> 2)), c0));
-                    sc[u][r] = fmaf(-r1, lg, fmaf(sc[u][r], sl2, mref));
-                }
-                if (masked) {                                       // wave-uniform branch
+                for (int r = 0; r < 16; ++r)
+                    sc[u][r] = fmaf(sc[u][r], sl2, bias[(KT / 32 - 1 - kg0 - u) * 32 + 27 - (r & 3) - 8 * (r >> 2)]);
+                if (masked) {                                       // keys of the previous chunk; a wave-uniform branch
 #pragma unroll
                     for (int r = 0; r < 16; ++r) {
                         const int kp = kbase + (r & 3) + 8 * (r >> 2);
                         float v = sc[u][r];
-                        if (kp > lim || kp < low) v = -INFINITY;
+                        if (kp < low) v = -INFINITY;
                         asm volatile("" : "+v"(v));                 // keeps the selects inside the branch
                         sc[u][r] = v;
                     }
@@ -488,9 +507,10 @@ __global__ __launch_bounds__(64 * NW, NW == 8 ? 2 : 1) void xattn_prefill_kernel
     for (int t = t0; t <= t1; ++t) {
         unsigned char* img = smem + (t & 1) * STAGE;
         stage(t, img);
+        fill(t, s_bias + (t & 1) * tsize);
         if (t < t1) issue(t + 1);
         __syncthreads();
-        if (t >= my0 && t <= my1) compute(t, img, t * KT + KT - 1 > lim_min || t * KT < low_max);
+        if (t >= my0 && t <= my1) compute(t, img, my_bias + (t & 1) * tsize, t * KT < low_max);
     }
 
     l += __shfl_xor(l, 32);
@@ -544,16 +564,37 @@ int decode_dv(const XattnParams& p, int qt, bool fused, int grid, hipStream_t st
 }
 
 template <int DV, int NW>
+constexpr int prefill_kt() { return NW == 8 && 2 * stage_bytes<DV>(128) <= 144 * 1024 ? 128 : 64; }
+
+// width of a bias table row: every distance between the workgroup's tokens and a tile's keys, the rows of the group's heads
+// spread over the LDS banks
+template <int DV, int NW>
+int bias_width(int g) {
+    int w = prefill_kt<DV, NW>() + (NW * 32 - 1) / g + 2;
+    const int want = g < 64 ? 64 / g : 1;
+    while (w % 64 != want % 64) ++w;
+    return w;
+}
+template <int DV, int NW>
+int prefill_lds(int g) { return 2 * stage_bytes<DV>(prefill_kt<DV, NW>()) + 8 * NW + 8 * g * bias_width<DV, NW>(g); }
+
+template <int DV, int NW>
 int launch_prefill(const XattnParams& p, int grid, hipStream_t st) {
-    constexpr int KT = NW == 8 && 2 * stage_bytes<DV>(128) <= 150 * 1024 ? 128 : 64;
-    constexpr int lds = 2 * stage_bytes<DV>(KT) + 8 * NW;
-    static_assert(lds <= 160 * 1024, "the two tile images must fit the CU");
+    static_assert(2 * stage_bytes<DV>(prefill_kt<DV, NW>()) <= 150 * 1024, "the two tile images must fit the CU");
     static MdPerDeviceOnce once;
-    auto k = xattn_prefill_kernel<DV, NW, KT>;
-    const int rc = raise_lds(k, lds, once);
+    auto k = xattn_prefill_kernel<DV, NW, prefill_kt<DV, NW>()>;
+    const int rc = raise_lds(k, 160 * 1024, once);
     if (rc != MD_OK) return rc;
-    hipLaunchKernelGGL(k, dim3(grid), dim3(64 * NW), lds, st, p);
+    const int lds = prefill_lds<DV, NW>(p.g), width = bias_width<DV, NW>(p.g);
+    hipLaunchKernelGGL(k, dim3(grid), dim3(64 * NW), lds, st, p, width);
     return MD_OK;
+}
+
+// wavefronts per workgroup for this many rows: 8 where the rows fill them and the bias table fits beside the tiles; 0: none fits
+template <int DV>
+int prefill_waves(int g, int rows) {
+    if (rows >= 256 && prefill_lds<DV, 8>(g) <= 160 * 1024) return 8;
+    return prefill_lds<DV, 4>(g) <= 160 * 1024 ? 4 : 0;
 }
 
 template <int DV>
@@ -574,6 +615,17 @@ int MD_CAT(md_internal_xattn_decode_, MD_XATTN_DK)(const XattnParams& p, int qt,
     case 128: return decode_dv<128>(p, qt, fused, grid, st);
     case 192: return decode_dv<192>(p, qt, fused, grid, st);
     default: return decode_dv<256>(p, qt, fused, grid, st);
+    }
+}
+
+int MD_CAT(md_internal_xattn_waves_, MD_XATTN_DK)(int dv, int g, int rows) {
+    switch (dv) {
+    case 32: return prefill_waves<32>(g, rows);
+    case 64: return prefill_waves<64>(g, rows);
+    case 96: return prefill_waves<96>(g, rows);
+    case 128: return prefill_waves<128>(g, rows);
+    case 192: return prefill_waves<192>(g, rows);
+    default: return prefill_waves<256>(g, rows);
     }
 }
 
