@@ -325,10 +325,14 @@ __global__ __launch_bounds__(256, (decode_wgs<DV, QT>())) void xattn_decode_kern
 }
 
 // ------------------------------------------------------------------------------------------------ prefill
+// heads of at most 64: 64-key tiles and 128 registers put two eight-wave workgroups on a CU
+template <int DV>
+constexpr bool small_heads() { return DK <= 64 && DV <= 64; }
+
 // NW wavefronts of 32 query rows (token-major: row = token * g + head of the group) share KT-key tiles through two LDS
 // images, one barrier per tile.  A workgroup visits the tiles from its first row's chunk start to its last row's position.
 template <int DV, int NW, int KT>
-__global__ __launch_bounds__(64 * NW, NW == 8 ? 2 : 1) void xattn_prefill_kernel(const XattnParams p, const int W) {
+__global__ __launch_bounds__(64 * NW, NW == 8 ? (small_heads<DV>() ? 4 : 2) : 1) void xattn_prefill_kernel(const XattnParams p, const int W) {
     constexpr int KS = DK / 16, NB = DV / 16, DB = DV / 32;
     constexpr int K_BYTES = KT * KROW, VG = NB * kVSub, STAGE = stage_bytes<DV>(KT);
     constexpr int CK = KT * DK / 8, CV = KT * DV / 8;            // 16-byte pieces of a tile
@@ -448,7 +452,7 @@ __global__ __launch_bounds__(64 * NW, NW == 8 ? 2 : 1) void xattn_prefill_kernel
     // the two 16-d sub-tiles one transpose read pairs lie NB / 2 apart (disjoint LDS banks at the usual widths)
     const int vra0 = K_BYTES + ((lane >> 4) & 1) * (NB / 2) * kVSub + (kh * 4 + (lq >> 2)) * 32 + (lq & 3) * 8;
     auto compute = [&](int t, const unsigned char* img, const float* bias, bool masked) {
-        constexpr int KGU = KT >= 64 ? 2 : 1;                      // 32-key blocks whose S products run interleaved
+        constexpr int KGU = NW == 8 && small_heads<DV>() ? 1 : 2;    // 32-key blocks whose S products run interleaved
 #pragma unroll
         for (int kg0 = 0; kg0 < KT / 32; kg0 += KGU) {
             f32x16 sc[KGU];
@@ -564,7 +568,7 @@ int decode_dv(const XattnParams& p, int qt, bool fused, int grid, hipStream_t st
 }
 
 template <int DV, int NW>
-constexpr int prefill_kt() { return NW == 8 && 2 * stage_bytes<DV>(128) <= 144 * 1024 ? 128 : 64; }
+constexpr int prefill_kt() { return NW == 8 && !small_heads<DV>() && 2 * stage_bytes<DV>(128) <= 144 * 1024 ? 128 : 64; }
 
 // width of a bias table row: every distance between the workgroup's tokens and a tile's keys, the rows of the group's heads
 // spread over the LDS banks
