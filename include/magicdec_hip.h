@@ -383,17 +383,17 @@ int md_linear_fused_split_add_rmsnorm(const void* x, int64_t ldx, const void* w_
  * md_resid_norm_shift   the same with h = the normalised row and y_t = h_t + (h_{t-1} - h_t) * shift.  The h of the last rows
  *                       of every sequence live in `ring` [slots][ring_len][width] fp32, position p in entry p % ring_len
  *                       (slots: ring row of request b; NULL = b); a sequence may be rolled back by ring_len - 2 positions.
- * md_xielu              y = z > 0 ? softplus(act[0]) z^2 + z / 2 : (1/2 + softplus(act[1])) (e^z - 1 - z) + z / 2 (fp32, one
- *                       rounding; in place allowed; act = two fp32 values on the device).
+ * md_xielu              y = z / 2 + (z > 0 ? a z z : b (expm1(z) - z)), a = log1p(exp(act[0])), b = 1/2 + log1p(exp(act[1])); one
+ *                       rounding (in place allowed; act = two fp32 values on the device).
  * md_linear_planes      x [M][K] . W^T as md_linear_planes_count fp32 partial planes [n][M][N] (0: unsupported) -- one of the
  *                       split-K GEMMs (W in the streaming layout) without its combine launch: md_resid_norm[_shift] adds the
  *                       planes to the residual.
  * md_linear_xielu, md_linear_block_xielu, MD_FL_XIELU (md_linear_fused): the linear with the activation as its epilogue.
- * md_qk_norm_append     qkv rows (q heads | k heads | v heads) -> q_out [rows][H][pad(D)] and the pages: q and k divided by
- *                       their root mean square per head when qk_norm is set, rows zero-padded.
- * md_xattn              softmax attention over the pages; position i sees j <= i in its chunk (chunk = 0: no chunks), score
- *                       = (q.k) * scale - r1[h] ln(1 + r2[h] (i - j)) (r1 = r2 = NULL: none), sink: one more score of 0
- *                       without a value.  With q = NULL and qkv given (md_xattn_fused_supported: decode / verify steps of at
+ * md_qk_norm_append     qkv rows (q heads | k heads | v heads) -> q_out [rows][H][pad(D)] and the pages: with qk_norm q
+ *                       and k heads are scaled to unit RMS (fp32, eps inside the root); rows zero-padded.
+ * md_xattn              softmax attention over the pages; a row at position t sees (t / chunk) * chunk .. t (chunk = 0: all
+ *                       before it); at distance d the score is scale q.k - a ln(1 + c d), a = r1[h], c = r2[h] (both NULL:
+ *                       no penalty); sink: the softmax denominator is 1 + the sum of the exponentials.  With q = NULL and qkv given (md_xattn_fused_supported: decode / verify steps of at
  *                       most 32 rows per kv head) the normalisation and the append happen in the same launch.
  *                       score_bound > 0: no score exceeds it (e.g. D * scale with qk_norm and r1 >= 0); needed by the
  *                       matrix-core kernels, 0 = unknown.

@@ -22,9 +22,9 @@ class AttentionSpec:
     vdim: int                     # value size per head
     scale: float
     chunk: int = 0                # positions see their own chunk only; 0: no chunks
-    qk_norm: bool = False         # queries and keys divided by their root mean square per head
-    distance_bias: bool = False   # r1_h ln(1 + r2_h (i - j)) taken off the score
-    sink: bool = False            # one more score of 0, without a value, in the softmax denominator
+    qk_norm: bool = False         # query and key heads scaled to unit RMS, without weights
+    distance_bias: bool = False   # logarithmic penalty on the distance, two coefficients per head
+    sink: bool = False            # the softmax leaves weight 1 / (1 + S) unassigned (S: the sum of the exponentials)
 
 
 @dataclass(frozen=True)
@@ -87,8 +87,8 @@ class _Reader:
 
 
 def _furitar(cfg) -> DecoderSpec:
-    """Furitar: pre-norm layers with a token shift in front of every mixer; chunked softmax attention with a query/key norm, a
-    logarithmic distance bias and a sink; learned positions; dense xIELU feed-forwards (or none)."""
+    """Furitar: pre-norm layers with a token shift in front of every mixer; chunked softmax attention with unit-RMS queries and keys, a
+    logarithmic distance penalty and a sink; learned positions; dense xIELU feed-forwards (or none)."""
     c = _Reader(cfg, "the model")
     c.get("architecture")
     emb, norm = c.sub("embedding"), c.sub("norm")

@@ -66,8 +66,8 @@ __device__ __forceinline__ float bf16_bits_to_f32(unsigned short b) {
 __device__ __forceinline__ bf16_t f32_to_bf16(float x) { return (bf16_t)x; }
 __device__ __forceinline__ float bf16_to_f32(bf16_t x) { return (float)x; }
 
-// xIELU: a quadratic with slope 1/2 at 0 on the right, an exponential one on the left; the coefficients are softplus of two
-// learned numbers.  fp32; expm1 keeps e^z - 1 - z accurate near 0
+// xIELU: z / 2 plus a quadratic on the right of 0 and an exponential remainder on the left, with learned coefficients (softplus
+// of the two stored numbers, the left one + 1/2).  fp32; expm1 keeps e^z - 1 - z accurate near 0
 struct Xielu {
     float ap, an;
     __device__ __forceinline__ explicit Xielu(const float* act) {

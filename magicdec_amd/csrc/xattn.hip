@@ -1,9 +1,9 @@
 // Extended paged attention (gfx950): the softmax attention of the layered decoder designs, every feature a parameter --
 //   * query/key and value head sizes of their own (K and V pages are separate slabs, rows padded to the kernels' widths);
-//   * queries and keys divided by their root mean square per head (fp32), at the append;
-//   * a distance bias taken off the score, r1_h ln(1 + r2_h (i - j));
-//   * a chunk mask: position i sees j <= i with floor(i / chunk) == floor(j / chunk);
-//   * a softmax sink: one more score of 0 without a value in the denominator.
+//   * unit-RMS query and key heads (scaled in fp32, no weights; keys once, at the append);
+//   * a distance penalty per query head, -a ln(1 + c d) at distance d (r1 = a, r2 = c);
+//   * block-diagonal causality: a row at position t sees the positions from (t / chunk) * chunk up to t;
+//   * a softmax sink: the denominator is 1 + (sum of the exponentials).
 // Positions come from pos0[b] + row, and a request's page list maps EVERY position it may reach (position p lies in its page
 // p / page_size), so that neither the append nor the attention needs a last-page length: decoding crosses pages, a step may
 // be run again, and a rolled-back sequence just writes its rows anew.

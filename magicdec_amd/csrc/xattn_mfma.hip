@@ -1,7 +1,7 @@
 // Matrix-core kernels of the extended paged attention (xattn.hip; bf16 pages).  Compiled once per padded query/key width:
 // -DMD_XATTN_DK=32 | 64 | 96 | 128 | 192 | 256; the value width is a template parameter of the same set.
 //
-// No running maximum.  Queries and keys are divided by their root mean square, so |q.k| <= dim and a score never exceeds
+// No running maximum.  Query and key heads have unit RMS, so |q.k| <= dim and a score never exceeds
 // dim * scale (plus what a negative bias coefficient can add): the host passes that bound, and softmax weights are taken
 // against the FIXED reference max(0, bound - 60) instead of the row's maximum.  The sink (weight exp(-reference)) keeps the
 // denominator away from 0, weights below exp(-87) of the reference are negligible next to it, and with the maximum gone

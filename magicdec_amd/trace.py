@@ -1,13 +1,14 @@
-"""Replays a trace: JSON steps on standard input, each bringing the next tokens of some sequences, through an engine's own
-`step` (Engine/backend_core.py) -- ragged batch, page pool, kernels -- and the logits of the asked-for places to files.
+"""Replay of a recorded trace through an engine's own `step` (Engine/backend_core.py: ragged batch, page pool, kernels).
 
-    trace_run --model DIR --dtype bfloat16|float32 --out DIR --max-tokens N
+    trace_run --model FOLDER --dtype bfloat16 --out RESULTS --max-tokens 4096 < trace.jsonl
 
-    {"step": 0, "entries": [{"id": "a", "tokens": [5, 17, 3], "want": [0, 2]}], "end": []}
+One JSON object per input line is one engine step: `step` (a number), `entries` (per sequence its `id`, its next `tokens` and
+in `want` the indexes among them whose logits are to be kept) and `end` (ids to release afterwards), for instance
 
-For a step in which something is wanted DIR/<step>.f32 receives the logits as little-endian float32 [wanted, vocab], in the
-order of the entries and their `want`; after every step the line `done <step>` is printed.  Sequences listed in `end` give
-their slot and pages back after the step.
+    {"step": 7, "entries": [{"id": "x", "tokens": [11], "want": [0]}, {"id": "y", "tokens": [2], "want": []}], "end": ["y"]}
+
+The kept logits of step 7 become RESULTS/7.f32 (rows of little-endian float32, entry by entry); `done 7` on standard output says
+that the step is finished.
 """
 from __future__ import annotations
 

@@ -6,40 +6,12 @@ Shapes: a sequence is [T, ...]; `pos` is the absolute position of its first row.
     embed            x_t = E[token_t] * scale + P[t]
     rms              x / sqrt(mean(x^2) + eps)                     (weighted: * w)
     token_shift      h_t + (h_{t-1} - h_t) * mu,  h_{-1} = 0
-    attention        s_ij = scale * <rms(q_i), rms(k_j)> - r1 ln(1 + r2 (i - j)),
-                     j <= i and floor(i / c) == floor(j / c);   p_ij = e^{s_ij} / (1 + sum_j e^{s_ij})
-    xielu            z > 0: softplus(p) z^2 + z / 2;   z <= 0: (1/2 + softplus(q)) (e^z - 1 - z) + z / 2
+    attention        E_ts = exp(scale <rms(q_t), rms(k_s)> - a ln(1 + c (t - s))) for c0(t) <= s <= t, c0 = first position of
+                     t's chunk;   o_t = sum_s E_ts v_s / (1 + sum_s E_ts)
+    xielu            z / 2 + A z^2 on the right of 0, z / 2 + B (expm1(z) - z) on the left; A, B - 1/2 = softplus of the two numbers
     head             rms(x) w . head^T * logit_scale
 """
-import json
-import os
-import struct
-
-import numpy as np
 import torch
-
-
-def read_safetensors(path):
-    with open(path, "rb") as f:
-        n = struct.unpack("<Q", f.read(8))[0]
-        head = json.loads(f.read(n))
-        data = f.read()
-    out = {}
-    for name, e in head.items():
-        if name == "__metadata__":
-            continue
-        lo, hi = e["data_offsets"]
-        buf = bytearray(data[lo:hi])
-        if e["dtype"] == "BF16":
-            t = torch.frombuffer(buf, dtype=torch.bfloat16)
-        elif e["dtype"] == "F32":
-            t = torch.frombuffer(buf, dtype=torch.float32)
-        elif e["dtype"] == "I32":
-            t = torch.frombuffer(buf, dtype=torch.int32)
-        else:
-            raise ValueError(e["dtype"])
-        out[name] = t.view(*e["shape"])
-    return out
 
 
 def rms(x, eps):
@@ -55,10 +27,6 @@ def token_shift(h, mu, before=None):
     first = torch.zeros_like(h[:1]) if before is None else before.view(1, -1)
     prev = torch.cat([first, h[:-1]], 0)
     return h + (prev - h) * mu
-
-
-def visible(i, j, chunk):
-    return j <= i and i // chunk == j // chunk
 
 
 def distance_bias(r1, r2, dist):
@@ -107,12 +75,6 @@ class RefModel:
     def __init__(self, cfg, tensors, dtype=torch.float64):
         self.cfg, self.dtype = cfg, dtype
         self.t = {k: v.to(dtype) for k, v in tensors.items()}
-
-    @classmethod
-    def load(cls, folder, dtype=torch.float64):
-        with open(os.path.join(folder, "config.json")) as f:
-            cfg = json.load(f)
-        return cls(cfg, read_safetensors(os.path.join(folder, "model.safetensors")), dtype)
 
     def new_state(self):
         return {"n": 0, "kv": [None] * len(self.cfg["layers"]), "h": [None] * len(self.cfg["layers"])}

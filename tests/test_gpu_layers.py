@@ -209,7 +209,7 @@ def attention_case(ops, H, KH, D, DV, chunk, seed, dtype, lens, score=12.0, r=(0
 
 
 ATT = [  # H, KH, D, DV, chunk
-    (4, 2, 32, 32, 48), (6, 1, 96, 48, 200), (8, 2, 64, 64, 130), (5, 5, 40, 24, 33), (7, 1, 20, 36, 1), (16, 1, 64, 128, 257),
+    (4, 2, 32, 32, 48), (10, 2, 88, 56, 190), (8, 2, 64, 64, 130), (5, 5, 40, 24, 33), (7, 1, 20, 36, 1), (16, 1, 64, 128, 257),
     (12, 4, 80, 112, 300), (4, 4, 128, 128, 129), (24, 1, 128, 64, 511), (3, 1, 192, 160, 77), (2, 2, 256, 256, 100),
     (33, 1, 32, 64, 64), (2, 1, 300, 40, 90), (2, 1, 50, 270, 90), (4, 2, 64, 64, 0)]
 

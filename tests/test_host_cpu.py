@@ -1227,7 +1227,7 @@ def test_command_line_flags_and_defaults_equal_the_reference_scripts():
     scripts differ (self-speculation defaults to B = 45, prefix 100000, gamma 7, budget 4097; StreamingLLM longspec to
     budget 1025; the baseline to B = 16, prefix 8065).  Deliberate differences: checkpoint paths are relative
     ("checkpoints/...", not "/scratch/models/..."), and the product adds --kv_dtype / --kv_layout (for the baseline
-    --dataset / --benchmark, for the two-model scripts --replicate_draft)."""
+    --dataset / --benchmark / --dtype / --ragged, for the two-model scripts --replicate_draft)."""
     from magicdec_amd import cli
     j = gc.load_json("cli_args.json")
     parsers = {"tests/SnapKV/longspec_benchmark.py": cli.longspec_parser("SnapKV"),
@@ -1253,7 +1253,7 @@ def test_command_line_flags_and_defaults_equal_the_reference_scripts():
                 assert repr(a.default) == ra["default"], (script, flag, a.default, ra["default"])
             else:
                 assert a.default is None, (script, flag, a.default)
-        allowed = extras | ({"--dataset", "--benchmark"} if "baseline" in script else set()) \
+        allowed = extras | ({"--dataset", "--benchmark", "--dtype", "--ragged"} if "baseline" in script else set()) \
             | ({"--replicate_draft"} if "longspec" in script else set())
         assert set(acts) - {r["flags"][0] for r in ref_args} <= allowed, (script, set(acts) - {r["flags"][0] for r in ref_args})
 
