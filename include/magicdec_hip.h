@@ -242,6 +242,7 @@ int md_silu_mul(const void* a, const void* b, int64_t a_row_stride, int64_t b_ro
 #define MD_W_INT8 1
 #define MD_EPI_NONE 0
 #define MD_EPI_SWIGLU 1
+#define MD_EPI_GEGLU 3 /* MD_EPI_SWIGLU's layout; out = bf16(gelu_tanh(h1) * h3), fp32 up to the one rounding */
 int md_linear_supported(int M, int N, int K, int epilogue);
 size_t md_linear_workspace_bytes(int M, int N, int K, int epilogue);
 int md_linear(const void* x, int64_t ldx, const void* w, int w_dtype, int w_packed, const void* scales,
@@ -315,6 +316,7 @@ int md_linear_block_add_rmsnorm(const void* x, int64_t ldx, const void* w_packed
 #define MD_FL_RESID 2
 #define MD_FL_ROPE_APPEND 3
 #define MD_FL_XIELU 4
+#define MD_FL_GEGLU 5  /* MD_FL_SWIGLU's layout; out = bf16(gelu_tanh(h1) * h3), fp32 up to the one rounding */
 typedef struct md_fused_linear_args {
     const void* x;            /* [M][K] bf16, row stride ldx (elements) */
     const void* w_packed;     /* streaming layout (md_linear, w_packed = 1) */
@@ -459,6 +461,76 @@ int md_xattn_fused_supported(const md_xattn_args* args);
 size_t md_xattn_workspace_bytes(const md_xattn_args* args);
 int md_qk_norm_append(const md_xattn_args* args, void* q_out, md_stream_t stream);
 int md_xattn(const md_xattn_args* args, md_stream_t stream);
+
+/* ------------------------------------------------------------------------
+ * K12  latent attention, bigram embedding, gated GELU, logit soft cap (layered decoder designs; no counterpart in the reference)
+ * A cache row [W = md_latent_row_width] of a token: latent (kv_rank) | rotated key part (rot_dim) | zeros; pages
+ * [pages][page_size][W], addressed by position.  cos_sin [max_pos][rot_pairs][2] (fp32): neighbouring elements of the first
+ * 2 * rot_pairs of a rotated vector turn.  Tensors are of `dtype` (MD_T_BF16 | MD_T_F32) unless said otherwise.
+ * md_latent_append   z rows = query latent (q_rank) | latent | key part: cq = rms(query latent) * dq_norm; with `append` the
+ *                    cache row (rms(latent) * kv_norm, rotated key part) of every row's position.
+ * md_latent_attn     q [rows][H][W] (absorbed queries | rotated parts | zeros) over the cache, causal, softmax of score * scale:
+ *                    out [rows][H][kv_rank].
+ * md_latent_gather   dst [ctx rows][kv_rank]: the latents of the positions 0 .. ctx_indptr[b+1] - ctx_indptr[b] - 1 of every
+ *                    request, dense (bf16; kv_rank % 8 == 0).
+ * md_latent_prefill  q [rows][H][dim + rot_dim] as projected (rotated here); kv [ctx rows][H * dim | H * vdim]: expanded keys and
+ *                    values of the context; gate (optional) [rows][ld_gate]: out *= sigmoid(gate[row][h]); out [rows][ldo].
+ * md_head_linear     out[row][h][n] = sum_k w[h][n][k] x[row][h][k] (* sigmoid(gate[row][h])); row / head strides in elements;
+ *                    with `tail` [row][h][tail_dim] also out[row][h][N ..] = rotated tail, zeros up to tail_pad.
+ * md_embed_bigram    out (fp32) = rms(table[token] + pairs[(mul_before * before + mul_token * token) mod buckets]) * norm_weight;
+ *                    row `buckets` of pairs for a sequence's first token; history (int32 [pages][page_size]) holds the tokens.
+ * md_gelu_mul        y = gelu_tanh(a) * b;  md_softcap  z = cap * tanh(z / cap), in place.
+ * ---------------------------------------------------------------------- */
+typedef struct md_latent_args {
+    const void* z;
+    const void* dq_norm;
+    const void* kv_norm;
+    void* cq;
+    void* cache;
+    const float* cos_sin;
+    const int32_t* qo_indptr;
+    const int32_t* pos0;
+    const int32_t* page_indices;
+    const int32_t* page_indptr;
+    const int32_t* ctx_indptr;
+    const void* q;
+    const void* kv;
+    const void* gate;
+    void* out;
+    void* workspace;
+    size_t workspace_bytes;
+    int64_t ldz, ldo, ld_gate;
+    float eps, scale;
+    int B, n_max, H, dim, rot_dim, rot_pairs, vdim, q_rank, kv_rank, page_size, max_pages, max_pos, append, dtype;
+    int force_plain;           /* 1: the plain attention kernel (comparison) */
+} md_latent_args;
+typedef struct md_head_linear_args {
+    const void* x;
+    const void* w;
+    void* out;
+    const void* gate;
+    const void* tail;
+    const float* cos_sin;
+    const int32_t* qo_indptr;
+    const int32_t* pos0;
+    int64_t ldx, hx, ldo, ho, ld_gate, ldt, ht;
+    int M, H, N, K, B, tail_dim, tail_pad, rot_pairs, max_pos, dtype;
+} md_head_linear_args;
+int md_latent_row_width(int kv_rank, int rot_dim);    /* 0: unsupported */
+int md_latent_append(const md_latent_args* args, md_stream_t stream);
+size_t md_latent_workspace_bytes(const md_latent_args* args);
+int md_latent_attn(const md_latent_args* args, md_stream_t stream);
+int md_latent_gather(const md_latent_args* args, int ctx_max, void* dst, md_stream_t stream);
+int md_latent_prefill_supported(const md_latent_args* args);
+int md_latent_prefill(const md_latent_args* args, md_stream_t stream);
+int md_head_linear(const md_head_linear_args* args, md_stream_t stream);
+int md_embed_bigram(const int64_t* tokens, const void* table, const void* pairs, const void* norm_weight, int dtype,
+                    const int32_t* qo_indptr, const int32_t* pos0, int B, int n_max, int width, int vocab, int buckets,
+                    int64_t mul_before, int64_t mul_token, int32_t* history, const int32_t* page_indices,
+                    const int32_t* page_indptr, int page_size, float eps, float* out, md_stream_t stream);
+int md_gelu_mul(const void* a, const void* b, int64_t a_row_stride, int64_t b_row_stride, void* y, int64_t y_row_stride, int rows,
+                int dim, int dtype, md_stream_t stream);
+int md_softcap(void* z, int64_t z_row_stride, float cap, int rows, int dim, int dtype, md_stream_t stream);
 
 /* ------------------------------------------------------------------------
  * K10  argmax over a vocab shard / TP merge

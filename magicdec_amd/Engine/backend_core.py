@@ -135,10 +135,13 @@ class _PagedState:
         self._get("paged_kv_indptr").copy_(torch.arange(B + 1, dtype=torch.int32, device=dev) * n_pages)
         self._set("paged_kv_last_page_len", torch.full((B,), last_page_len, dtype=torch.int32, device=dev))
 
-    def table(self):
+    def table(self, lengths=None):
+        """lengths: (new rows, positions after the step), the same for every request of the batch."""
         # (no slots: request b of a fixed batch is entry b of per-sequence state)
+        B = self.o.batch_size
         return PageTable(self._get("paged_kv_indices"), self._get("paged_kv_indptr"),
-                         self._get("paged_kv_last_page_len"), max(self.host_pages, 1))
+                         self._get("paged_kv_last_page_len"), max(self.host_pages, 1),
+                         lengths=tuple([v] * B for v in lengths) if lengths else None)
 
 
 class _BackendBase:
@@ -174,7 +177,8 @@ class _BackendBase:
         if self.mapped:
             self.max_num_pages_per_request = _mapped_pages_per_request(max_seq_length)
             self.max_num_pages = max_batch_size * self.max_num_pages_per_request
-            self.prefill_chunk = max(CHUNK, min(4096, PREFILL_ROWS // max_batch_size // CHUNK * CHUNK))
+            rows = max(PREFILL_ROWS, getattr(self.model, "prefill_rows", 0))
+            self.prefill_chunk = max(CHUNK, min(4096, rows // max_batch_size // CHUNK * CHUNK))
 
     def _sequence_state(self, dec_len):
         """Extra setup_caches arguments of models with per-sequence state: one entry per request, deep enough for rejecting
@@ -305,7 +309,7 @@ class SnapKVTargetBackend(_BackendBase):
                 is_last = True
             self._t.map_pages(i + 1, n)                       # pre_encode
             self.model.skip_head = i != num_chunks - 1
-            tokens = self.model.prefill(ids, self.cachelens, self._qo(n), self._t.table(), is_last=is_last,
+            tokens = self.model.prefill(ids, self.cachelens, self._qo(n), self._t.table((n, done + n)), is_last=is_last,
                                         draft_tab=self._d.table() if (self.is_spec and is_last) else None,
                                         ctx_len=done + n)
             self.cachelens += n
@@ -346,7 +350,7 @@ class SnapKVTargetBackend(_BackendBase):
             self._prefill_begin()
         while any(d < t.numel() for d, t in zip(done, ids)):
             live = [k for k, t in enumerate(ids) if done[k] < t.numel()]
-            portion = max(1, PREFILL_ROWS // len(live))
+            portion = max(1, max(PREFILL_ROWS, getattr(self.model, "prefill_rows", 0)) // len(live))
             take = {k: min(portion, ids[k].numel() - done[k]) for k in live}
             rows, row0 = [], 0                             # (entry, place | None = sampled only, flat row)
             for k in live:
@@ -389,7 +393,8 @@ class SnapKVTargetBackend(_BackendBase):
         # one upload for all the integers of the step
         flat = torch.tensor(pos + slots + pages + indptr + last + qo, dtype=torch.int32).to(dev)
         cut = torch.split(flat, [B, B, len(pages), B + 1, B, B + 1])
-        tab = PageTable(cut[2], cut[3], cut[4], max(indptr[i + 1] - indptr[i] for i in range(B)), slots=cut[1])
+        tab = PageTable(cut[2], cut[3], cut[4], max(indptr[i + 1] - indptr[i] for i in range(B)), slots=cut[1],
+                        lengths=(n, [p + k for p, k in zip(pos, n)]))
         ids = torch.cat([t for _, t in parts]).to(dev)
         self.model.skip_head = not head_rows
         rows = torch.tensor(head_rows, dtype=torch.long).to(dev) if head_rows else None
@@ -507,7 +512,7 @@ class SnapKVDraftBackend(_BackendBase):
                 is_last = True
             self._t.map_pages(i + 1, n)
             self.model.skip_head = i != num_chunks - 1
-            tokens = self.model.prefill(ids, self.cachelens, self._qo(n), self._t.table(), is_last=is_last,
+            tokens = self.model.prefill(ids, self.cachelens, self._qo(n), self._t.table((n, done + n)), is_last=is_last,
                                         draft_tab=self._d.table() if (self.is_compress and is_last) else None,
                                         ctx_len=done + n)
             self.cachelens += n

@@ -10,7 +10,7 @@ from __future__ import annotations
 import json
 from dataclasses import dataclass
 from pathlib import Path
-from typing import Optional, Tuple
+from typing import Optional, Tuple, Union
 
 
 @dataclass(frozen=True)
@@ -28,16 +28,58 @@ class AttentionSpec:
 
 
 @dataclass(frozen=True)
+class YarnSpec:
+    """YaRN scaling of rotary frequencies (ops.RotaryTable)."""
+    factor: float
+    original: float
+    fast: float
+    slow: float
+
+
+@dataclass(frozen=True)
+class RotarySpec:
+    """Rotary positions on neighbouring pairs of the first `dims` elements."""
+    dims: int
+    base: float
+    yarn: Optional[YarnSpec] = None
+
+
+@dataclass(frozen=True)
+class LatentAttentionSpec:
+    """Softmax attention whose keys and values are linear maps of one latent row per token, beside one rotated key part that all
+    heads share; queries come through a latent of their own (ops.LatentSpec holds the same numbers for the kernels)."""
+    heads: int
+    dim: int                      # unrotated query / key size per head
+    rot_dim: int                  # rotated query / key size per head
+    vdim: int
+    q_rank: int
+    kv_rank: int
+    scale: float
+    rotary: RotarySpec
+    gate: bool = False            # a head's output is multiplied by the sigmoid of its own logit
+    kv_from: Optional[int] = None   # layer whose cache rows this layer attends to; None: its own
+
+
+@dataclass(frozen=True)
 class MLPSpec:
     ff: int
-    act: str = "xielu"
+    act: str = "xielu"            # "xielu": down . act(up . h);  "gelu_gated": down . (gelu_tanh(gate . h) * (up . h))
+
+
+@dataclass(frozen=True)
+class BigramSpec:
+    """A second embedding, of the pair (token before, token): row (mul_before * before + mul_token * token) mod buckets."""
+    buckets: int
+    mul_before: int
+    mul_token: int
 
 
 @dataclass(frozen=True)
 class LayerSpec:
-    attention: AttentionSpec
+    attention: Union[AttentionSpec, LatentAttentionSpec]
     mlp: Optional[MLPSpec]
     token_shift: bool = False
+    parallel: bool = False        # mixer and feed-forward read one norm and are added together
 
 
 @dataclass(frozen=True)
@@ -50,6 +92,10 @@ class DecoderSpec:
     embed_scale: float = 1.0
     logit_scale: float = 1.0
     max_positions: int = 0        # learned position vectors; 0: none
+    bigram: Optional[BigramSpec] = None
+    embed_norm: bool = False      # weighted norm behind the embedding
+    tied_head: bool = False       # the embedding table is the output head
+    logit_softcap: Optional[float] = None
 
     @property
     def n_layer(self):
@@ -64,6 +110,9 @@ class _Reader:
             raise ValueError(f"config.json: {where} must be an object, got {obj!r}")
         self.obj, self.where, self.seen = obj, where, set()
 
+    def has(self, key):
+        return self.obj.get(key) is not None
+
     def get(self, key, kind=None):
         if key not in self.obj:
             raise ValueError(f"config.json: {self.where} has no '{key}'")
@@ -76,6 +125,10 @@ class _Reader:
                 raise ValueError(f"config.json: {self.where}.{key} must be a number, got {v!r}")
             v = float(v)
         return v
+
+    def skip(self, key):
+        """An optional key that may be present as null."""
+        self.seen.add(key)
 
     def sub(self, key):
         return _Reader(self.get(key), f"{self.where}.{key}")
@@ -125,7 +178,71 @@ def _furitar(cfg) -> DecoderSpec:
     return spec
 
 
-DESIGNS = {"Furitar": _furitar}
+def _rotary(r: _Reader) -> RotarySpec:
+    dims, base, yarn = r.get("dims", int), r.get("base", float), None
+    r.skip("scaling")
+    if r.has("scaling"):
+        s = r.sub("scaling")
+        yarn = YarnSpec(*(s.get(k, float) for k in ("factor", "original", "fast", "slow")))
+        s.done()
+    r.done()
+    if dims % 2:
+        raise ValueError(f"config.json: {r.where}.dims must be even, got {dims}")
+    return RotarySpec(dims, base, yarn)
+
+
+def _bufodra(cfg) -> DecoderSpec:
+    """Bufodra: parallel layers (latent attention beside a gated GELU feed-forward, one norm); of the two kinds of mixer one gates
+    its heads, the other may attend to an earlier layer's cache; a bigram embedding under a norm, a tied head, a logit soft cap."""
+    c = _Reader(cfg, "the model")
+    c.get("architecture")
+    norm, emb = c.sub("norm"), c.sub("embedding")
+    big = emb.sub("bigram")
+    bigram = BigramSpec(buckets=big.get("buckets", int), mul_before=big.get("mul_prev"), mul_token=big.get("mul_cur"))
+    if not all(isinstance(v, int) and not isinstance(v, bool) for v in (bigram.mul_before, bigram.mul_token)):
+        raise ValueError("config.json: the bigram's multipliers must be integers")
+    layers = []
+    for i, obj in enumerate(c.get("layers")):
+        L = _Reader(obj, f"layers[{i}]")
+        kind = L.get("type")
+        if kind not in ("latent_attention", "latent_attention_2"):
+            raise ValueError(f"config.json: layers[{i}]: unknown mixer {kind!r}")
+        m = L.sub("mixer")
+        m.skip("kv_from")
+        att = LatentAttentionSpec(heads=m.get("heads", int), dim=m.get("dim", int), rot_dim=m.get("rot_dim", int),
+                                  vdim=m.get("vdim", int), q_rank=m.get("q_rank", int), kv_rank=m.get("kv_rank", int),
+                                  scale=m.get("scale", float), rotary=_rotary(m.sub("rot")), gate=kind == "latent_attention",
+                                  kv_from=m.get("kv_from") if m.has("kv_from") else None)
+        m.done()
+        if att.rotary.dims > att.rot_dim:
+            raise ValueError(f"config.json: layers[{i}]: {att.rotary.dims} rotated dimensions of {att.rot_dim}")
+        if att.kv_from is not None:
+            src = layers[att.kv_from].attention if isinstance(att.kv_from, int) and 0 <= att.kv_from < i else None
+            if src is None or src.kv_from is not None or (src.kv_rank, src.rot_dim, src.rotary) != (att.kv_rank, att.rot_dim, att.rotary):
+                raise ValueError(f"config.json: layers[{i}]: kv_from must name an earlier layer with a cache of its own and the same "
+                                 "kv_rank, rot_dim and rotation")
+        mlp = None
+        if L.get("mlp") is not None:
+            f = L.sub("mlp")
+            if f.get("kind") != "dense":
+                raise ValueError(f"config.json: layers[{i}]: unknown feed-forward {f.obj['kind']!r}")
+            mlp = MLPSpec(ff=f.get("ff", int), act="gelu_gated")
+            f.done()
+        L.done()
+        layers.append(LayerSpec(attention=att, mlp=mlp, parallel=True))
+    spec = DecoderSpec(design="Bufodra", vocab_size=c.get("vocab", int), dim=c.get("width", int), norm_eps=norm.get("eps", float),
+                       layers=tuple(layers), bigram=bigram, embed_norm=True, tied_head=True,
+                       logit_softcap=c.get("logit_softcap", float))
+    for r in (norm, big, emb, c):
+        r.done()
+    if not layers:
+        raise ValueError("config.json: the model has no layers")
+    if not spec.logit_softcap > 0:
+        raise ValueError("config.json: logit_softcap must be positive")
+    return spec
+
+
+DESIGNS = {"Furitar": _furitar, "Bufodra": _bufodra}
 
 
 def spec_from_config(cfg) -> DecoderSpec:
@@ -143,11 +260,27 @@ def _furitar_config(vocab, width, n_layer, heads, kv_heads, dim, vdim, ff, chunk
             "logit_scale": 1.0, "max_positions": max_positions, "layers": [layer] * n_layer}
 
 
+def _bufodra_config(vocab, width, n_layer, heads, dim, rot_dim, vdim, q_rank, kv_rank, ff, original=4096):
+    """Pairs of a gated layer and a YaRN layer; every second YaRN layer attends to the cache of the one before it."""
+    def layer(i):
+        mixer = {"heads": heads, "dim": dim, "rot_dim": rot_dim, "vdim": vdim, "q_rank": q_rank, "kv_rank": kv_rank,
+                 "scale": (dim + rot_dim) ** -0.5, "rot": {"base": 10000.0, "dims": rot_dim}}
+        if i % 2:
+            mixer["rot"] = dict(mixer["rot"], scaling={"factor": 8.0, "original": original, "fast": 32.0, "slow": 1.0})
+            if i % 4 == 3:
+                mixer["kv_from"] = i - 2
+        return {"type": "latent_attention_2" if i % 2 else "latent_attention", "mixer": mixer, "mlp": {"kind": "dense", "ff": ff}}
+    return {"architecture": "Bufodra", "vocab": vocab, "width": width, "norm": {"eps": 1e-5}, "logit_softcap": 30.0,
+            "embedding": {"bigram": {"buckets": 65536, "mul_prev": 31337, "mul_cur": 7919}}, "layers": [layer(i) for i in range(n_layer)]}
+
+
 # named configurations of the designs (random weights where no checkpoint exists): the widths of the model zoo's
 # Llama-3.2-1B and Llama-3.1-8B, so that the two families can be measured side by side
 design_configs = {
     "furitar-1b": _furitar_config(128256, 2048, 16, 32, 8, 64, 64, 8192, 8192, 32768),
     "furitar-8b": _furitar_config(128256, 4096, 32, 32, 8, 128, 128, 14336, 8192, 32768),
+    "bufodra-1b": _bufodra_config(128256, 2048, 16, 16, 128, 64, 128, 768, 512, 5632),
+    "bufodra-8b": _bufodra_config(128256, 4096, 32, 32, 128, 64, 128, 1536, 512, 12288),
 }
 
 

@@ -245,6 +245,7 @@ class PageTable:
     last_page_len: torch.Tensor
     max_pages: int  # host upper bound of pages per request
     slots: Optional[torch.Tensor] = None   # entry of request b in per-sequence state (int32); None: b
+    lengths: Optional[tuple] = None   # host lists (new rows, positions after the step) per request, where known and worth telling
 
 
 class Transformer(nn.Module):
@@ -460,7 +461,7 @@ class Transformer(nn.Module):
         N, K = w.shape
         int8 = w.dtype == torch.int8
         if self.decode_rows is None or _MODE != "auto" or int8:
-            return want_packed(N, K, role == "w13", int8)
+            return want_packed(N, K, role in ("w13", "gated"), int8)
         if _PACKED == "0" or K % 64:
             return False
         return any(self._decode_hows(role, N, K, int8, M) - {"lib"} for M in self.decode_rows if M <= 256)

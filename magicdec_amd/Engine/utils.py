@@ -178,7 +178,9 @@ def _load_design(spec, checkpoint_path, device, precision, use_tp, seed=1234):
     else:
         print(f"[magicdec_amd] {weights} not found: seeded random weights for this {spec.design} configuration")
         _design_weights_(model, seed, device, precision)
-    return model.requires_grad_(False).to(device=device, dtype=precision).eval()
+    model = model.requires_grad_(False).to(device=device, dtype=precision).eval()
+    model.tie_weights()
+    return model
 
 
 def _load(transformer_cls, checkpoint_path, device, precision, use_tp, rank_group, group, seed=1234, is_draft=False):

@@ -12,7 +12,7 @@ from ctypes import c_char_p, c_double, c_float, c_int, c_int64, c_size_t, c_void
 _HERE = os.path.dirname(os.path.abspath(__file__))
 # MAGICDEC_HIP_LIB: development only -- another build of the same sources (e.g. `make TIMING=1`'s instrumented library)
 LIB_PATH = os.environ.get("MAGICDEC_HIP_LIB") or os.path.join(_HERE, "libmagicdec_hip.so")
-ABI_VERSION = 11
+ABI_VERSION = 12
 
 _lib = None
 _err = None
@@ -48,6 +48,23 @@ class XattnArgs(ctypes.Structure):
                 ("score_bound", c_float), ("B", I), ("n_max", I), ("H", I), ("KH", I), ("D", I), ("DV", I),
                 ("page_size", I), ("max_pages", I), ("chunk", I), ("sink", I), ("qk_norm", I), ("dtype", I),
                 ("force_plain", I)]
+
+
+class LatentArgs(ctypes.Structure):
+    """md_latent_args of include/magicdec_hip.h."""
+    _fields_ = [("z", P), ("dq_norm", P), ("kv_norm", P), ("cq", P), ("cache", P), ("cos_sin", P), ("qo_indptr", P), ("pos0", P),
+                ("page_indices", P), ("page_indptr", P), ("ctx_indptr", P), ("q", P), ("kv", P), ("gate", P), ("out", P),
+                ("workspace", P), ("workspace_bytes", c_size_t), ("ldz", L), ("ldo", L), ("ld_gate", L), ("eps", c_float),
+                ("scale", c_float), ("B", I), ("n_max", I), ("H", I), ("dim", I), ("rot_dim", I), ("rot_pairs", I), ("vdim", I),
+                ("q_rank", I), ("kv_rank", I), ("page_size", I), ("max_pages", I), ("max_pos", I), ("append", I), ("dtype", I),
+                ("force_plain", I)]
+
+
+class HeadLinearArgs(ctypes.Structure):
+    """md_head_linear_args of include/magicdec_hip.h."""
+    _fields_ = [("x", P), ("w", P), ("out", P), ("gate", P), ("tail", P), ("cos_sin", P), ("qo_indptr", P), ("pos0", P),
+                ("ldx", L), ("hx", L), ("ldo", L), ("ho", L), ("ld_gate", L), ("ldt", L), ("ht", L), ("M", I), ("H", I), ("N", I),
+                ("K", I), ("B", I), ("tail_dim", I), ("tail_pad", I), ("rot_pairs", I), ("max_pos", I), ("dtype", I)]
 
 
 _SIGNATURES = {
@@ -109,6 +126,17 @@ _SIGNATURES = {
     "md_xattn_workspace_bytes": (c_size_t, [ctypes.POINTER(XattnArgs)]),
     "md_qk_norm_append": (c_int, [ctypes.POINTER(XattnArgs), P, P]),
     "md_xattn": (c_int, [ctypes.POINTER(XattnArgs), P]),
+    "md_latent_row_width": (c_int, [I, I]),
+    "md_latent_append": (c_int, [ctypes.POINTER(LatentArgs), P]),
+    "md_latent_workspace_bytes": (c_size_t, [ctypes.POINTER(LatentArgs)]),
+    "md_latent_attn": (c_int, [ctypes.POINTER(LatentArgs), P]),
+    "md_latent_gather": (c_int, [ctypes.POINTER(LatentArgs), I, P, P]),
+    "md_latent_prefill_supported": (c_int, [ctypes.POINTER(LatentArgs)]),
+    "md_latent_prefill": (c_int, [ctypes.POINTER(LatentArgs), P]),
+    "md_head_linear": (c_int, [ctypes.POINTER(HeadLinearArgs), P]),
+    "md_embed_bigram": (c_int, [P, P, P, P, I, P, P, I, I, I, I, I, L, L, P, P, P, I, c_float, P, P]),
+    "md_gelu_mul": (c_int, [P, P, L, L, P, L, I, I, I, P]),
+    "md_softcap": (c_int, [P, L, c_float, I, I, I, P]),
     "md_argmax": (c_int, [P, L, I, I, L, P, P, P]),
     "md_argmax_f32": (c_int, [P, L, I, I, P, P]),
     "md_argmax_tp_slots": (c_int, [P, L, I, I, L, I, I, P, P, P]),

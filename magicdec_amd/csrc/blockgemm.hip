@@ -49,7 +49,7 @@ constexpr int kStageB = BN * BK * 2;            // 16 KiB: [4 column tiles][4 k-
 constexpr int kEpiPitch = BN + 4;               // fp32 epilogue tile [256][132]: 135 168 B inside the rings
 constexpr int lds_bytes(int XS, int WS) { return XS * kStageA + WS * kStageB; }
 
-enum { BE_NONE = 0, BE_SWIGLU = 1, BE_XIELU = 2 };
+enum { BE_NONE = 0, BE_SWIGLU = 1, BE_XIELU = 2, BE_GEGLU = 3 };   // BE_GEGLU: BE_SWIGLU's kernels with p.gelu
 
 struct BlockParams {
     const bf16_t* x;
@@ -60,6 +60,7 @@ struct BlockParams {
     float* partial;         // split: [S][M][N] fp32, GEMM-column order ([w1; w3] for BE_SWIGLU)
     int64_t ldx, ldo;
     int M, N, K, S, nsteps;     // nsteps = K / 64
+    int gelu;                   // BE_SWIGLU: GELU (tanh form), fp32 up to the product's one rounding, instead of SiLU
     unsigned int x_bytes;       // bytes of x a row index may address: rows >= M read zeros through the buffer bound
 };
 
@@ -289,8 +290,10 @@ __global__ __launch_bounds__(512) void block_gemm_kernel(const BlockParams p) {
             bf16x8 o;
 #pragma unroll
             for (int e = 0; e < 4; ++e) {
-                o[e] = f32_to_bf16(silu_bf16(bf16_to_f32(f32_to_bf16(h1a[e]))) * bf16_to_f32(f32_to_bf16(h3a[e])));
-                o[4 + e] = f32_to_bf16(silu_bf16(bf16_to_f32(f32_to_bf16(h1b[e]))) * bf16_to_f32(f32_to_bf16(h3b[e])));
+                o[e] = f32_to_bf16(p.gelu ? gelu_tanh(h1a[e]) * h3a[e]
+                                          : silu_bf16(bf16_to_f32(f32_to_bf16(h1a[e]))) * bf16_to_f32(f32_to_bf16(h3a[e])));
+                o[4 + e] = f32_to_bf16(p.gelu ? gelu_tanh(h1b[e]) * h3b[e]
+                                              : silu_bf16(bf16_to_f32(f32_to_bf16(h1b[e]))) * bf16_to_f32(f32_to_bf16(h3b[e])));
             }
             *reinterpret_cast<bf16x8*>(p.out + (int64_t)row * p.ldo + (tn * 4 + t) * 16 + i8) = o;
         }
@@ -384,6 +387,7 @@ int setup(BlockParams& p, const void* x, int64_t ldx, const void* w, int M, int 
     p.w = (const bf16_t*)w;
     p.bias = nullptr;
     p.act = nullptr;
+    p.gelu = 0;
     p.out = nullptr;
     p.ldx = ldx;
     p.ldo = 0;
@@ -414,7 +418,7 @@ extern "C" void md_debug_set_block_gemm(int target_blocks, int weights_nontempor
 
 extern "C" int md_linear_block_supported(int M, int N, int K, int epilogue) {
     if (!shape_ok(M, N, K)) return 0;
-    return (epilogue == BE_NONE || epilogue == BE_SWIGLU) ? 1 : 0;
+    return (epilogue == BE_NONE || epilogue == BE_SWIGLU || epilogue == BE_GEGLU) ? 1 : 0;
 }
 
 extern "C" size_t md_linear_block_workspace_bytes(int M, int N, int K, int force_split) {
@@ -427,8 +431,9 @@ extern "C" int md_linear_block(const void* x, int64_t ldx, const void* w_packed,
                                int M, int N, int K, int epilogue, void* workspace, size_t workspace_bytes,
                                md_stream_t stream) {
     MD_CHECK_ARG(out && (((uintptr_t)out) & 15) == 0 && ldo % 8 == 0, "md_linear_block: out must be 16-byte aligned, ldo %% 8 == 0");
-    MD_CHECK_ARG(epilogue == BE_NONE || epilogue == BE_SWIGLU, "md_linear_block: unknown epilogue %d", epilogue);
-    MD_CHECK_ARG(!(epilogue == BE_SWIGLU && bias), "md_linear_block: the SwiGLU epilogue takes no bias");
+    const bool gated = epilogue == BE_SWIGLU || epilogue == BE_GEGLU;
+    MD_CHECK_ARG(epilogue == BE_NONE || gated, "md_linear_block: unknown epilogue %d", epilogue);
+    MD_CHECK_ARG(!(gated && bias), "md_linear_block: the gated epilogues take no bias");
     MD_CHECK_ARG(!bias || (((uintptr_t)bias) & 15) == 0, "md_linear_block: bias must be 16-byte aligned (read as bf16x8)");
     BlockParams p;
     int rc = setup(p, x, ldx, w_packed, M, N, K, false, workspace, workspace_bytes, "md_linear_block");
@@ -438,7 +443,8 @@ extern "C" int md_linear_block(const void* x, int64_t ldx, const void* w_packed,
     p.bias = p.S > 1 ? nullptr : (const bf16_t*)bias;
     hipStream_t st = (hipStream_t)stream;
     const int grid = (N / BN) * p.S;
-    rc = epilogue == BE_SWIGLU ? launch_epi<BE_SWIGLU>(p, grid, st) : launch_epi<BE_NONE>(p, grid, st);
+    p.gelu = epilogue == BE_GEGLU;
+    rc = gated ? launch_epi<BE_SWIGLU>(p, grid, st) : launch_epi<BE_NONE>(p, grid, st);
     if (rc != MD_OK) return rc;
     if (p.S > 1) {
         rc = md_internal_launch_skinny_reduce(p.partial, p.S, M, N, epilogue, bias, out, ldo, st);

@@ -194,6 +194,56 @@ __global__ __launch_bounds__(256) void xielu_kernel(const T* __restrict__ z, int
     }
 }
 
+template <typename T, int VEC>
+struct RowPiece {
+    typedef T vec __attribute__((ext_vector_type(VEC)));
+    static __device__ __forceinline__ void load(const T* p, float (&f)[VEC]) {
+        const vec v = *reinterpret_cast<const vec*>(p);
+#pragma unroll
+        for (int e = 0; e < VEC; ++e) f[e] = (float)v[e];
+    }
+    static __device__ __forceinline__ void store(T* p, const float (&f)[VEC]) {
+        vec v;
+#pragma unroll
+        for (int e = 0; e < VEC; ++e) v[e] = (T)f[e];
+        *reinterpret_cast<vec*>(p) = v;
+    }
+};
+
+// y = gelu(a) * b in fp32, one rounding
+template <typename T, int VEC>
+__global__ __launch_bounds__(256) void gelu_mul_kernel(const T* __restrict__ a, const T* __restrict__ b, int64_t as, int64_t bs,
+                                                       T* y, int64_t ys, int rows, int dim) {
+    const int nvec = dim / VEC;
+    const int64_t total = (int64_t)rows * nvec;
+    for (int64_t i = (int64_t)blockIdx.x * blockDim.x + threadIdx.x; i < total; i += (int64_t)gridDim.x * blockDim.x) {
+        const int64_t row = i / nvec;
+        const int c = (int)(i - row * nvec) * VEC;
+        float f[VEC], g[VEC];
+        RowPiece<T, VEC>::load(a + row * as + c, f);
+        RowPiece<T, VEC>::load(b + row * bs + c, g);
+#pragma unroll
+        for (int e = 0; e < VEC; ++e) f[e] = gelu_tanh(f[e]) * g[e];
+        RowPiece<T, VEC>::store(y + row * ys + c, f);
+    }
+}
+
+// z = cap * tanh(z / cap), in place
+template <typename T, int VEC>
+__global__ __launch_bounds__(256) void softcap_kernel(T* z, int64_t zs, float cap, int rows, int dim) {
+    const int nvec = dim / VEC;
+    const int64_t total = (int64_t)rows * nvec;
+    for (int64_t i = (int64_t)blockIdx.x * blockDim.x + threadIdx.x; i < total; i += (int64_t)gridDim.x * blockDim.x) {
+        const int64_t row = i / nvec;
+        const int c = (int)(i - row * nvec) * VEC;
+        float f[VEC];
+        RowPiece<T, VEC>::load(z + row * zs + c, f);
+#pragma unroll
+        for (int e = 0; e < VEC; ++e) f[e] = cap * tanhf(f[e] / cap);
+        RowPiece<T, VEC>::store(z + row * zs + c, f);
+    }
+}
+
 // one workgroup of NT threads per row; lowest index among equal maxima.  Decode steps have few rows (64..256) of a
 // 128K vocabulary: with NT = 1024 (16 waves, 4 loads in flight each) a row is limited by its CU's load issue rate
 // instead of by one wave's memory latency (49 -> ~15 us for 64 rows)
@@ -366,6 +416,42 @@ extern "C" int md_xielu(const void* z, int64_t z_row_stride, const float* act, v
         else hipLaunchKernelGGL((xielu_kernel<bf16_t, 1>), dim3(grid), dim3(256), 0, st, (const bf16_t*)z, z_row_stride, act, (bf16_t*)y, rows, dim);
     }
     MD_CHECK_LAUNCH("md_xielu");
+    return MD_OK;
+}
+
+extern "C" int md_gelu_mul(const void* a, const void* b, int64_t a_row_stride, int64_t b_row_stride, void* y, int64_t y_row_stride,
+                           int rows, int dim, int dtype, md_stream_t stream) {
+    MD_CHECK_ARG(a && b && y, "md_gelu_mul: null pointer argument");
+    MD_CHECK_ARG(rows > 0 && dim > 0 && a_row_stride >= dim && b_row_stride >= dim && y_row_stride >= dim,
+                 "md_gelu_mul: bad shape rows=%d dim=%d", rows, dim);
+    MD_CHECK_ARG(dtype == MD_T_BF16 || dtype == MD_T_F32, "md_gelu_mul: dtype must be MD_T_BF16 or MD_T_F32");
+    const bool vec = dim % 8 == 0 && (a_row_stride | b_row_stride | y_row_stride) % 8 == 0 &&
+                     (((uintptr_t)a | (uintptr_t)b | (uintptr_t)y) & 15) == 0;
+    const int64_t total = (int64_t)rows * (vec ? dim / (dtype == MD_T_F32 ? 4 : 8) : dim);
+    const int grid = (int)(total + 255 > 4096 * 256 ? 4096 : (total + 255) / 256);
+    hipStream_t st = (hipStream_t)stream;
+#define MD_GM(T, V) hipLaunchKernelGGL((gelu_mul_kernel<T, V>), dim3(grid), dim3(256), 0, st, (const T*)a, (const T*)b, \
+                                       a_row_stride, b_row_stride, (T*)y, y_row_stride, rows, dim)
+    if (dtype == MD_T_F32) { if (vec) MD_GM(float, 4); else MD_GM(float, 1); }
+    else { if (vec) MD_GM(bf16_t, 8); else MD_GM(bf16_t, 1); }
+#undef MD_GM
+    MD_CHECK_LAUNCH("md_gelu_mul");
+    return MD_OK;
+}
+
+extern "C" int md_softcap(void* z, int64_t z_row_stride, float cap, int rows, int dim, int dtype, md_stream_t stream) {
+    MD_CHECK_ARG(z, "md_softcap: null pointer argument");
+    MD_CHECK_ARG(rows > 0 && dim > 0 && z_row_stride >= dim && cap != 0.f, "md_softcap: bad shape rows=%d dim=%d or cap", rows, dim);
+    MD_CHECK_ARG(dtype == MD_T_BF16 || dtype == MD_T_F32, "md_softcap: dtype must be MD_T_BF16 or MD_T_F32");
+    const bool vec = dim % 8 == 0 && z_row_stride % 8 == 0 && ((uintptr_t)z & 15) == 0;
+    const int64_t total = (int64_t)rows * (vec ? dim / (dtype == MD_T_F32 ? 4 : 8) : dim);
+    const int grid = (int)(total + 255 > 4096 * 256 ? 4096 : (total + 255) / 256);
+    hipStream_t st = (hipStream_t)stream;
+#define MD_SC(T, V) hipLaunchKernelGGL((softcap_kernel<T, V>), dim3(grid), dim3(256), 0, st, (T*)z, z_row_stride, cap, rows, dim)
+    if (dtype == MD_T_F32) { if (vec) MD_SC(float, 4); else MD_SC(float, 1); }
+    else { if (vec) MD_SC(bf16_t, 8); else MD_SC(bf16_t, 1); }
+#undef MD_SC
+    MD_CHECK_LAUNCH("md_softcap");
     return MD_OK;
 }
 

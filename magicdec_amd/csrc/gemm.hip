@@ -36,7 +36,7 @@ constexpr int kSlabK = 128;                 // k depth of one LDS activation sla
 constexpr int kStepsPerSlab = kSlabK / 16;  // 8 MFMA k-steps (32x32x16) per slab
 constexpr int kPitch = kSlabK * 2 + 16;     // LDS row pitch in bytes (272: rows start 4 banks apart)
 
-enum { EPI_NONE = 0, EPI_SWIGLU = 1, EPI_XIELU = 2 };
+enum { EPI_NONE = 0, EPI_SWIGLU = 1, EPI_XIELU = 2, EPI_GEGLU = 3 };   // EPI_GEGLU: EPI_SWIGLU's kernels with p.gelu
 
 struct GemmParams {
     const bf16_t* x;      // [M][K], row stride ldx (elements)
@@ -55,6 +55,7 @@ struct GemmParams {
     float pro_eps;
     int pro_tiles;
     const float* act;     // EPI_XIELU: the two numbers of the activation
+    int gelu;             // EPI_SWIGLU: GELU (tanh form), fp32 up to the one rounding of the product, instead of SiLU
 };
 
 __device__ __forceinline__ f32x2 unpack2(unsigned int v) {          // the two bf16 of a dword as fp32 (low half first)
@@ -334,10 +335,10 @@ __global__ __launch_bounds__(64 * NW) void skinny_gemm_kernel(const GemmParams p
             const int row = mt * 32 + (r & 3) + 8 * (r >> 2) + 4 * kh;
             float v = acc[mt][r];
             if constexpr (EPI == EPI_SWIGLU) {
-                float h = bf16_to_f32(f32_to_bf16(v));
+                float h = p.gelu ? v : bf16_to_f32(f32_to_bf16(v));
                 if (W8) h = bf16_to_f32(f32_to_bf16(h * bf16_to_f32(p.scales[col])));
                 const float h3 = __shfl_xor(h, 16);                 // lanes j and j^16 hold w1 / w3 of one column
-                v = silu_bf16(h) * h3;
+                v = (p.gelu ? gelu_tanh(h) : silu_bf16(h)) * h3;
             } else if constexpr (EPI == EPI_XIELU) {
                 v = Xielu(p.act)(v);
             } else {
@@ -383,12 +384,12 @@ __global__ __launch_bounds__(256) void skinny_reduce_kernel(const GemmParams p) 
     for (int e = 0; e < 4; ++e) {
         float v = a[e];
         if constexpr (EPI == EPI_SWIGLU) {
-            float h1 = bf16_to_f32(f32_to_bf16(v)), h3 = bf16_to_f32(f32_to_bf16(b3[e]));
+            float h1 = p.gelu ? v : bf16_to_f32(f32_to_bf16(v)), h3 = p.gelu ? b3[e] : bf16_to_f32(f32_to_bf16(b3[e]));
             if (W8) {
                 h1 = bf16_to_f32(f32_to_bf16(h1 * bf16_to_f32(p.scales[c0 + e])));
                 h3 = bf16_to_f32(f32_to_bf16(h3 * bf16_to_f32(p.scales[(p.N >> 1) + c0 + e])));
             }
-            v = silu_bf16(h1) * h3;
+            v = (p.gelu ? gelu_tanh(h1) : silu_bf16(h1)) * h3;
         } else if constexpr (EPI == EPI_XIELU) {
             v = Xielu(p.act)(v);
         } else {
@@ -525,7 +526,8 @@ int launch_mt(const GemmParams& p, int nw, int n_blocks, hipStream_t st) {
 }
 
 bool nw_allowed(int M, bool w8) { return !w8 && M <= 128; }
-int wave_tiles(int N, int epilogue) { return epilogue == EPI_SWIGLU ? ((N >> 1) + 15) / 16 : (N + 31) / 32; }
+bool is_gated(int epilogue) { return epilogue == EPI_SWIGLU || epilogue == EPI_GEGLU; }
+int wave_tiles(int N, int epilogue) { return is_gated(epilogue) ? ((N >> 1) + 15) / 16 : (N + 31) / 32; }
 
 }  // namespace
 
@@ -538,14 +540,15 @@ int md_internal_launch_skinny_reduce(const float* partial, int S, int M, int N, 
     p.S = S;
     p.M = M;
     p.N = N;
-    p.Nout = epilogue == EPI_SWIGLU ? N / 2 : N;
+    p.Nout = is_gated(epilogue) ? N / 2 : N;
+    p.gelu = epilogue == EPI_GEGLU;
     p.bias = epilogue == EPI_XIELU ? nullptr : (const bf16_t*)bias;
     p.act = epilogue == EPI_XIELU ? (const float*)bias : nullptr;
     p.out = (bf16_t*)out;
     p.ldo = ldo;
     const int64_t threads = (int64_t)M * (p.Nout / 4);
     const dim3 grid((unsigned)((threads + 255) / 256));
-    if (epilogue == EPI_SWIGLU)
+    if (is_gated(epilogue))
         hipLaunchKernelGGL((skinny_reduce_kernel<EPI_SWIGLU, false>), grid, dim3(256), 0, st, p);
     else if (epilogue == EPI_XIELU)
         hipLaunchKernelGGL((skinny_reduce_kernel<EPI_XIELU, false>), grid, dim3(256), 0, st, p);
@@ -568,7 +571,7 @@ extern "C" size_t md_linear_workspace_bytes(int M, int N, int K, int epilogue) {
 
 extern "C" int md_linear_supported(int M, int N, int K, int epilogue) {
     if (M < 1 || M > 256 || K < kSlabK || K % kSlabK) return 0;
-    if (epilogue == EPI_SWIGLU) return (N % 32 == 0) ? 1 : 0;     // N = 2*I, I % 16 == 0
+    if (is_gated(epilogue)) return (N % 32 == 0) ? 1 : 0;     // N = 2*I, I % 16 == 0
     return (N % 4 == 0) ? 1 : 0;
 }
 
@@ -580,12 +583,12 @@ int linear_impl(const void* x, int64_t ldx, const void* w, int w_dtype, int w_pa
     MD_CHECK_ARG(x && w && out, "md_linear: null pointer argument");
     MD_CHECK_ARG(md_linear_supported(M, N, K, epilogue), "md_linear: unsupported shape M=%d N=%d K=%d epilogue=%d "
                  "(need 1 <= M <= 256, K %% 128 == 0, N %% 4 == 0)", M, N, K, epilogue);
-    MD_CHECK_ARG(epilogue == EPI_NONE || epilogue == EPI_SWIGLU || (epilogue == EPI_XIELU && act && !pro_ssq &&
+    MD_CHECK_ARG(epilogue == EPI_NONE || is_gated(epilogue) || (epilogue == EPI_XIELU && act && !pro_ssq &&
                                                                           w_dtype == MD_W_BF16 && !bias),
                  "md_linear: unknown epilogue %d", epilogue);
     MD_CHECK_ARG(w_dtype == MD_W_BF16 || (w_dtype == MD_W_INT8 && scales), "md_linear: w_dtype must be MD_W_BF16 or "
                  "MD_W_INT8 (with per-channel scales)");
-    MD_CHECK_ARG(!(epilogue == EPI_SWIGLU && bias), "md_linear: SwiGLU epilogue takes no bias");
+    MD_CHECK_ARG(!(is_gated(epilogue) && bias), "md_linear: gated epilogues take no bias");
     MD_CHECK_ARG((((uintptr_t)x | (uintptr_t)w | (uintptr_t)out) & 15) == 0 && ldx % 8 == 0 && ldo % 4 == 0,
                  "md_linear: x / w / out must be 16-byte aligned, ldx %% 8 == 0, ldo %% 4 == 0");
     GemmParams p = {};
@@ -599,7 +602,8 @@ int linear_impl(const void* x, int64_t ldx, const void* w, int w_dtype, int w_pa
     p.M = M;
     p.N = N;
     p.K = K;
-    p.Nout = epilogue == EPI_SWIGLU ? N / 2 : N;
+    p.Nout = is_gated(epilogue) ? N / 2 : N;
+    p.gelu = epilogue == EPI_GEGLU;
     p.packed = w_packed ? 1 : 0;
     p.skip_reduce = 0;
     p.act = act;
@@ -629,11 +633,11 @@ int linear_impl(const void* x, int64_t ldx, const void* w, int w_dtype, int w_pa
     hipStream_t st = (hipStream_t)stream;
     int rc;
     if (pro)
-        rc = epilogue == EPI_SWIGLU ? launch_mt<EPI_SWIGLU, false, true>(p, pl.nw, n_blocks, st)
+        rc = is_gated(epilogue) ? launch_mt<EPI_SWIGLU, false, true>(p, pl.nw, n_blocks, st)
                                     : launch_mt<EPI_NONE, false, true>(p, pl.nw, n_blocks, st);
     else if (epilogue == EPI_XIELU)
         rc = launch_mt<EPI_XIELU, false>(p, pl.nw, n_blocks, st);
-    else if (epilogue == EPI_SWIGLU)
+    else if (is_gated(epilogue))
         rc = w8 ? launch_mt<EPI_SWIGLU, true>(p, pl.nw, n_blocks, st) : launch_mt<EPI_SWIGLU, false>(p, pl.nw, n_blocks, st);
     else
         rc = w8 ? launch_mt<EPI_NONE, true>(p, pl.nw, n_blocks, st) : launch_mt<EPI_NONE, false>(p, pl.nw, n_blocks, st);

@@ -80,6 +80,11 @@ struct Xielu {
     }
 };
 
+// GELU in its tanh form, z / 2 (1 + tanh(sqrt(2/pi) (z + 0.044715 z^3))), written as z * sigmoid of twice the argument (fp32)
+__device__ __forceinline__ float gelu_tanh(float z) {
+    return z / (1.0f + expf(-1.5957691216057308f * fmaf(0.044715f * z * z, z, z)));
+}
+
 __device__ __forceinline__ float wave_reduce_sum(float v) {
 #pragma unroll
     for (int o = 32; o > 0; o >>= 1) v += __shfl_xor(v, o);

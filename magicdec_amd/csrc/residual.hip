@@ -2,12 +2,17 @@
 // weighted RMS norm + token shift between two sub-layers, in one launch.
 //
 //   md_embed_pos        x = float(E[token]) * scale + float(P[pos])                                     (fp32 rows)
+//   md_embed_bigram     x = rms(float(E[token]) + float(G[(a * before + b * token) % n])) * w            (fp32 rows)
 //   md_resid_norm       x += delta;  h = x / sqrt(mean(x^2) + eps) * w  (fp32);  y = h * out_scale  (rounded to the model dtype)
 //   md_resid_norm_shift the same with the token shift  y = h_t + (h_{t-1} - h_t) * mu  in front of the rounding
 //
 // `delta` is the output of the sub-layer's projection: model-dtype rows, or the S fp32 partial planes [S][rows][width] a
 // split-K GEMM left in its workspace (the add and the norm then ARE that GEMM's combine launch, and the projection reaches
 // the fp32 residual without a 16-bit rounding in between).
+//
+// Bigram embedding.  The token before a row is the step's own previous row, or -- first row of a portion -- comes from a token
+// history that is paged like a KV cache: position p of a sequence lies in its page p / page_size.  A row writes its own entry
+// only, so a step may be repeated, rolled back or continued in any portions without further state.
 //
 // Token shift.  h_{t-1} of a row is the previous row's own h: the workgroup recomputes it from x + delta of that row (x_out is
 // a different buffer from x, so no workgroup sees a half-updated residual), except for the first row of a portion, whose
@@ -281,6 +286,85 @@ void launch_embed(const int64_t* tokens, const void* table, const void* pos_tabl
                        qo_indptr, pos0, width, vocab, max_pos, scale, out);
 }
 
+struct BigramParams {
+    const int64_t* tokens;
+    const void* table;       // [vocab][width]
+    const void* pairs;       // [buckets + 1][width]; row `buckets`: a sequence's first token
+    const void* w;           // norm weight
+    const int32_t* qo_indptr;
+    const int32_t* pos0;
+    const int32_t* page_indices;
+    const int32_t* page_indptr;
+    int32_t* history;        // [pages][page_size]
+    float* out;
+    int64_t mul_before, mul_token;
+    int width, vocab, buckets, page_size;
+    float eps;
+};
+
+__device__ __forceinline__ int64_t clamp_token(int64_t t, int vocab) {   // the host refuses such ids; never index past the table
+    return t < 0 ? 0 : (t >= vocab ? vocab - 1 : t);
+}
+
+template <typename T, int VEC, int MAXV>
+__global__ __launch_bounds__(256) void embed_bigram_kernel(const BigramParams p) {
+    __shared__ float red[8];
+    const int b = blockIdx.y, j = blockIdx.x;
+    const int q0 = p.qo_indptr[b];
+    if (j >= p.qo_indptr[b + 1] - q0) return;
+    const int pos = p.pos0[b] + j, pg0 = p.page_indptr[b], cap = (p.page_indptr[b + 1] - pg0) * p.page_size;
+    const int64_t tok = clamp_token(p.tokens[q0 + j], p.vocab);
+    int64_t before = 0;
+    if (j > 0) before = clamp_token(p.tokens[q0 + j - 1], p.vocab);
+    else if (pos > 0 && pos - 1 < cap) before = p.history[(int64_t)p.page_indices[pg0 + (pos - 1) / p.page_size] * p.page_size + (pos - 1) % p.page_size];
+    if (threadIdx.x == 0) {
+        if (pos >= 0 && pos < cap) p.history[(int64_t)p.page_indices[pg0 + pos / p.page_size] * p.page_size + pos % p.page_size] = (int32_t)tok;
+    }
+    int64_t pair = pos <= 0 ? p.buckets : (before * p.mul_before + tok * p.mul_token) % p.buckets;
+    if (pair < 0) pair += p.buckets;
+    const int nvec = p.width / VEC;
+    float h[MAXV][VEC], ss = 0.f;
+#pragma unroll
+    for (int it = 0; it < MAXV; ++it) {
+        const int i = threadIdx.x + it * 256;
+        if (i < nvec) {
+            float g[VEC];
+            ld_vec<VEC>(reinterpret_cast<const T*>(p.table) + tok * p.width + i * VEC, h[it]);
+            ld_vec<VEC>(reinterpret_cast<const T*>(p.pairs) + pair * p.width + i * VEC, g);
+#pragma unroll
+            for (int e = 0; e < VEC; ++e) {
+                h[it][e] += g[e];
+                ss += h[it][e] * h[it][e];
+            }
+        }
+    }
+    const float rs = 1.0f / sqrtf(block_sum(ss, red) / (float)p.width + p.eps);
+#pragma unroll
+    for (int it = 0; it < MAXV; ++it) {
+        const int i = threadIdx.x + it * 256;
+        if (i < nvec) {
+            float w[VEC];
+            ld_vec<VEC>(reinterpret_cast<const T*>(p.w) + i * VEC, w);
+#pragma unroll
+            for (int e = 0; e < VEC; ++e) h[it][e] = (h[it][e] * rs) * w[e];
+            st_vec<VEC>(p.out + (int64_t)(q0 + j) * p.width + i * VEC, h[it]);
+        }
+    }
+}
+
+template <typename T>
+void launch_bigram(const BigramParams& p, bool vec, dim3 grid, hipStream_t st) {
+    const int trips = (p.width / (vec ? 8 : 1) + 255) / 256;
+    if (vec) {
+        if (trips <= 1) hipLaunchKernelGGL((embed_bigram_kernel<T, 8, 1>), grid, dim3(256), 0, st, p);
+        else if (trips <= 2) hipLaunchKernelGGL((embed_bigram_kernel<T, 8, 2>), grid, dim3(256), 0, st, p);
+        else hipLaunchKernelGGL((embed_bigram_kernel<T, 8, 4>), grid, dim3(256), 0, st, p);
+    } else {
+        if (trips <= 4) hipLaunchKernelGGL((embed_bigram_kernel<T, 1, 4>), grid, dim3(256), 0, st, p);
+        else hipLaunchKernelGGL((embed_bigram_kernel<T, 1, 32>), grid, dim3(256), 0, st, p);
+    }
+}
+
 bool aligned16(const void* q) { return ((uintptr_t)q & 15) == 0; }
 
 int resid_check(const char* who, const md_resid_norm_args* a) {
@@ -361,6 +445,24 @@ extern "C" int md_embed_pos(const int64_t* tokens, const void* table, const void
                                : (vec ? launch_embed<bf16_t, 8> : launch_embed<bf16_t, 1>);
     k(tokens, table, pos_table, qo_indptr, pos0, dim3(n_max, B), width, vocab, max_pos, scale, out, (hipStream_t)stream);
     MD_CHECK_LAUNCH("md_embed_pos");
+    return MD_OK;
+}
+
+extern "C" int md_embed_bigram(const int64_t* tokens, const void* table, const void* pairs, const void* norm_weight, int dtype,
+                               const int32_t* qo_indptr, const int32_t* pos0, int B, int n_max, int width, int vocab, int buckets,
+                               int64_t mul_before, int64_t mul_token, int32_t* history, const int32_t* page_indices,
+                               const int32_t* page_indptr, int page_size, float eps, float* out, md_stream_t stream) {
+    MD_CHECK_ARG(tokens && table && pairs && norm_weight && qo_indptr && pos0 && history && page_indices && page_indptr && out,
+                 "md_embed_bigram: null pointer argument");
+    MD_CHECK_ARG(B > 0 && B <= 65535 && n_max > 0 && width > 0 && width <= 8192 && vocab > 0 && buckets > 0 && page_size > 0,
+                 "md_embed_bigram: bad shape B=%d n_max=%d width=%d (<= 8192) buckets=%d", B, n_max, width, buckets);
+    MD_CHECK_ARG(dtype == MD_T_BF16 || dtype == MD_T_F32, "md_embed_bigram: dtype must be MD_T_BF16 or MD_T_F32");
+    BigramParams p = {tokens, table, pairs, norm_weight, qo_indptr, pos0, page_indices, page_indptr, history, out,
+                      mul_before, mul_token, width, vocab, buckets, page_size, eps};
+    const bool vec = width % 8 == 0 && aligned16(table) && aligned16(pairs) && aligned16(norm_weight) && aligned16(out);
+    if (dtype == MD_T_F32) launch_bigram<float>(p, vec, dim3(n_max, B), (hipStream_t)stream);
+    else launch_bigram<bf16_t>(p, vec, dim3(n_max, B), (hipStream_t)stream);
+    MD_CHECK_LAUNCH("md_embed_bigram");
     return MD_OK;
 }
 

@@ -62,7 +62,8 @@ constexpr int kWaveLds = 32 * kPitch;    // wave-private activation image (8704 
 
 enum { FL_NONE = 0, FL_SWIGLU = 1, FL_RESID = 2, FL_ROPE_APPEND = 3,
        FL_XIELU = 4,
-       FL_PARTIAL = 5 };      // internal: the K range is ALSO split over workgroups; fp32 partial tiles -> workspace
+       FL_GEGLU = 5,           // FL_SWIGLU's kernels with p.gelu
+       FL_PARTIAL = 6 };      // internal: the K range is ALSO split over workgroups; fp32 partial tiles -> workspace
 
 struct KvTable {
     void* cache;
@@ -87,6 +88,7 @@ struct TileParams {
     const float* k_scale;
     const float* v_scale;
     const float* act;         // XIELU: the two numbers of the activation
+    int gelu;                 // SWIGLU: GELU (tanh form), fp32 up to the product's one rounding, instead of SiLU
     unsigned int* overflow;   // dropped-row counter (md_page_overflow_count)
     // deferred RMSNorm (see the kernel header): producer side (RESID) / consumer side (PRO)
     float* ssq_out;           // RESID: [M][n_tiles] sum of squares of the tile's 32 output columns per row, or null
@@ -484,9 +486,9 @@ __global__ __launch_bounds__(64 * NW, MT * NT > 1 ? 2 : 4) void tile_gemm_kernel
         } else if constexpr (EPI == FL_SWIGLU) {
             const int I = p.N >> 1;
             const int i = tn * 16 + cp;
-            const float h1 = bf16_to_f32(f32_to_bf16(tile_sum1(cp)));
-            const float h3 = bf16_to_f32(f32_to_bf16(tile_sum1(16 + cp)));
-            if (gm < p.M && i < I) p.out[(int64_t)gm * p.ldo + i] = f32_to_bf16(silu_bf16(h1) * h3);
+            const float a1 = tile_sum1(cp), a3 = tile_sum1(16 + cp);
+            const float v = p.gelu ? gelu_tanh(a1) * a3 : silu_bf16(bf16_to_f32(f32_to_bf16(a1))) * bf16_to_f32(f32_to_bf16(a3));
+            if (gm < p.M && i < I) p.out[(int64_t)gm * p.ldo + i] = f32_to_bf16(v);
             continue;
         } else {
             const int n = tn * 32 + 2 * cp;
@@ -794,7 +796,7 @@ extern "C" void md_debug_set_fused_nw(int nw) {
 
 extern "C" int md_linear_fused_supported(int M, int N, int K, int epilogue) {
     if (M < 1 || M > 256 || K < 128 || K % 128 || N < 32 || N % 32) return 0;
-    return (epilogue >= FL_NONE && epilogue <= FL_XIELU) ? 1 : 0;
+    return (epilogue >= FL_NONE && epilogue <= FL_GEGLU) ? 1 : 0;
 }
 
 extern "C" int md_linear_fused(const md_fused_linear_args* a, md_stream_t stream) {
@@ -804,7 +806,8 @@ extern "C" int md_linear_fused(const md_fused_linear_args* a, md_stream_t stream
                  "N %% 32 == 0)", a->M, a->N, a->K, a->epilogue);
     MD_CHECK_ARG(aligned16(a->x) && aligned16(a->w_packed) && aligned16(a->out) && a->ldx % 8 == 0 && a->ldo % 2 == 0,
                  "md_linear_fused: x / w / out must be 16-byte aligned, ldx %% 8 == 0, ldo %% 2 == 0");
-    MD_CHECK_ARG(!(a->epilogue == FL_SWIGLU && a->bias), "md_linear_fused: the SwiGLU epilogue takes no bias");
+    const bool gated = a->epilogue == FL_SWIGLU || a->epilogue == FL_GEGLU;
+    MD_CHECK_ARG(!(gated && a->bias), "md_linear_fused: the gated epilogues take no bias");
     // the kernel addresses x with 32-bit byte offsets from a scalar base
     MD_CHECK_ARG(a->ldx > 0 && ((int64_t)(a->M - 1) * a->ldx + a->K) * 2 < ((int64_t)1 << 32),
                  "md_linear_fused: x spans more than 4 GiB (M=%d, ldx=%lld): pass a compact activation tensor", a->M,
@@ -822,7 +825,7 @@ extern "C" int md_linear_fused(const md_fused_linear_args* a, md_stream_t stream
     p.n_tiles = a->N / 32;
     p.m_tiles = (a->M + 31) / 32;
     if (a->pro_ssq) {
-        MD_CHECK_ARG(a->epilogue == FL_SWIGLU || a->epilogue == FL_ROPE_APPEND,
+        MD_CHECK_ARG(gated || a->epilogue == FL_ROPE_APPEND,
                      "md_linear_fused: the deferred-RMSNorm prologue exists for the qkv and w1|w3 linears");
         MD_CHECK_ARG(a->pro_norm_w && a->pro_tiles > 0 && aligned16(a->pro_norm_w),
                      "md_linear_fused: the deferred-RMSNorm prologue needs the norm weight (16-byte aligned) and pro_tiles");
@@ -842,6 +845,9 @@ extern "C" int md_linear_fused(const md_fused_linear_args* a, md_stream_t stream
     case FL_NONE:
         rc = launch_tile<FL_NONE, false>(p, st);
         break;
+    case FL_GEGLU:
+        p.gelu = 1;
+        [[fallthrough]];
     case FL_SWIGLU:
         rc = launch_tile<FL_SWIGLU, false>(p, st);
         break;

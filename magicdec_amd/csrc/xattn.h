@@ -18,10 +18,14 @@ struct XattnParams {
     float* ws;                // split-KV partials
     unsigned int* overflow;
     int B, n_max, H, KH, g, D, DV, DKp, DVp, page_size;
+    int ldk, ldv;             // plain kernel: elements between rows of a page
     int chunk;                // > 0; 0x7fffffff: no chunk mask
     int sink, qk_norm, nsplit, n_qgroups, rows_cap;
     float eps, scale, scale_log2, ref_log2;   // ref_log2: the fixed softmax reference of the matrix-core kernels, log2 units
 };
+
+// the plain kernel of xattn.hip (16- or 32-bit pages): any head sizes up to 1024, online softmax in fp32
+int md_internal_xattn_plain(const XattnParams& p, int dtype, hipStream_t st);
 
 // one translation unit per padded query/key width; false: no kernel for (DKp, DVp)
 #define MD_XATTN_DECL(DK)                                                                                       \

@@ -156,7 +156,7 @@ __global__ __launch_bounds__(256) void xattn_plain_kernel(const XattnParams p) {
         if (kp <= hi) {
             const int page = p.page_indices[pg0 + kp / p.page_size];
             const T* k = reinterpret_cast<const T*>(p.k_cache) +
-                         (((int64_t)page * p.KH + kvh) * p.page_size + kp % p.page_size) * p.DKp;
+                         (((int64_t)page * p.KH + kvh) * p.page_size + kp % p.page_size) * p.ldk;
             s = dot_row<T>(k, sq, p.DKp) * p.scale;
             if (p.r1) s -= r1 * logf(1.0f + r2 * (float)(pos - kp));
         }
@@ -180,7 +180,7 @@ __global__ __launch_bounds__(256) void xattn_plain_kernel(const XattnParams p) {
             const int kq = base + k;
             const int page = p.page_indices[pg0 + kq / p.page_size];
             const T* vr = reinterpret_cast<const T*>(p.v_cache) +
-                          (((int64_t)page * p.KH + kvh) * p.page_size + kq % p.page_size) * p.DVp;
+                          (((int64_t)page * p.KH + kvh) * p.page_size + kq % p.page_size) * p.ldv;
             const float pk = sp[k];
             if (p.DVp < 256) {
                 acc[0] = fmaf(pk, (float)vr[vd], acc[0]);
@@ -288,6 +288,8 @@ XattnParams make_params(const md_xattn_args* a) {
     p.DV = a->DV;
     p.DKp = bucket(a->D);
     p.DVp = bucket(a->DV);
+    p.ldk = p.DKp;
+    p.ldv = p.DVp;
     p.page_size = a->page_size;
     p.chunk = a->chunk > 0 ? a->chunk : 0x7fffffff;
     p.sink = a->sink;
@@ -317,6 +319,16 @@ int check_args(const char* who, const md_xattn_args* a) {
 }
 
 }  // namespace
+
+int md_internal_xattn_plain(const XattnParams& p, int dtype, hipStream_t st) {
+    const dim3 grid(p.n_max, p.H, p.B);
+    if (dtype == MD_T_F32)
+        hipLaunchKernelGGL((xattn_plain_kernel<float>), grid, dim3(256), 0, st, p);
+    else
+        hipLaunchKernelGGL((xattn_plain_kernel<bf16_t>), grid, dim3(256), 0, st, p);
+    MD_CHECK_LAUNCH("attention(plain)");
+    return MD_OK;
+}
 
 extern "C" int md_xattn_head_pad(int head_size) { return head_size > 0 && bucket(head_size) <= kMaxHead ? bucket(head_size) : 0; }
 
@@ -380,13 +392,7 @@ extern "C" int md_xattn(const md_xattn_args* a, md_stream_t stream) {
     }
     if (!mfma_ok(a) || a->force_plain || (rows > 32 && nw == 0)) {
         MD_CHECK_ARG(!fused, "md_xattn: the plain kernel takes normalised queries");
-        const dim3 grid(a->n_max, a->H, a->B);
-        if (a->dtype == MD_T_F32)
-            hipLaunchKernelGGL((xattn_plain_kernel<float>), grid, dim3(256), 0, st, p);
-        else
-            hipLaunchKernelGGL((xattn_plain_kernel<bf16_t>), grid, dim3(256), 0, st, p);
-        MD_CHECK_LAUNCH("md_xattn(plain)");
-        return MD_OK;
+        return md_internal_xattn_plain(p, a->dtype, st);
     }
     int rc;
     if (rows <= 32) {

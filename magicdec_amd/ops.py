@@ -267,7 +267,7 @@ def streaming_rotate(kv_cache, rot_cache, B, valid_len, pages_per_req, table: Ro
 
 # ----------------------------------------------------------------------------- K8
 MD_W_BF16, MD_W_INT8 = 0, 1
-EPI_NONE, EPI_SWIGLU = 0, 1
+EPI_NONE, EPI_SWIGLU, EPI_GEGLU = 0, 1, 3
 
 
 def linear_supported(M, N, K, swiglu=False):
@@ -323,14 +323,15 @@ def _act_numbers(act):
 
 
 def linear(x, weight, bias=None, scales=None, swiglu=False, workspace: "AttnWorkspace" = None, out=None,
-           pro: "DeferredNorm" = None, xielu=None):
+           pro: "DeferredNorm" = None, xielu=None, gelu=False):
     """F.linear(x, weight, bias) for M = x.shape[0] <= 256 rows on the hand-written gfx950 skinny GEMM (md_linear).
     x [M, K] bf16 with unit inner stride (row stride free); weight: a contiguous [N, K] tensor or a PackedWeight
     (streaming layout), bf16 -- or int8 with bf16 per-row `scales` (WeightOnlyInt8Linear semantics:
     bf16(x.w^T) * scales).  swiglu=True: weight = [w1; w3] (N = 2*I rows) and the result is
     silu(x.w1^T) * (x.w3^T) [M, I] with the reference's bf16 rounding points.
     pro (bf16 weights): x is pro.h, the un-normalised hidden state, and is normalised on the fly (md_linear_normed).
-    xielu (bf16 weights): the two numbers of the activation applied to the result (md_linear_xielu)."""
+    xielu (bf16 weights): the two numbers of the activation applied to the result (md_linear_xielu).
+    gelu (with swiglu): gelu_tanh(h1) * h3 instead, fp32 up to the one rounding of the product."""
     packed = isinstance(weight, PackedWeight)
     wt = weight.data if packed else weight
     _gpu(x, wt, bias, scales)
@@ -355,7 +356,7 @@ def linear(x, weight, bias=None, scales=None, swiglu=False, workspace: "AttnWork
         wd = MD_W_BF16
     else:
         raise TypeError(f"linear: weight dtype {wt.dtype} unsupported (bf16 or int8)")
-    epi = EPI_SWIGLU if swiglu else EPI_NONE
+    epi = (EPI_GEGLU if gelu else EPI_SWIGLU) if swiglu else EPI_NONE
     n_out = N // 2 if swiglu else N
     if out is None:
         out = torch.empty((M, n_out), dtype=x.dtype, device=x.device)
@@ -518,7 +519,7 @@ def _block_bias(bias, N):
 
 
 def linear_block(x, weight: "PackedWeight", bias=None, swiglu=False, workspace: "AttnWorkspace" = None, out=None,
-                 xielu=None):
+                 xielu=None, gelu=False):
     """F.linear(x, W, bias) (or silu(x.w1^T) * (x.w3^T) for swiglu=True, weight = [w1; w3]) for 129..256 rows on the
     block-tile GEMM md_linear_block; same contract and rounding points as linear()."""
     M, N, K = _block_args(x, weight, swiglu)
@@ -539,7 +540,8 @@ def linear_block(x, weight: "PackedWeight", bias=None, swiglu=False, workspace: 
                                         K, wsp, nbytes, _stream()), "md_linear_block_xielu")
         return out
     check(lib.md_linear_block(_p(x), x.stride(0), _p(weight.data), _p(bias), _p(out), out.stride(0), M, N, K,
-                              EPI_SWIGLU if swiglu else EPI_NONE, wsp, nbytes, _stream()), "md_linear_block")
+                              (EPI_GEGLU if gelu else EPI_SWIGLU) if swiglu else EPI_NONE, wsp, nbytes, _stream()),
+          "md_linear_block")
     return out
 
 
@@ -563,7 +565,7 @@ def linear_block_add_rmsnorm(x, weight: "PackedWeight", resid, norm_weight, eps,
 
 
 # ----------------------------------------------------------------------------- K8b
-FL_NONE, FL_SWIGLU, FL_RESID, FL_ROPE_APPEND, FL_XIELU = 0, 1, 2, 3, 4
+FL_NONE, FL_SWIGLU, FL_RESID, FL_ROPE_APPEND, FL_XIELU, FL_GEGLU = 0, 1, 2, 3, 4, 5
 
 
 def fused_linear_supported(M, N, K, epilogue=FL_NONE):
@@ -580,7 +582,7 @@ def _fused_args(x, weight: "PackedWeight", bias, epilogue):
     M, K = x.shape
     if weight.K != K:
         raise ValueError(f"fused linear: x has K={K}, weight has K={weight.K}")
-    if weight.swiglu != (epilogue == FL_SWIGLU):
+    if weight.swiglu != (epilogue in (FL_SWIGLU, FL_GEGLU)):
         raise ValueError("PackedWeight was packed for a different epilogue")
     a = _lib.FusedLinearArgs()
     a.x, a.ldx, a.w_packed, a.bias = x.data_ptr(), x.stride(0), weight.data.data_ptr(), (bias.data_ptr() if bias is not None else None)
@@ -616,12 +618,12 @@ def _set_pro(a, x, pro: "DeferredNorm"):
 
 
 def fused_linear(x, weight: "PackedWeight", bias=None, swiglu=False, resid=None, out=None, want_ssq=False,
-                 pro: "DeferredNorm" = None, xielu=None):
+                 pro: "DeferredNorm" = None, xielu=None, gelu=False):
     """One launch (md_linear_fused): F.linear(x, W, bias) for M <= 256 rows over a PackedWeight, optionally followed by
     SiLU(h1) * h3 (swiglu=True, weight = [w1; w3]) or by the bf16 residual add `resid + linear` (resid [M, N]).
     want_ssq (with resid): also return the per-row partial sums of squares [M, N/32] of the result (the producer half of
     a deferred RMSNorm).  pro (with swiglu): x is pro.h and is normalised on the fly (the consumer half)."""
-    epi = FL_SWIGLU if swiglu else (FL_RESID if resid is not None else (FL_XIELU if xielu is not None else FL_NONE))
+    epi = (FL_GEGLU if gelu else FL_SWIGLU) if swiglu else (FL_RESID if resid is not None else (FL_XIELU if xielu is not None else FL_NONE))
     if xielu is not None and epi != FL_XIELU:
         raise ValueError("fused linear: the xIELU epilogue takes nothing beside it")
     a = _fused_args(x, weight, bias, epi)
@@ -941,6 +943,234 @@ def extended_attention(qkv, s: XattnSpec, k_cache, v_cache, rows: StepRows, page
         a.workspace, a.workspace_bytes = ws.data_ptr() + off, nbytes
     check(lib.md_xattn(ctypes.byref(a), _stream()), "md_xattn")
     return out
+
+
+# ----------------------------------------------------------------------------- K12
+class RotaryTable:
+    """(cos, sin) of every position and neighbouring pair, float32 [max_pos, dims / 2, 2], computed in float64 on the host.
+    base^(-2i / dims) with optional YaRN scaling (factor, original, fast, slow): frequencies below `slow` turns over the original
+    length are divided by the factor, those above `fast` turns stay, a linear ramp between; the amplitude is 1 + ln(factor) / 10."""
+
+    def __init__(self, dims, base, max_pos, scaling=None, device="cuda"):
+        if dims <= 0 or dims % 2:
+            raise ValueError(f"rotary positions: {dims} dimensions do not form pairs")
+        i = torch.arange(dims // 2, dtype=torch.float64)
+        freq, amp = base ** (-2.0 * i / dims), 1.0
+        if scaling is not None:
+            factor, original, fast, slow = scaling
+
+            def index(turns):
+                return dims * math.log(original / (2 * math.pi * turns)) / (2 * math.log(base))
+            lo, hi = max(math.floor(index(fast)), 0), min(math.ceil(index(slow)), dims - 1)
+            ramp = ((i - lo) / max(hi - lo, 0.001)).clamp(0, 1)
+            freq, amp = freq / factor * ramp + freq * (1 - ramp), 0.1 * math.log(factor) + 1.0
+        ang = torch.arange(max_pos, dtype=torch.float64).view(-1, 1) * freq
+        self.table = (torch.stack([ang.cos(), ang.sin()], -1) * amp).float().contiguous().to(device)
+        self.max_pos, self.pairs = int(max_pos), dims // 2
+
+
+def latent_row_width(kv_rank, rot_dim):
+    """Elements of a latent cache row: latent, rotated key part, padding."""
+    n = int(_lib.load().md_latent_row_width(int(kv_rank), int(rot_dim)))
+    if n == 0:
+        raise ValueError(f"latent size {kv_rank} with a rotated part of {rot_dim} is unsupported")
+    return n
+
+
+class LatentSpec:
+    """The constants of one latent-attention layer (md_latent_args): heads, sizes, score scale, rotation, and its weights in the
+    kernels' layouts: absorb [H, kv_rank, dim] (keys, moved to the query), expand [H * (dim + vdim), kv_rank] (keys, then values),
+    values [H, vdim, kv_rank] (a view of expand's second part)."""
+
+    def __init__(self, H, dim, rot_dim, vdim, q_rank, kv_rank, scale, eps, rotary: RotaryTable, expand, dq_norm, kv_norm=None):
+        self.H, self.dim, self.rot_dim, self.vdim = int(H), int(dim), int(rot_dim), int(vdim)
+        self.q_rank, self.kv_rank, self.scale, self.eps, self.rotary = int(q_rank), int(kv_rank), float(scale), float(eps), rotary
+        self.width = latent_row_width(kv_rank, rot_dim)
+        if tuple(expand.shape) != (H * (dim + vdim), kv_rank) or not expand.is_contiguous() or 2 * rotary.pairs > rot_dim:
+            raise ValueError("latent attention: expand must be [H * (dim + vdim), kv_rank], the rotation within rot_dim")
+        self.expand, self.dq_norm, self.kv_norm = expand, dq_norm, kv_norm
+        self.absorb = expand[:H * dim].view(H, dim, kv_rank).transpose(1, 2).contiguous()
+        self.values = expand[H * dim:].view(H, vdim, kv_rank)
+
+    def flops(self, new, ctx):
+        """(absorbed, expanded) multiply-adds per head for `new` rows per request at the end of `ctx` positions (host lists):
+        which form of the attention a step should take."""
+        R = self.kv_rank
+        pairs = sum(n * (c - (n - 1) / 2) for n, c in zip(new, ctx))
+        absorbed = pairs * (2 * R + self.rot_dim) + sum(new) * R * (self.dim + self.vdim)
+        expanded = pairs * (self.dim + self.rot_dim + self.vdim) + sum(ctx) * R * (self.dim + self.vdim)
+        return absorbed, expanded
+
+
+def _latent_args(s: LatentSpec, cache, rows: StepRows, page_indices, page_indptr, max_pages, dtype):
+    _gpu(cache)
+    _dense(cache)
+    if cache.dim() != 3 or cache.shape[2] != s.width or cache.dtype != dtype:
+        raise ValueError("latent attention: pages must be [pages, page_size, row width] of the model's dtype")
+    if page_indptr.numel() != rows.B + 1:
+        raise ValueError("latent attention: page table of another batch")
+    a = _lib.LatentArgs()
+    a.cache, a.cos_sin, a.max_pos, a.rot_pairs = cache.data_ptr(), s.rotary.table.data_ptr(), s.rotary.max_pos, s.rotary.pairs
+    a.qo_indptr, a.pos0, a.B, a.n_max = rows.qo_indptr.data_ptr(), rows.pos0.data_ptr(), rows.B, rows.n_max
+    a.page_indices, a.page_indptr = _i32(page_indices).data_ptr(), _i32(page_indptr).data_ptr()
+    a.page_size, a.max_pages = cache.shape[1], int(max_pages)
+    a.H, a.dim, a.rot_dim, a.vdim, a.q_rank, a.kv_rank = s.H, s.dim, s.rot_dim, s.vdim, s.q_rank, s.kv_rank
+    a.scale, a.eps, a.dtype = s.scale, s.eps, _MODEL_DTYPES[dtype]
+    return a
+
+
+def latent_append(z, s: LatentSpec, cache, rows: StepRows, page_indices, page_indptr, max_pages):
+    """z [M, >= q_rank (+ kv_rank + rot_dim)]: the normalised query latents [M, q_rank]; with s.kv_norm the normalised latent and
+    the rotated key part of every row go to its position's cache row."""
+    _gpu(z)
+    if z.dim() != 2 or z.stride(1) != 1 or z.shape[1] < s.q_rank + (s.kv_rank + s.rot_dim if s.kv_norm is not None else 0):
+        raise ValueError("latent_append: rows must hold the query latent, the latent and the key part")
+    a = _latent_args(s, cache, rows, page_indices, page_indptr, max_pages, z.dtype)
+    cq = torch.empty((z.shape[0], s.q_rank), dtype=z.dtype, device=z.device)
+    a.z, a.ldz, a.cq, a.dq_norm = z.data_ptr(), z.stride(0), cq.data_ptr(), s.dq_norm.data_ptr()
+    if s.kv_norm is not None:
+        a.kv_norm, a.append = s.kv_norm.data_ptr(), 1
+    check(_lib.load().md_latent_append(ctypes.byref(a), _stream()), "md_latent_append")
+    return cq
+
+
+def head_linear(x, w, out, gate=None):
+    """out[:, h] = x[:, h] . w[h]^T (* sigmoid(gate[:, h])) for x [M, H, K], w [H, N, K], out [M, H, >= N] (strides free in the
+    first two dimensions)."""
+    _head_linear(x, w, out, gate)
+    return out
+
+
+def _head_linear(x, w, out, gate=None, tail=None, tail_pad=0, rotary=None, rows=None):
+    _gpu(x, w, out, gate, tail)
+    _dense(w)
+    M, H, K = x.shape
+    if w.dim() != 3 or w.shape[0] != H or w.shape[2] != K or tuple(out.shape[:2]) != (M, H):
+        raise ValueError(f"head_linear: x {tuple(x.shape)}, w {tuple(w.shape)}, out {tuple(out.shape)}")
+    for t in (x, out) + ((tail,) if tail is not None else ()) + ((gate,) if gate is not None else ()):
+        if t.stride(-1) != 1 or t.dtype != w.dtype:
+            raise ValueError("head_linear: unit inner strides and one dtype expected")
+    a = _lib.HeadLinearArgs()
+    a.x, a.w, a.out, a.ldx, a.hx, a.ldo, a.ho = x.data_ptr(), w.data_ptr(), out.data_ptr(), x.stride(0), x.stride(1), out.stride(0), out.stride(1)
+    a.M, a.H, a.N, a.K, a.dtype = M, H, w.shape[1], K, _model_dtype(w)
+    if out.shape[2] < a.N + tail_pad:
+        raise ValueError("head_linear: out is too narrow")
+    if gate is not None:
+        if tuple(gate.shape) != (M, H):
+            raise ValueError("head_linear: gate must be [rows, heads]")
+        a.gate, a.ld_gate = gate.data_ptr(), gate.stride(0)
+    if tail is not None:
+        a.tail, a.ldt, a.ht, a.tail_dim, a.tail_pad = tail.data_ptr(), tail.stride(0), tail.stride(1), tail.shape[2], tail_pad
+        a.cos_sin, a.max_pos, a.rot_pairs = rotary.table.data_ptr(), rotary.max_pos, rotary.pairs
+        a.qo_indptr, a.pos0, a.B = rows.qo_indptr.data_ptr(), rows.pos0.data_ptr(), rows.B
+    check(_lib.load().md_head_linear(ctypes.byref(a), _stream()), "md_head_linear")
+
+
+def latent_attention(q, s: LatentSpec, cache, rows: StepRows, page_indices, page_indptr, max_pages, workspace: AttnWorkspace, out,
+                     gate=None, ctx=None, plain=False):
+    """out [M, H, vdim] (row stride free) = softmax attention of q [M, H * (dim + rot_dim)] (as projected) over the cache, which
+    latent_append has brought up to the step's own rows, times sigmoid(gate [M, H]).  ctx = `LatentContext`: the expanded form is
+    taken where it is cheaper; without it, in 32-bit or for unusual sizes the absorbed form.  plain: its plain kernel."""
+    _gpu(q, out)
+    M = q.shape[0]
+    if tuple(q.shape) != (M, s.H * (s.dim + s.rot_dim)) or not q.is_contiguous() or tuple(out.shape) != (M, s.H, s.vdim):
+        raise ValueError("latent attention: q must be [rows, H * (dim + rot_dim)], out [rows, H, vdim]")
+    if out.stride(2) != 1 or out.stride(1) != s.vdim or (gate is not None and gate.stride(1) != 1):
+        raise ValueError("latent attention: heads of out must be dense")
+    lib = _lib.load()
+    a = _latent_args(s, cache, rows, page_indices, page_indptr, max_pages, q.dtype)
+    a.force_plain = int(plain)
+    if ctx is not None and not plain and ctx.expanded(s) and out.stride(0) % 4 == 0 and lib.md_latent_prefill_supported(ctypes.byref(a)):
+        dense = torch.empty((ctx.total, s.kv_rank), dtype=q.dtype, device=q.device)
+        a.ctx_indptr = ctx.indptr.data_ptr()
+        check(lib.md_latent_gather(ctypes.byref(a), ctx.longest, _p(dense), _stream()), "md_latent_gather")
+        kv = torch.nn.functional.linear(dense, s.expand)
+        a.q, a.kv, a.out, a.ldo = q.data_ptr(), kv.data_ptr(), out.data_ptr(), out.stride(0)
+        if gate is not None:
+            a.gate, a.ld_gate = gate.data_ptr(), gate.stride(0)
+        check(lib.md_latent_prefill(ctypes.byref(a), _stream()), "md_latent_prefill")
+        return out
+    heads = q.view(M, s.H, s.dim + s.rot_dim)
+    qa = torch.empty((M, s.H, s.width), dtype=q.dtype, device=q.device)
+    _head_linear(heads[..., :s.dim], s.absorb, qa, tail=heads[..., s.dim:], tail_pad=s.width - s.kv_rank, rotary=s.rotary, rows=rows)
+    lat = torch.empty((M, s.H, s.kv_rank), dtype=q.dtype, device=q.device)
+    a.q, a.out = qa.data_ptr(), lat.data_ptr()
+    nbytes = lib.md_latent_workspace_bytes(ctypes.byref(a))
+    if nbytes:
+        ws = workspace.get(nbytes + 256)
+        a.workspace, a.workspace_bytes = ws.data_ptr() + (-ws.data_ptr()) % 256, nbytes
+    check(lib.md_latent_attn(ctypes.byref(a), _stream()), "md_latent_attn")
+    _head_linear(lat, s.values, out, gate=gate)
+    return out
+
+
+class LatentContext:
+    """What the host knows of a step's requests: `new` rows each, at the end of `ctx` positions."""
+    MAX_EXPANDED_BYTES = 24 << 30
+
+    def __init__(self, new, ctx, device):
+        self.new, self.ctx, self.total, self.longest = list(new), list(ctx), sum(ctx), max(ctx)
+        self._device, self._indptr, self._choice = device, None, {}
+
+    @property
+    def indptr(self):
+        if self._indptr is None:
+            at = [0]
+            for c in self.ctx:
+                at.append(at[-1] + c)
+            self._indptr = torch.tensor(at, dtype=torch.int32).to(self._device)
+        return self._indptr
+
+    def expanded(self, s: LatentSpec):
+        """Does the expanded form take fewer operations (and fit) for these requests?"""
+        key = (s.H, s.dim, s.rot_dim, s.vdim, s.kv_rank)
+        if key not in self._choice:
+            absorbed, expanded = s.flops(self.new, self.ctx)
+            size = self.total * s.H * (s.dim + s.vdim) * 2
+            self._choice[key] = expanded < absorbed and max(self.new) >= 64 and size <= self.MAX_EXPANDED_BYTES
+        return self._choice[key]
+
+
+def embed_bigram(tokens, table, pairs, norm_weight, eps, mul_before, mul_token, history, rows: StepRows, page_indices, page_indptr):
+    """float32 rows rms(table[t] + pairs[(mul_before * before + mul_token * t) mod n]) * norm_weight; the last row of `pairs`
+    (row n) for a sequence's first token.  history: int32 [pages, page_size], the tokens of every sequence by position."""
+    _gpu(tokens, table, pairs, norm_weight, history)
+    _dense(tokens, table, pairs, norm_weight, history)
+    vocab, width = table.shape
+    if tokens.dtype != torch.int64 or history.dtype != torch.int32 or history.dim() != 2:
+        raise TypeError("embed_bigram: token ids are int64, the token history int32 [pages, page_size]")
+    if pairs.shape[1] != width or pairs.shape[0] < 2 or norm_weight.numel() != width or pairs.dtype != table.dtype or norm_weight.dtype != table.dtype:
+        raise ValueError("embed_bigram: tables of different widths or dtypes")
+    if page_indptr.numel() != rows.B + 1:
+        raise ValueError("embed_bigram: page table of another batch")
+    out = torch.empty((tokens.numel(), width), dtype=torch.float32, device=table.device)
+    check(_lib.load().md_embed_bigram(_p(tokens), _p(table), _p(pairs), _p(norm_weight), _model_dtype(table), _p(rows.qo_indptr),
+                                      _p(rows.pos0), rows.B, rows.n_max, width, vocab, pairs.shape[0] - 1, int(mul_before),
+                                      int(mul_token), _p(history), _p(_i32(page_indices)), _p(_i32(page_indptr)), history.shape[1],
+                                      float(eps), _p(out), _stream()), "md_embed_bigram")
+    return out
+
+
+def gelu_mul(a, b, out=None):
+    """gelu_tanh(a) * b of 2-D rows with unit inner stride (fp32, one rounding)."""
+    _gpu(a, b, out)
+    if a.dim() != 2 or a.shape != b.shape or a.stride(1) != 1 or b.stride(1) != 1 or a.dtype != b.dtype:
+        raise ValueError("gelu_mul expects 2-D rows of one shape with unit inner stride")
+    y = torch.empty(a.shape, dtype=a.dtype, device=a.device) if out is None else out
+    if y.shape != a.shape or y.stride(1) != 1 or y.dtype != a.dtype:
+        raise ValueError("gelu_mul: out of another shape or dtype")
+    check(_lib.load().md_gelu_mul(_p(a), _p(b), a.stride(0), b.stride(0), _p(y), y.stride(0), a.shape[0], a.shape[1], _model_dtype(a),
+                                  _stream()), "md_gelu_mul")
+    return y
+
+
+def softcap_(z, cap):
+    """cap * tanh(z / cap) of 2-D rows, in place."""
+    _gpu(z)
+    if z.dim() != 2 or z.stride(1) != 1:
+        raise ValueError("softcap_ expects 2-D rows with unit inner stride")
+    check(_lib.load().md_softcap(_p(z), z.stride(0), float(cap), z.shape[0], z.shape[1], _model_dtype(z), _stream()), "md_softcap")
+    return z
 
 
 # ----------------------------------------------------------------------------- K10
