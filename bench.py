@@ -105,7 +105,7 @@ def parse(argv=None):
                          "Default (round 6): peaked with miss = 0.2, so that the driver's line carries a MEASURED "
                          "acceptance next to the replay that defines `value`; timings are weight-value independent "
                          "(ms_per_step of the two agree to 0.1 %%: profiles/r06_bench_cfg3_peaked_miss_sweep_c7.json)")
-    ap.add_argument("--design", default=None, metavar="furitar",
+    ap.add_argument("--design", default=None, metavar="furitar|bufodra",
                     help="instead of a workload: prefill and decode throughput of a layered decoder design at a few sizes, beside "
                          "the Llama-style model of equal size (magicdec_amd/design_bench.py)")
     ap.add_argument("--design-sizes", nargs="*", default=None, help="sizes of --design (default: all)")

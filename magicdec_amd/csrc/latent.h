@@ -26,7 +26,7 @@ struct LatentParams {
     float eps, scale_log2;
 };
 
-// rows of one absorbed workgroup: 16 or 32 (token, head) pairs
+// absorbed form; qt: 16-row tiles of (token, head) pairs per workgroup (1 or 2)
 int md_internal_latent_absorbed(const LatentParams& p, int qt, hipStream_t st);
 bool md_internal_latent_absorbed_ok(int kv_rank, int W, int qt);
 // expanded form; DK: padded dim + rot_dim, one translation unit each

@@ -123,20 +123,24 @@ __device__ __forceinline__ float sigmoid(float v) { return 1.0f / (1.0f + expf(-
 
 template <typename T>
 __device__ __forceinline__ void head_tail(const HeadLinearParams& p, int h, int row0, int nrow) {
-    for (int i = threadIdx.x; i < nrow * p.tail_pad; i += 256) {
-        const int row = row0 + i / p.tail_pad, d = i % p.tail_pad;
-        if (row >= p.M) return;
-        float v = 0.f;
-        if (d < p.tail_dim) {
-            int lo = 0, hi = p.B;                                   // request of the row: qo_indptr[lo] <= row < qo_indptr[lo + 1]
-            while (hi - lo > 1) {
-                const int mid = (lo + hi) >> 1;
-                if (p.qo_indptr[mid] <= row) lo = mid; else hi = mid;
-            }
-            const int pos = min(max(p.pos0[lo] + row - p.qo_indptr[lo], 0), p.max_pos - 1);
-            v = rotated(reinterpret_cast<const T*>(p.tail) + row * p.ldt + h * p.ht, d, p.rot_pairs,
-                        p.cos_sin + (int64_t)pos * p.rot_pairs * 2);
+    // the column blocks of a row tile share its tail: this block's rows are row0 + blockIdx.x, + gridDim.x, ...
+    __shared__ int s_pos[64];
+    if (threadIdx.x < nrow) {
+        const int row = min(row0 + (int)threadIdx.x, p.M - 1);
+        int lo = 0, hi = p.B;                                       // request of the row: qo_indptr[lo] <= row < qo_indptr[lo + 1]
+        while (hi - lo > 1) {
+            const int mid = (lo + hi) >> 1;
+            if (p.qo_indptr[mid] <= row) lo = mid; else hi = mid;
         }
+        s_pos[threadIdx.x] = min(max(p.pos0[lo] + row - p.qo_indptr[lo], 0), p.max_pos - 1);
+    }
+    __syncthreads();
+    const int mine = (nrow - (int)blockIdx.x + (int)gridDim.x - 1) / (int)gridDim.x;
+    for (int i = threadIdx.x; i < mine * p.tail_pad; i += 256) {
+        const int r = blockIdx.x + i / p.tail_pad * gridDim.x, d = i % p.tail_pad, row = row0 + r;
+        if (row >= p.M) break;
+        const float v = d < p.tail_dim ? rotated(reinterpret_cast<const T*>(p.tail) + row * p.ldt + h * p.ht, d, p.rot_pairs,
+                                                 p.cos_sin + (int64_t)s_pos[r] * p.rot_pairs * 2) : 0.f;
         (reinterpret_cast<T*>(p.out) + row * p.ldo + h * p.ho)[p.N + d] = (T)v;
     }
 }
@@ -146,6 +150,7 @@ template <int RT, bool VEC>
 __global__ __launch_bounds__(256) void head_linear_mfma_kernel(const HeadLinearParams p) {
     const int lane = threadIdx.x & 63, lq = lane & 15, lc = lane >> 4, wave = threadIdx.x >> 6;
     const int h = blockIdx.z, row0 = blockIdx.y * 16 * RT, n0 = blockIdx.x * 64 + wave * 16;
+    if (p.tail) head_tail<bf16_t>(p, h, row0, 16 * RT);
     const bf16x8 z8 = {0, 0, 0, 0, 0, 0, 0, 0};
     auto piece = [&](const bf16_t* src, int k, bool ok) {
         if (VEC) return ok && k < p.K ? *reinterpret_cast<const bf16x8*>(src + k) : z8;
@@ -169,12 +174,18 @@ __global__ __launch_bounds__(256) void head_linear_mfma_kernel(const HeadLinearP
             xp[r] = reinterpret_cast<const bf16_t*>(p.x) + (int64_t)(r_ok[r] ? row : 0) * p.ldx + h * p.hx;
             acc[r] = f32x4{0.f, 0.f, 0.f, 0.f};
         }
-#pragma unroll 4
-        for (int k0 = 0; k0 < p.K; k0 += 32) {
-            const bf16x8 wf = piece(wp, k0 + lc * 8, n_ok);
+        for (int kb = 0; kb < p.K; kb += 128) {                     // four steps requested together (zeros past K)
+            bf16x8 wf[4], xf[4][RT];
 #pragma unroll
-            for (int r = 0; r < RT; ++r)
-                acc[r] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wf, piece(xp[r], k0 + lc * 8, r_ok[r]), acc[r], 0, 0, 0);
+            for (int u = 0; u < 4; ++u) {
+                wf[u] = piece(wp, kb + u * 32 + lc * 8, n_ok);
+#pragma unroll
+                for (int r = 0; r < RT; ++r) xf[u][r] = piece(xp[r], kb + u * 32 + lc * 8, r_ok[r]);
+            }
+#pragma unroll
+            for (int u = 0; u < 4; ++u)
+#pragma unroll
+                for (int r = 0; r < RT; ++r) acc[r] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wf[u], xf[u][r], acc[r], 0, 0, 0);
         }
         // acc[r][e] = y[row0 + r * 16 + lq][n0 + lc * 4 + e]
 #pragma unroll
@@ -192,7 +203,6 @@ __global__ __launch_bounds__(256) void head_linear_mfma_kernel(const HeadLinearP
             }
         }
     }
-    if (p.tail && blockIdx.x == 0) head_tail<bf16_t>(p, h, row0, 16 * RT);
 }
 
 // 32-bit: a thread per output
@@ -206,11 +216,11 @@ __global__ __launch_bounds__(256) void head_linear_f32_kernel(const HeadLinearPa
         if (p.gate) s *= sigmoid(reinterpret_cast<const float*>(p.gate)[row * p.ld_gate + h]);
         (reinterpret_cast<float*>(p.out) + row * p.ldo + h * p.ho)[n] = s;
     }
-    if (p.tail && blockIdx.x == 0) head_tail<float>(p, h, row0, 16);
+    if (p.tail) head_tail<float>(p, h, row0, 16);
 }
 
 // ------------------------------------------------------------------------------------------------ merge, gather
-// partials of the kv splits: ws = sums [slot][16 qt][Rp], then (max, weight) [slot][16 qt][2]; slot = (b * groups + g) * nsplit + s
+// partials of the kv splits: ws = sums [slot][rows_wg][Rp], then (reference, weight) [slot][rows_wg][2]; slot = (b * groups + g) * nsplit + s
 __global__ __launch_bounds__(256) void latent_merge_kernel(const LatentParams p, int rows_wg, int Rp) {
     const int b = blockIdx.y, q0 = p.qo_indptr[b], nrows = (p.qo_indptr[b + 1] - q0) * p.H;
     const int d4 = Rp / 4;
@@ -221,14 +231,33 @@ __global__ __launch_bounds__(256) void latent_merge_kernel(const LatentParams p,
     const int64_t slot0 = ((int64_t)b * p.n_groups + g) * p.nsplit;
     const float* ml = p.ws + (int64_t)p.B * p.n_groups * p.nsplit * rows_wg * Rp;
     float m = -INFINITY;
-    for (int s = 0; s < p.nsplit; ++s) m = fmaxf(m, ml[((slot0 + s) * rows_wg + r) * 2]);
+    // eight splits requested together, added in order
+    for (int s0 = 0; s0 < p.nsplit; s0 += 8) {
+        float t[8];
+#pragma unroll
+        for (int u = 0; u < 8; ++u) t[u] = s0 + u < p.nsplit ? ml[((slot0 + s0 + u) * rows_wg + r) * 2] : -INFINITY;
+#pragma unroll
+        for (int u = 0; u < 8; ++u) m = fmaxf(m, t[u]);
+    }
     f32x4 o = {0.f, 0.f, 0.f, 0.f};
     float l = 0.f;
-    for (int s = 0; s < p.nsplit; ++s) {
-        const int64_t at = (slot0 + s) * rows_wg + r;
-        const float w = ml[at * 2] == -INFINITY ? 0.f : __builtin_amdgcn_exp2f(ml[at * 2] - m);
-        o += *reinterpret_cast<const f32x4*>(p.ws + at * Rp + d) * w;
-        l += ml[at * 2 + 1] * w;
+    for (int s0 = 0; s0 < p.nsplit; s0 += 8) {
+        f32x2 t[8];
+        f32x4 v[8];
+#pragma unroll
+        for (int u = 0; u < 8; ++u)
+            if (s0 + u < p.nsplit) {                                  // uniform
+                const int64_t at = (slot0 + s0 + u) * rows_wg + r;
+                t[u] = *reinterpret_cast<const f32x2*>(ml + at * 2);
+                v[u] = *reinterpret_cast<const f32x4*>(p.ws + at * Rp + d);
+            }
+#pragma unroll
+        for (int u = 0; u < 8; ++u)
+            if (s0 + u < p.nsplit) {
+                const float w = t[u][0] == -INFINITY ? 0.f : __builtin_amdgcn_exp2f(t[u][0] - m);
+                o += v[u] * w;
+                l += t[u][1] * w;
+            }
     }
     const float inv = l > 0.f ? 1.0f / l : 0.f;
     bf16_t* op = reinterpret_cast<bf16_t*>(p.out) + ((int64_t)q0 * p.H + row) * p.kv_rank + d;
@@ -265,12 +294,13 @@ bool mfma_ok(const md_latent_args* a) {
            md_internal_latent_absorbed_ok(a->kv_rank, row_width(a->kv_rank, a->rot_dim), row_tiles(a));
 }
 
-int g_target_wgs = 256;
+constexpr int kTargetWgs = 512;              // 16-row workgroups: two per CU (of 32 rows: one)
 
 int kv_splits(const md_latent_args* a) {
-    const long tiles = ((long)a->max_pages * a->page_size + 63) / 64, groups = (long)a->B * row_groups(a);
-    long want = (g_target_wgs + groups - 1) / groups;
-    const long cap = tiles / 4 > 1 ? tiles / 4 : 1;                  // >= 256 keys per workgroup
+    const long tiles = ((long)a->max_pages * a->page_size + 31) / 32, groups = (long)a->B * row_groups(a);
+    const long target = kTargetWgs / row_tiles(a);
+    long want = (target + groups - 1) / groups;
+    const long cap = tiles / 8 > 1 ? tiles / 8 : 1;                  // >= 256 keys per workgroup
     if (want > cap) want = cap;
     return (int)(want < 1 ? 1 : want > 64 ? 64 : want);
 }

@@ -1,35 +1,61 @@
 // Absorbed latent attention on the matrix cores (bf16 pages, gfx950): queries of W numbers per (token, head) against cache rows
 // every head shares; the value row is the first kv_rank numbers of the key row, so a key tile is staged once and read twice.
 //
-// A workgroup owns 16 QT (token, head) rows of one request (token-major) and one range of 64-key tiles.  Per tile
-//   1. the tile, requested one iteration ahead (a linear copy: rows of a page are contiguous), goes from registers to LDS;
-//   2. S^T = K Q^T on 16x16x32: a wavefront takes 16 keys of one 16-row tile, queries and keys both from LDS; the scaled, masked
-//      scores of the whole tile meet in LDS (fp32);
-//   3. every wavefront forms the same running maximum and weights for its rows (two 16-byte reads per 32 keys: the weights are
-//      the PV operand as they are) and adds O^T += V^T P^T for its share of the kv_rank columns, V^T by transposing LDS reads.
-// Weights enter the product as a bf16 part and a bf16 rest (error 2^-17).  Splits leave sums, maximum and weight per row.
+// A workgroup of 4 QT wavefronts owns 16 QT (token, head) rows of one request (token-major) and one range of 32-key tiles.  Per tile
+//   1. the tile, requested two iterations ahead (a linear copy: rows of a page are contiguous), goes from registers to LDS;
+//   2. S^T = K Q^T on 16x16x32: a wavefront takes 16 keys, 16 rows and half of the depth; scores meet in LDS (fp32, two halves);
+//   3. 16 lanes per row add the halves, mask, and follow the maximum -- lazily: the reference moves only when a tile exceeds it by
+//      8 in the exponent -- and leave the weights in LDS as a bf16 part and a bf16 rest (error 2^-17), in operand order;
+//   4. every wavefront adds O^T += V^T P^T for its share of the kv_rank columns, V^T by transposing LDS reads.
+// Two tiles are in flight per workgroup and their LDS images are small (37 KB at W = 576): a CU holds one workgroup of 32 rows or
+// two of 16.  Splits leave sums, reference and weight per row.
 #include "attn_common.h"
 #include "latent.h"
 
+#include <type_traits>
+
 namespace {
 
-constexpr int KT = 64;
+constexpr int KT = 32;
 constexpr int kSPitch = KT + 4;                     // floats per score row
+constexpr int kPPitch = KT * 2 + 16;                // bytes per weight row
 
 __host__ __device__ constexpr int row_pitch(int W) { return W * 2 + 16; }
 
-// QT: 16-row tiles; NBW: 16-column blocks of the latent per wavefront
-template <int QT, int NBW>
-__global__ __launch_bounds__(256 * QT, 1) void latent_absorbed_kernel(const LatentParams p) {
-    constexpr int NW = 4 * QT, NT = 64 * NW, ROWS = 16 * QT;
-    constexpr int MAXP = 2 * NBW + 4;               // 16-byte pieces of a tile per thread (W <= 64 NBW QT + 128)
+// over the 16 lanes of a row (rotations within it: no LDS)
+template <int N>
+__device__ __forceinline__ float row_ror(float v) {
+    return __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(v), 0x120 + N, 0xf, 0xf, false));
+}
+__device__ __forceinline__ float row_max(float v) {
+    v = fmaxf(v, row_ror<8>(v));
+    v = fmaxf(v, row_ror<4>(v));
+    v = fmaxf(v, row_ror<2>(v));
+    return fmaxf(v, row_ror<1>(v));
+}
+__device__ __forceinline__ float row_sum(float v) {
+    v += row_ror<8>(v);
+    v += row_ror<4>(v);
+    v += row_ror<2>(v);
+    return v + row_ror<1>(v);
+}
+
+// NBW: 16-column blocks of the latent per wavefront; KS: 32-deep steps of a score where known at compile time (a wavefront's
+// queries then live in registers), 0: any
+template <int QT, int NBW, int KS>
+__global__ __launch_bounds__(256 * QT, 2) void latent_absorbed_kernel(const LatentParams p) {
+    constexpr int ROWS = 16 * QT, NT = 256 * QT;
+    constexpr int MAXP = KS ? (KS * 128 + NT - 1) / NT : NBW + 2;                // 16-byte pieces of a tile per thread (W <= 64 QT NBW + 128)
+    constexpr int KH = (KS + 1) / 2;                    // steps of the first half
     extern __shared__ __attribute__((aligned(16))) unsigned char smem[];
     const int tid = threadIdx.x, lane = tid & 63, lq = lane & 15, lc = lane >> 4;
     const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
-    const int W = p.W, pitch = row_pitch(W), R = p.kv_rank;
+    const int W = KS ? KS * 32 : p.W, pitch = row_pitch(W), R = p.kv_rank;
     unsigned char* ldsK = smem;
     unsigned char* ldsQ = smem + KT * pitch;
-    float* ldsS = reinterpret_cast<float*>(ldsQ + ROWS * pitch);
+    float* ldsS = reinterpret_cast<float*>(ldsQ + (KS ? 0 : ROWS * pitch));     // [half][row][key]
+    float* ldsA = ldsS + 2 * ROWS * kSPitch;                                    // per row: factor of the sums so far
+    unsigned char* ldsP = reinterpret_cast<unsigned char*>(ldsA + ROWS);        // weights: bf16 parts, then rests
 
     // request fastest: with a multiple of 8 requests one request's workgroups share an XCD (and its L2)
     const int b = blockIdx.x % p.B, sub = blockIdx.x / p.B, group = sub % p.n_groups, split = sub / p.n_groups;
@@ -43,158 +69,171 @@ __global__ __launch_bounds__(256 * QT, 1) void latent_absorbed_kernel(const Late
     const int t_begin = split * tps, t_end = min(ntiles, t_begin + tps);
 
     const int per_row = W / 8, pieces = KT * per_row;
-    {   // queries of the workgroup; rows past the last one are zero
-        const u32x4* src = reinterpret_cast<const u32x4*>(reinterpret_cast<const bf16_t*>(p.q) + ((int64_t)q0 * p.H + row0) * W);
-        const int have = min(ROWS, nrows - row0) * per_row;
-        for (int c = tid; c < ROWS * per_row; c += NT)
-            *reinterpret_cast<u32x4*>(ldsQ + (c / per_row) * pitch + (c % per_row) * 16) = c < have ? src[c] : u32x4{0u, 0u, 0u, 0u};
-    }
     int at[MAXP];                                   // LDS byte of this thread's pieces
 #pragma unroll
     for (int i = 0; i < MAXP; ++i) {
         const int c = i * NT + tid;
         at[i] = (c / per_row) * pitch + (c % per_row) * 16;
     }
-    u32x4 kr[MAXP];
-    auto issue = [&](int t) {
+    auto issue = [&](int t, u32x4 (&kr)[MAXP]) {
         const int pos = t * KT, page = p.page_indices[pg0 + pos / p.page_size];
         const u32x4* src = reinterpret_cast<const u32x4*>(reinterpret_cast<const bf16_t*>(p.cache) +
                                                           ((int64_t)page * p.page_size + pos % p.page_size) * W);
 #pragma unroll
         for (int i = 0; i < MAXP; ++i)
-            if (i * NT + tid < pieces) kr[i] = __builtin_nontemporal_load(src + i * NT + tid);
+            if (KS * 128 % NT == 0 || i * NT + tid < pieces) kr[i] = __builtin_nontemporal_load(src + i * NT + tid);
     };
-    auto stage = [&](int t) {
-        const bool tail = t * KT + KT - 1 > written;                // rows not written yet may hold anything (NaN)
+    auto stage = [&](int t, u32x4 (&kr)[MAXP]) {
+        if (t * KT + KT - 1 > written) {                            // rows not written yet may hold anything (NaN)
+#pragma unroll
+            for (int i = 0; i < MAXP; ++i)
+                if (t * KT + (i * NT + tid) / per_row > written) kr[i] = u32x4{0u, 0u, 0u, 0u};
+        }
 #pragma unroll
         for (int i = 0; i < MAXP; ++i)
-            if (i * NT + tid < pieces) {
-                if (tail && t * KT + (i * NT + tid) / per_row > written) kr[i] = u32x4{0u, 0u, 0u, 0u};
-                *reinterpret_cast<u32x4*>(ldsK + at[i]) = kr[i];
-            }
+            if (KS * 128 % NT == 0 || i * NT + tid < pieces) *reinterpret_cast<u32x4*>(ldsK + at[i]) = kr[i];
     };
+    u32x4 kx[MAXP], ky[MAXP];
+    if (t_begin < t_end) issue(t_begin, kx);
+    if (t_begin + 1 < t_end) issue(t_begin + 1, ky);
 
-    // score step: this wavefront's 16 keys and 16-row tile
-    const int ks = wave & 3, rt = wave >> 2;
-    const int my_row = row0 + rt * 16 + lq;
-    const int lim = my_row < nrows ? min(pos_b + my_row / p.H, cap - 1) : -1;
-    const unsigned char* ka = ldsK + (ks * 16 + lq) * pitch + lc * 16;
-    const unsigned char* qa = ldsQ + (rt * 16 + lq) * pitch + lc * 16;
-    float* s_out = ldsS + (rt * 16 + lq) * kSPitch + ks * 16 + lc * 4;
-    const int steps = W / 32;
+    // score step: this wavefront's 16 keys and half of the depth
+    const int ks = wave & 1, half = wave >> 1 & 1, rt = wave >> 2;
+    const int steps = W / 32, k_begin = half ? (steps + 1) / 2 : 0, k_end = half ? steps : (steps + 1) / 2;
+    const unsigned char* ka = ldsK + (ks * 16 + lq) * pitch + lc * 16 + k_begin * 64;
+    const unsigned char* qa = ldsQ + (rt * 16 + lq) * pitch + lc * 16 + k_begin * 64;
+    float* s_out = ldsS + (half * ROWS + rt * 16 + lq) * kSPitch + ks * 16 + lc * 4;
+    bf16x8 qf[KS ? KH : 1];
+    if constexpr (KS > 0) {
+        const bf16_t* qp = reinterpret_cast<const bf16_t*>(p.q) + ((int64_t)q0 * p.H + min(row0 + rt * 16 + lq, nrows - 1)) * W + k_begin * 32 + lc * 8;
+        const bf16x8 z = {0, 0, 0, 0, 0, 0, 0, 0};
+#pragma unroll
+        for (int k = 0; k < KH; ++k) qf[k] = k_begin + k < k_end ? *reinterpret_cast<const bf16x8*>(qp + k * 32) : z;
+    } else {                                        // queries of the workgroup; rows past the last one are zero
+        const u32x4* src = reinterpret_cast<const u32x4*>(reinterpret_cast<const bf16_t*>(p.q) + ((int64_t)q0 * p.H + row0) * W);
+        const int have = min(ROWS, nrows - row0) * per_row;
+        for (int c = tid; c < ROWS * per_row; c += NT)
+            *reinterpret_cast<u32x4*>(ldsQ + (c / per_row) * pitch + (c % per_row) * 16) = c < have ? src[c] : u32x4{0u, 0u, 0u, 0u};
+    }
+    // weight step: this lane's row and two keys; key k of a tile stands at (k / 4 % 4) * 8 + k / 16 * 4 + k % 4
+    const int wr = tid >> 4, wk = (tid & 15) * 2;
+    const int lim = row0 + wr < nrows ? min(pos_b + (row0 + wr) / p.H, cap - 1) : -1;
+    const float* s_in = ldsS + wr * kSPitch + wk;
+    unsigned char* p_out = ldsP + wr * kPPitch + ((wk >> 2 & 3) * 8 + (wk >> 4) * 4 + (wk & 3)) * 2;
+    const unsigned char* p_in = ldsP + lq * kPPitch + lc * 16;
+    float m = -INFINITY, l = 0.f;
 
     f32x4 o[QT][NBW];
-    float m[QT], l[QT];
 #pragma unroll
-    for (int qt = 0; qt < QT; ++qt) {
-        m[qt] = -INFINITY;
-        l[qt] = 0.f;
+    for (int qt = 0; qt < QT; ++qt)
 #pragma unroll
         for (int nb = 0; nb < NBW; ++nb) o[qt][nb] = f32x4{0.f, 0.f, 0.f, 0.f};
-    }
-    const int vra = (lc * 4 + (lq >> 2)) * pitch + (lq & 3) * 8;
+    const unsigned char* va = ldsK + (lc * 4 + (lq >> 2)) * pitch + (lq & 3) * 8 + wave * NBW * 32;
 
-    if (t_begin < t_end) issue(t_begin);
-    for (int t = t_begin; t < t_end; ++t) {
-        stage(t);
-        if (t + 1 < t_end) issue(t + 1);
+    auto process = [&](auto steady, int t, u32x4 (&kr)[MAXP]) {
+        stage(t, kr);
+        if (decltype(steady)::value || t + 2 < t_end) issue(t + 2, kr);
         __syncthreads();
         {
             f32x4 s0 = {0.f, 0.f, 0.f, 0.f}, s1 = {0.f, 0.f, 0.f, 0.f};
-            int k = 0;
-            for (; k + 2 <= steps; k += 2) {
-                s0 = __builtin_amdgcn_mfma_f32_16x16x32_bf16(lds_read_b128(ka + k * 64), lds_read_b128(qa + k * 64), s0, 0, 0, 0);
-                s1 = __builtin_amdgcn_mfma_f32_16x16x32_bf16(lds_read_b128(ka + k * 64 + 64), lds_read_b128(qa + k * 64 + 64), s1, 0, 0, 0);
-            }
-            if (k < steps)
-                s0 = __builtin_amdgcn_mfma_f32_16x16x32_bf16(lds_read_b128(ka + k * 64), lds_read_b128(qa + k * 64), s0, 0, 0, 0);
-            const int kp = t * KT + ks * 16 + lc * 4;
+            if constexpr (KS > 0) {
 #pragma unroll
-            for (int e = 0; e < 4; ++e) {
-                s0[e] = (s0[e] + s1[e]) * p.scale_log2;
-                if (kp + e > lim) s0[e] = -INFINITY;
+                for (int k = 0; k < KH; ++k) {      // (an odd KS: the second half's last step multiplies by zeros)
+                    f32x4& s = k & 1 ? s1 : s0;
+                    s = __builtin_amdgcn_mfma_f32_16x16x32_bf16(lds_read_b128(ka + (k_begin + k < k_end ? k : 0) * 64), qf[k], s, 0, 0, 0);
+                }
+            } else {
+                int k = 0;
+                const int n = k_end - k_begin;
+                for (; k + 2 <= n; k += 2) {
+                    s0 = __builtin_amdgcn_mfma_f32_16x16x32_bf16(lds_read_b128(ka + k * 64), lds_read_b128(qa + k * 64), s0, 0, 0, 0);
+                    s1 = __builtin_amdgcn_mfma_f32_16x16x32_bf16(lds_read_b128(ka + k * 64 + 64), lds_read_b128(qa + k * 64 + 64), s1, 0, 0, 0);
+                }
+                if (k < n)
+                    s0 = __builtin_amdgcn_mfma_f32_16x16x32_bf16(lds_read_b128(ka + k * 64), lds_read_b128(qa + k * 64), s0, 0, 0, 0);
             }
-            *reinterpret_cast<f32x4*>(s_out) = s0;
+            *reinterpret_cast<f32x4*>(s_out) = s0 + s1;
         }
         __syncthreads();
-        bf16x8 ph[QT][2], pl[QT][2];
+        {
+            f32x2 s = (*reinterpret_cast<const f32x2*>(s_in) + *reinterpret_cast<const f32x2*>(s_in + ROWS * kSPitch)) * p.scale_log2;
+#pragma unroll
+            for (int e = 0; e < 2; ++e)
+                if (t * KT + wk + e > lim) s[e] = -INFINITY;
+            const float mx = row_max(fmaxf(s[0], s[1]));
+            float alpha = 1.f;
+            if (mx > m + 8.f) {
+                alpha = __builtin_amdgcn_exp2f(m - mx);
+                m = mx;
+            }
+            const float ref = m == -INFINITY ? 0.f : m;             // (nothing seen yet: the weights below are 0)
+            const f32x2 w = {__builtin_amdgcn_exp2f(s[0] - ref), __builtin_amdgcn_exp2f(s[1] - ref)};
+            l = l * alpha + (w[0] + w[1]);
+            const bf16x2 hi = __builtin_convertvector(w, bf16x2);
+            *reinterpret_cast<bf16x2*>(p_out) = hi;
+            *reinterpret_cast<bf16x2*>(p_out + ROWS * kPPitch) = __builtin_convertvector(w - __builtin_convertvector(hi, f32x2), bf16x2);
+            if (wk == 0) ldsA[wr] = alpha;
+        }
+        __syncthreads();
+        bf16x8 ph[QT], pl[QT];
 #pragma unroll
         for (int qt = 0; qt < QT; ++qt) {
-            const float* sr = ldsS + (qt * 16 + lq) * kSPitch + lc * 4;
-            f32x4 s[4];
-            float mx = -INFINITY;
-#pragma unroll
-            for (int u = 0; u < 4; ++u) {
-                s[u] = *reinterpret_cast<const f32x4*>(sr + u * 16);
-                mx = fmaxf(mx, fmaxf(fmaxf(s[u][0], s[u][1]), fmaxf(s[u][2], s[u][3])));
-            }
-            mx = fmaxf(mx, __shfl_xor(mx, 16));
-            mx = fmaxf(mx, __shfl_xor(mx, 32));
-            const float mn = fmaxf(m[qt], mx), ref = mn == -INFINITY ? 0.f : mn;
-            const float alpha = __builtin_amdgcn_exp2f(m[qt] - ref);
-            float sum = 0.f;
-#pragma unroll
-            for (int kk = 0; kk < 2; ++kk) {
-                f32x8 pv;
-#pragma unroll
-                for (int e = 0; e < 8; ++e) {
-                    pv[e] = __builtin_amdgcn_exp2f(s[kk * 2 + (e >> 2)][e & 3] - ref);
-                    sum += pv[e];
-                }
-                ph[qt][kk] = __builtin_convertvector(pv, bf16x8);
-                pl[qt][kk] = __builtin_convertvector(pv - __builtin_convertvector(ph[qt][kk], f32x8), bf16x8);
-            }
-            l[qt] = l[qt] * alpha + sum;
-            if (__any(mn != m[qt])) {
+            ph[qt] = lds_read_b128(p_in + qt * 16 * kPPitch);
+            pl[qt] = lds_read_b128(p_in + (ROWS + qt * 16) * kPPitch);
+            const float alpha = ldsA[qt * 16 + lq];
+            if (__any(alpha != 1.f)) {
 #pragma unroll
                 for (int nb = 0; nb < NBW; ++nb) o[qt][nb] *= alpha;
             }
-            m[qt] = mn;
         }
 #pragma unroll
-        for (int nb = 0; nb < NBW; ++nb) {
-            const int col = (wave + nb * NW) * 16;
-            if (col < R) {                          // wave-uniform
+        for (int nb = 0; nb < NBW; ++nb)
+            if (KS || (wave * NBW + nb) * 16 < R) { // wave-uniform
+                const bf16x4 v0 = lds_read_tr(va + nb * 32), v1 = lds_read_tr(va + 16 * pitch + nb * 32);
+                const bf16x8 vf = __builtin_shufflevector(v0, v1, 0, 1, 2, 3, 4, 5, 6, 7);
 #pragma unroll
-                for (int kk = 0; kk < 2; ++kk) {
-                    const unsigned char* va = ldsK + vra + kk * 32 * pitch + col * 2;
-                    const bf16x4 v0 = lds_read_tr(va), v1 = lds_read_tr(va + 16 * pitch);
-                    const bf16x8 vf = __builtin_shufflevector(v0, v1, 0, 1, 2, 3, 4, 5, 6, 7);
+                for (int qt = 0; qt < QT; ++qt) o[qt][nb] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, ph[qt], o[qt][nb], 0, 0, 0);
 #pragma unroll
-                    for (int qt = 0; qt < QT; ++qt) {
-                        o[qt][nb] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, ph[qt][kk], o[qt][nb], 0, 0, 0);
-                        o[qt][nb] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, pl[qt][kk], o[qt][nb], 0, 0, 0);
-                    }
-                }
+                for (int qt = 0; qt < QT; ++qt) o[qt][nb] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, pl[qt], o[qt][nb], 0, 0, 0);
             }
-        }
         __syncthreads();
+    };
+    int t = t_begin;
+    for (; t + 3 < t_end; t += 2) {                 // branch-free prefetch: the waits count only the tile being consumed
+        process(std::true_type{}, t, kx);
+        process(std::true_type{}, t + 1, ky);
+    }
+    for (; t < t_end; t += 2) {
+        process(std::false_type{}, t, kx);
+        if (t + 1 < t_end) process(std::false_type{}, t + 1, ky);
     }
 
-    // o[qt][nb][e] = O[row qt * 16 + lq][(wave + nb * NW) * 16 + lc * 4 + e]
+    // o[qt][nb][e] = O[row qt * 16 + lq][(wave * NBW + nb) * 16 + lc * 4 + e]
     const int Rp = (R + 15) / 16 * 16;
     const int64_t slot = ((int64_t)b * p.n_groups + group) * p.nsplit + split;
+    l = row_sum(l);
+    if (wk == 0) {
+        ldsA[wr] = l > 0.f ? 1.0f / l : 0.f;
+        if (p.nsplit > 1) {
+            float* ml = p.ws + (int64_t)p.B * p.n_groups * p.nsplit * ROWS * Rp + (slot * ROWS + wr) * 2;
+            ml[0] = m;
+            ml[1] = l;
+        }
+    }
+    __syncthreads();
 #pragma unroll
     for (int qt = 0; qt < QT; ++qt) {
-        l[qt] += __shfl_xor(l[qt], 16);
-        l[qt] += __shfl_xor(l[qt], 32);
         const int r = qt * 16 + lq;
-        const bool valid = row0 + r < nrows;
-        const float inv = l[qt] > 0.f ? 1.0f / l[qt] : 0.f;
-        if (p.nsplit > 1 && wave == 0 && lc == 0) {
-            float* ml = p.ws + (int64_t)p.B * p.n_groups * p.nsplit * ROWS * Rp + (slot * ROWS + r) * 2;
-            ml[0] = m[qt];
-            ml[1] = l[qt];
-        }
+        const float inv = ldsA[r];
 #pragma unroll
         for (int nb = 0; nb < NBW; ++nb) {
-            const int c = (wave + nb * NW) * 16 + lc * 4;
-            if ((wave + nb * NW) * 16 >= R) continue;
+            const int c = (wave * NBW + nb) * 16 + lc * 4;
+            if ((wave * NBW + nb) * 16 >= R) continue;
             if (p.nsplit > 1) {
                 *reinterpret_cast<f32x4*>(p.ws + (slot * ROWS + r) * Rp + c) = o[qt][nb];
                 continue;
             }
-            if (!valid) continue;
+            if (row0 + r >= nrows) continue;
             bf16_t* op = reinterpret_cast<bf16_t*>(p.out) + ((int64_t)q0 * p.H + row0 + r) * R + c;
             if (R % 4 == 0) {
                 if (c < R) *reinterpret_cast<bf16x4*>(op) = __builtin_convertvector(o[qt][nb] * inv, bf16x4);
@@ -207,11 +246,13 @@ __global__ __launch_bounds__(256 * QT, 1) void latent_absorbed_kernel(const Late
     }
 }
 
-int lds_bytes(int W, int qt) { return (KT + 16 * qt) * row_pitch(W) + 16 * qt * kSPitch * 4; }
+int lds_bytes(int W, int qt, bool q_in_regs) {
+    return (KT + (q_in_regs ? 0 : 16 * qt)) * row_pitch(W) + 16 * qt * (2 * kSPitch * 4 + 4 + 2 * kPPitch);
+}
 
-template <int QT, int NBW>
+template <int QT, int NBW, int KS = 0>
 int launch(const LatentParams& p, hipStream_t st) {
-    auto k = latent_absorbed_kernel<QT, NBW>;
+    auto k = latent_absorbed_kernel<QT, NBW, KS>;
     static MdPerDeviceOnce once;
     if (once.first() && hipFuncSetAttribute(reinterpret_cast<const void*>(k), hipFuncAttributeMaxDynamicSharedMemorySize,
                                             160 * 1024) != hipSuccess) {
@@ -221,7 +262,7 @@ int launch(const LatentParams& p, hipStream_t st) {
     }
     const int64_t grid = (int64_t)p.B * p.n_groups * p.nsplit;
     MD_CHECK_ARG(grid < ((int64_t)1 << 31), "md_latent_attn: grid too large");
-    hipLaunchKernelGGL(k, dim3((unsigned)grid), dim3(256 * QT), lds_bytes(p.W, QT), st, p);
+    hipLaunchKernelGGL(k, dim3((unsigned)grid), dim3(256 * QT), lds_bytes(p.W, QT, KS > 0), st, p);
     return MD_OK;
 }
 
@@ -235,10 +276,11 @@ int blocks_per_wave(int kv_rank, int W, int qt) {
 }  // namespace
 
 bool md_internal_latent_absorbed_ok(int kv_rank, int W, int qt) {
-    return blocks_per_wave(kv_rank, W, qt) > 0 && lds_bytes(W, qt) <= 160 * 1024;
+    return blocks_per_wave(kv_rank, W, qt) > 0 && lds_bytes(W, qt, false) <= 160 * 1024;
 }
 
 int md_internal_latent_absorbed(const LatentParams& p, int qt, hipStream_t st) {
+    if (p.kv_rank == 512 && p.W == 576) return qt == 1 ? launch<1, 8, 18>(p, st) : launch<2, 4, 18>(p, st);   // usual for large models
     const int n = blocks_per_wave(p.kv_rank, p.W, qt);
     if (qt == 1) return n == 1 ? launch<1, 1>(p, st) : n == 2 ? launch<1, 2>(p, st) : n == 4 ? launch<1, 4>(p, st) : launch<1, 8>(p, st);
     return n == 1 ? launch<2, 1>(p, st) : n == 2 ? launch<2, 2>(p, st) : launch<2, 4>(p, st);
