@@ -81,7 +81,7 @@ __global__ __launch_bounds__(256 * QT, 2) void latent_absorbed_kernel(const Late
                                                           ((int64_t)page * p.page_size + pos % p.page_size) * W);
 #pragma unroll
         for (int i = 0; i < MAXP; ++i)
-            if (KS * 128 % NT == 0 || i * NT + tid < pieces) kr[i] = __builtin_nontemporal_load(src + i * NT + tid);
+            if ((KS > 0 && KS * 128 % NT == 0) || i * NT + tid < pieces) kr[i] = __builtin_nontemporal_load(src + i * NT + tid);
     };
     auto stage = [&](int t, u32x4 (&kr)[MAXP]) {
         if (t * KT + KT - 1 > written) {                            // rows not written yet may hold anything (NaN)
@@ -91,7 +91,7 @@ __global__ __launch_bounds__(256 * QT, 2) void latent_absorbed_kernel(const Late
         }
 #pragma unroll
         for (int i = 0; i < MAXP; ++i)
-            if (KS * 128 % NT == 0 || i * NT + tid < pieces) *reinterpret_cast<u32x4*>(ldsK + at[i]) = kr[i];
+            if ((KS > 0 && KS * 128 % NT == 0) || i * NT + tid < pieces) *reinterpret_cast<u32x4*>(ldsK + at[i]) = kr[i];
     };
     u32x4 kx[MAXP], ky[MAXP];
     if (t_begin < t_end) issue(t_begin, kx);

@@ -118,6 +118,13 @@ def test_every_entry_point_rejects_null_arguments():
     assert lib.md_xattn_fused_supported(None) == 0 and lib.md_linear_planes_count(3, 64, 2048, 1024) == 0
     assert lib.md_linear_planes_count(1, 64, 2048, 1024) > 0 and lib.md_linear_planes_count(1, 64, 2040, 1024) == 0
     skip |= {"md_xattn_head_pad", "md_xattn_fused_supported", "md_linear_planes_count"}
+    # ... and of the latent attention
+    assert lib.md_latent_row_width(0, 8) == 0 and lib.md_latent_row_width(100, 20) == 128 and lib.md_latent_row_width(1000, 64) == 0
+    assert lib.md_latent_prefill_supported(None) == 0 and lib.md_latent_workspace_bytes(None) == 0
+    ha = _lib.HeadLinearArgs()
+    ha.x = ha.w = ha.out = 4096
+    assert lib.md_head_linear(ctypes.byref(ha), None) < 0 and "bad shape" in lib.md_last_error_string().decode()
+    skip |= {"md_latent_row_width", "md_latent_prefill_supported"}
     for name, (restype, argtypes) in _lib._SIGNATURES.items():
         if name in skip:
             continue
