@@ -20,6 +20,21 @@ typedef float f32x16 __attribute__((ext_vector_type(16)));
 constexpr int DK = MD_LATENT_DK, KT = 64, NW = kLatentPrefillRows / 32, NT = 64 * NW;
 constexpr int KROW = DK * 2 + 16;
 
+// weights -> upper 16 bits (truncated: bf16) and the rest rounded to bf16
+__device__ __forceinline__ void split(const f32x8 w, bf16x8& hi, bf16x8& lo) {
+    u32x4 h;
+    f32x8 r;
+#pragma unroll
+    for (int e = 0; e < 8; e += 2) {
+        const unsigned int a = __float_as_uint(w[e]), b = __float_as_uint(w[e + 1]);
+        h[e / 2] = __builtin_amdgcn_perm(b, a, 0x07060302);
+        r[e] = w[e] - __uint_as_float(a & 0xffff0000u);
+        r[e + 1] = w[e + 1] - __uint_as_float(b & 0xffff0000u);
+    }
+    hi = *reinterpret_cast<const bf16x8*>(&h);
+    lo = __builtin_convertvector(r, bf16x8);
+}
+
 template <int DV>
 constexpr int stage_bytes() { return KT * KROW + (KT / 32) * (DV / 16) * kVSub; }
 
@@ -54,27 +69,47 @@ __global__ __launch_bounds__(NT, 2) void latent_prefill_kernel(const LatentParam
 
     bf16x8 qf[KS];
     {
+        // rows past the last one read the first row's query; every load is requested before the first is used
         const bf16_t* qp = reinterpret_cast<const bf16_t*>(p.q) + ((int64_t)(q0 + (valid ? qi : 0)) * p.H + h) * dq;
         const float* cs = p.cos_sin + (int64_t)min(max(pos, 0), p.max_pos - 1) * p.rot_pairs * 2;
         const bf16x8 z = {0, 0, 0, 0, 0, 0, 0, 0};
         const float sign = p.scale_log2 < 0.f ? -1.f : 1.f;
+        f32x4 ca[KS], cb[KS];                                       // (cos, sin) of the four pairs of an 8-element piece
 #pragma unroll
         for (int ks = 0; ks < KS; ++ks) {
-            const int d = ks * 16 + kh * 8;
-            const bf16x8 raw = valid && d < dq ? *reinterpret_cast<const bf16x8*>(qp + d) : z;
-            f32x8 v = __builtin_convertvector(raw, f32x8);
-            if (d >= p.dim && d < dq) {
+            const int d = ks * 16 + kh * 8, e = d - p.dim;
+            qf[ks] = d < dq ? *reinterpret_cast<const bf16x8*>(qp + d) : z;
+            ca[ks] = cb[ks] = f32x4{1.f, 0.f, 1.f, 0.f};
+            if (p.rot_pairs % 4 == 0) {                             // uniform: pieces are rotated as a whole or not at all
+                if (e >= 0 && e < 2 * p.rot_pairs) {
+                    ca[ks] = *reinterpret_cast<const f32x4*>(cs + e);
+                    cb[ks] = *reinterpret_cast<const f32x4*>(cs + e + 4);
+                }
+            } else if (e >= 0) {
 #pragma unroll
-                for (int e = 0; e < 8; e += 2) {
-                    const int i = (d - p.dim + e) >> 1;
-                    if (i < p.rot_pairs) {
-                        const float c = cs[2 * i], s = cs[2 * i + 1], a = v[e], w = v[e + 1];
-                        v[e] = a * c - w * s;
-                        v[e + 1] = w * c + a * s;
-                    }
+                for (int u = 0; u < 4; ++u) {
+                    if (e + u < 2 * p.rot_pairs) ca[ks][u] = cs[e + u];
+                    if (e + 4 + u < 2 * p.rot_pairs) cb[ks][u] = cs[e + 4 + u];
                 }
             }
-            qf[ks] = __builtin_convertvector(v * sign, bf16x8);
+        }
+#pragma unroll
+        for (int ks = 0; ks < KS; ++ks) {
+            f32x8 v = __builtin_convertvector(qf[ks], f32x8);
+#pragma unroll
+            for (int u = 0; u < 4; ++u) {
+                const float c = u < 2 ? ca[ks][u * 2] : cb[ks][u * 2 - 4], s = u < 2 ? ca[ks][u * 2 + 1] : cb[ks][u * 2 - 3];
+                const float x = v[u * 2], y = v[u * 2 + 1];
+                v[u * 2] = (x * c - y * s) * sign;
+                v[u * 2 + 1] = (y * c + x * s) * sign;
+            }
+            qf[ks] = __builtin_convertvector(v, bf16x8);
+        }
+    }
+    if (dq < DK) {                                                  // the images' columns behind a key stay zero
+        for (int c = tid; c < 2 * KT * (DK - dq) / 8; c += NT) {
+            const int row = c / ((DK - dq) / 8), d = dq + c % ((DK - dq) / 8) * 8;
+            *reinterpret_cast<u32x4*>(smem + (row / KT) * STAGE + row % KT * KROW + d * 2) = u32x4{0u, 0u, 0u, 0u};
         }
     }
     f32x16 o[DB];
@@ -85,38 +120,35 @@ __global__ __launch_bounds__(NT, 2) void latent_prefill_kernel(const LatentParam
     float m = -INFINITY, l = 0.f;
 
     u32x4 kreg[NK], vreg[NV];
-    const u32x4 z4 = {0u, 0u, 0u, 0u};
-    const int64_t ldkv = (int64_t)p.H * (p.dim + p.vdim);
-    const bf16_t* kv = reinterpret_cast<const bf16_t*>(p.kv);
-    const int hk = h * p.dim, hv = p.H * p.dim + h * p.vdim;
+    const int ldkv = p.H * (p.dim + p.vdim), hk = h * p.dim, hv = p.H * p.dim + h * p.vdim;
     auto issue = [&](int t) {
-        const int kp0 = t * KT;
-        const int64_t crow = (int64_t)p.page_indices[pg0 + kp0 / p.page_size] * p.page_size + kp0 % p.page_size;
-        const bf16_t* rp = reinterpret_cast<const bf16_t*>(p.cache) + crow * p.W + p.kv_rank;
+        const int kp0 = t * KT, rem = ctx - 1 - kp0;                // rows past the context repeat its last row: they are masked
+        const bf16_t* kvb = reinterpret_cast<const bf16_t*>(p.kv) + (int64_t)(c0 + kp0) * ldkv;
+        const bf16_t* rpb = reinterpret_cast<const bf16_t*>(p.cache) + p.kv_rank +
+                            ((int64_t)p.page_indices[pg0 + kp0 / p.page_size] * p.page_size + kp0 % p.page_size) * p.W;
 #pragma unroll
         for (int i = 0; i < NK; ++i) {
-            const int c = i * NT + tid, row = c / (DK / 8), d = (c % (DK / 8)) * 8;
-            kreg[i] = z4;
-            if (kp0 + row < ctx && d < dq)
-                kreg[i] = d < p.dim ? *reinterpret_cast<const u32x4*>(kv + (c0 + kp0 + row) * ldkv + hk + d)
-                                    : *reinterpret_cast<const u32x4*>(rp + (int64_t)row * p.W + d - p.dim);
+            const int c = i * NT + tid, row = min(c / (DK / 8), rem), d = (c % (DK / 8)) * 8;
+            const bf16_t* src = d < p.dim ? kvb + (row * ldkv + hk + d) : rpb + (row * p.W + d - p.dim);
+            if (d < dq) kreg[i] = *reinterpret_cast<const u32x4*>(src);
         }
 #pragma unroll
         for (int i = 0; i < NV; ++i) {
-            const int c = i * NT + tid, row = c / (DV / 8), d = (c % (DV / 8)) * 8;
-            vreg[i] = kp0 + row < ctx && d < p.vdim ? *reinterpret_cast<const u32x4*>(kv + (c0 + kp0 + row) * ldkv + hv + d) : z4;
+            const int c = i * NT + tid, row = min(c / (DV / 8), rem), d = (c % (DV / 8)) * 8;
+            if (d < p.vdim) vreg[i] = *reinterpret_cast<const u32x4*>(kvb + (row * ldkv + hv + d));
         }
     };
     auto stage = [&](unsigned char* img) {
 #pragma unroll
         for (int i = 0; i < NK; ++i) {
             const int c = i * NT + tid;
-            *reinterpret_cast<u32x4*>(img + (c / (DK / 8)) * KROW + (c % (DK / 8)) * 16) = kreg[i];
+            if ((c % (DK / 8)) * 8 < dq) *reinterpret_cast<u32x4*>(img + (c / (DK / 8)) * KROW + (c % (DK / 8)) * 16) = kreg[i];
         }
 #pragma unroll
-        for (int i = 0; i < NV; ++i) {
+        for (int i = 0; i < NV; ++i) {                              // (columns behind a value reach only sums that are not stored)
             const int c = i * NT + tid, row = c / (DV / 8), ch = c % (DV / 8);
-            *reinterpret_cast<u32x4*>(img + K_BYTES + (row >> 5) * VG + (ch >> 1) * kVSub + (row & 31) * 32 + (ch & 1) * 16) = vreg[i];
+            if (ch * 8 < p.vdim)
+                *reinterpret_cast<u32x4*>(img + K_BYTES + (row >> 5) * VG + (ch >> 1) * kVSub + (row & 31) * 32 + (ch & 1) * 16) = vreg[i];
         }
     };
     const int kra0 = j * KROW + kh * 16, lq = lane & 15;
@@ -164,8 +196,8 @@ __global__ __launch_bounds__(NT, 2) void latent_prefill_kernel(const LatentParam
                     pv[e] = __builtin_amdgcn_exp2f(fmaf(sc[u][s16 * 8 + e], sl2, -m));
                     l += pv[e];
                 }
-                const bf16x8 ph = __builtin_convertvector(pv, bf16x8);
-                const bf16x8 pl = __builtin_convertvector(pv - __builtin_convertvector(ph, f32x8), bf16x8);
+                bf16x8 ph, pl;
+                split(pv, ph, pl);
 #pragma unroll
                 for (int db = 0; db < DB; ++db) {
                     const unsigned char* vb = img + u * VG + db * kVSub + vra0 + s16 * 16 * 32;
