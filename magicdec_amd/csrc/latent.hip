@@ -220,45 +220,42 @@ __global__ __launch_bounds__(256) void head_linear_f32_kernel(const HeadLinearPa
 }
 
 // ------------------------------------------------------------------------------------------------ merge, gather
-// partials of the kv splits: ws = sums [slot][rows_wg][Rp], then (reference, weight) [slot][rows_wg][2]; slot = (b * groups + g) * nsplit + s
+// partials of the kv splits: ws = sums [slot][rows_wg][Rp], then (reference, weight) [slot][rows_wg][2]; slot =
+// (b * groups + g) * nsplit + s.  Lane s knows split s's factor; Q wavefronts share 256 columns of one row, each adds every Q-th split
+// (four requested together), and their sums meet in LDS in order
+template <int Q>
 __global__ __launch_bounds__(256) void latent_merge_kernel(const LatentParams p, int rows_wg, int Rp) {
-    const int b = blockIdx.y, q0 = p.qo_indptr[b], nrows = (p.qo_indptr[b + 1] - q0) * p.H;
-    const int d4 = Rp / 4;
-    const int id = blockIdx.x * 256 + threadIdx.x;
-    const int row = id / d4, d = (id - row * d4) * 4;
-    if (row >= nrows) return;
-    const int g = row / rows_wg, r = row - g * rows_wg;
+    __shared__ f32x4 part[4][64];
+    const int lane = threadIdx.x & 63, all = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), wave = Q == 4 ? all : 0;
+    const int b = blockIdx.z, row = Q == 4 ? blockIdx.x : blockIdx.x * 4 + all, q0 = p.qo_indptr[b];
+    if (row >= (p.qo_indptr[b + 1] - q0) * p.H) return;               // (Q == 4: whole workgroup)
+    const int g = row / rows_wg, r = row - g * rows_wg, d = (blockIdx.y * 64 + lane) * 4;
     const int64_t slot0 = ((int64_t)b * p.n_groups + g) * p.nsplit;
     const float* ml = p.ws + (int64_t)p.B * p.n_groups * p.nsplit * rows_wg * Rp;
-    float m = -INFINITY;
-    // eight splits requested together, added in order
-    for (int s0 = 0; s0 < p.nsplit; s0 += 8) {
-        float t[8];
-#pragma unroll
-        for (int u = 0; u < 8; ++u) t[u] = s0 + u < p.nsplit ? ml[((slot0 + s0 + u) * rows_wg + r) * 2] : -INFINITY;
-#pragma unroll
-        for (int u = 0; u < 8; ++u) m = fmaxf(m, t[u]);
-    }
+    f32x2 t = {-INFINITY, 0.f};
+    if (lane < p.nsplit) t = *reinterpret_cast<const f32x2*>(ml + ((slot0 + lane) * rows_wg + r) * 2);
+    const float m = wave_reduce_max(t[0]), w = t[0] == -INFINITY ? 0.f : __builtin_amdgcn_exp2f(t[0] - m);
+    const float l = wave_reduce_sum(t[1] * w);
     f32x4 o = {0.f, 0.f, 0.f, 0.f};
-    float l = 0.f;
-    for (int s0 = 0; s0 < p.nsplit; s0 += 8) {
-        f32x2 t[8];
-        f32x4 v[8];
+    for (int s0 = wave; s0 < p.nsplit; s0 += 4 * Q) {
+        f32x4 v[4];
 #pragma unroll
-        for (int u = 0; u < 8; ++u)
-            if (s0 + u < p.nsplit) {                                  // uniform
-                const int64_t at = (slot0 + s0 + u) * rows_wg + r;
-                t[u] = *reinterpret_cast<const f32x2*>(ml + at * 2);
-                v[u] = *reinterpret_cast<const f32x4*>(p.ws + at * Rp + d);
-            }
+        for (int u = 0; u < 4; ++u)
+            if (s0 + Q * u < p.nsplit && d < Rp) v[u] = *reinterpret_cast<const f32x4*>(p.ws + ((slot0 + s0 + Q * u) * rows_wg + r) * Rp + d);
 #pragma unroll
-        for (int u = 0; u < 8; ++u)
-            if (s0 + u < p.nsplit) {
-                const float w = t[u][0] == -INFINITY ? 0.f : __builtin_amdgcn_exp2f(t[u][0] - m);
-                o += v[u] * w;
-                l += t[u][1] * w;
+        for (int u = 0; u < 4; ++u)
+            if (s0 + Q * u < p.nsplit) {                              // uniform
+                const float f = __shfl(w, s0 + Q * u);
+                if (d < Rp) o += v[u] * f;
             }
     }
+    if constexpr (Q == 4) {
+        part[wave][lane] = o;
+        __syncthreads();
+        if (wave > 0) return;
+        o = (part[0][lane] + part[1][lane]) + (part[2][lane] + part[3][lane]);
+    }
+    if (d >= Rp) return;
     const float inv = l > 0.f ? 1.0f / l : 0.f;
     bf16_t* op = reinterpret_cast<bf16_t*>(p.out) + ((int64_t)q0 * p.H + row) * p.kv_rank + d;
     if (p.kv_rank % 4 == 0) {
@@ -302,7 +299,7 @@ int kv_splits(const md_latent_args* a) {
     long want = (target + groups - 1) / groups;
     const long cap = tiles / 8 > 1 ? tiles / 8 : 1;                  // >= 256 keys per workgroup
     if (want > cap) want = cap;
-    return (int)(want < 1 ? 1 : want > 64 ? 64 : want);
+    return (int)(want < 1 ? 1 : want > 64 ? 64 : want);            // (the merge holds a split per lane)
 }
 
 int check_args(const char* who, const md_latent_args* a) {
@@ -497,8 +494,9 @@ extern "C" int md_latent_attn(const md_latent_args* a, md_stream_t stream) {
     if (rc != MD_OK) return rc;
     if (p.nsplit > 1) {
         const int Rp = (a->kv_rank + 15) / 16 * 16;
-        const int64_t threads = (int64_t)a->n_max * a->H * (Rp / 4);
-        hipLaunchKernelGGL(latent_merge_kernel, dim3((unsigned)((threads + 255) / 256), a->B), dim3(256), 0, st, p, 16 * qt, Rp);
+        const int rows = a->n_max * a->H, cols = (Rp + 255) / 256;
+        if (p.nsplit > 8) hipLaunchKernelGGL((latent_merge_kernel<4>), dim3(rows, cols, a->B), dim3(256), 0, st, p, 16 * qt, Rp);
+        else hipLaunchKernelGGL((latent_merge_kernel<1>), dim3((rows + 3) / 4, cols, a->B), dim3(256), 0, st, p, 16 * qt, Rp);
     }
     MD_CHECK_LAUNCH("md_latent_attn");
     return MD_OK;
