@@ -199,6 +199,13 @@ class _BackendBase:
         B = self.batch_size
         return sorted({B * int(n) for n in (1,) + ((2,) if two_token_step else ()) + tuple(per_request) if n})
 
+    def _last_rows(self, n):
+        """Extra prefill arguments of models addressed by position: logits for the last of every request's n rows only (their
+        portions are long; encode then returns [B, 1])."""
+        if not self.mapped:
+            return {}
+        return dict(head_rows=torch.arange(1, self.batch_size + 1, device=self.device) * n - 1)
+
     def _prefill_begin(self):
         """Prefill-sized products run on the library GEMM over the row-major weights: re-materialise the ones released
         after the previous prefill (Transformer.restore_rowmajor)."""
@@ -311,10 +318,12 @@ class SnapKVTargetBackend(_BackendBase):
             self.model.skip_head = i != num_chunks - 1
             tokens = self.model.prefill(ids, self.cachelens, self._qo(n), self._t.table((n, done + n)), is_last=is_last,
                                         draft_tab=self._d.table() if (self.is_spec and is_last) else None,
-                                        ctx_len=done + n)
+                                        ctx_len=done + n, **self._last_rows(n))
             self.cachelens += n
             done += n
         self.model.skip_head = False
+        if self.mapped:
+            tokens = tokens.view(-1, 1)
         if self.is_spec:
             if not is_last:
                 raise ValueError("SnapKV self-speculation: prefix_len is a multiple of 128, so no last chunk ran the "
@@ -514,10 +523,12 @@ class SnapKVDraftBackend(_BackendBase):
             self.model.skip_head = i != num_chunks - 1
             tokens = self.model.prefill(ids, self.cachelens, self._qo(n), self._t.table((n, done + n)), is_last=is_last,
                                         draft_tab=self._d.table() if (self.is_compress and is_last) else None,
-                                        ctx_len=done + n)
+                                        ctx_len=done + n, **self._last_rows(n))
             self.cachelens += n
             done += n
         self.model.skip_head = False
+        if self.mapped:
+            tokens = tokens.view(-1, 1)
         if self.is_compress and not is_last:
             raise ValueError("SnapKV draft: prefix_len is a multiple of 128, so no last chunk ran the select and the "
                              "draft cache is empty (need (prefix_len - window_size) % 128 == 0)")

@@ -404,7 +404,9 @@ class LayeredTransformer(Transformer):
         flat = idx.reshape(-1).contiguous()
         rows = ops.StepRows(qo_indptr, offsets, idx.shape[1] if idx.dim() == 2 else n_max, tab.slots)
         x = self._embed(flat, rows, tab)
-        ctx = ops.LatentContext(*tab.lengths, x.device) if tab.lengths is not None and self.output.weight.dtype == torch.bfloat16 else None
+        ctx = None
+        if tab.lengths is not None and self.output.weight.dtype == torch.bfloat16:
+            ctx = ops.LatentContext(*tab.lengths, x.device)
         delta = None
         for i, layer in enumerate(self.layers):
             att, kvc = layer.attention, layer.attention.kv_cache

@@ -46,14 +46,15 @@ __device__ __forceinline__ float row_sum(float v) {
 template <int QT, int NBW, int KS>
 __global__ __launch_bounds__(256 * QT, 2) void latent_absorbed_kernel(const LatentParams p) {
     constexpr int ROWS = 16 * QT, NT = 256 * QT, PARTS = 2 * QT;                 // PARTS: of a score's depth
-    constexpr int MAXP = KS ? (KS * 128 + NT - 1) / NT : NBW + 2;                // 16-byte pieces of a tile per thread (W <= 64 QT NBW + 128)
+    constexpr int MAXP = KS ? (KS * 128 + NT - 1) / NT : NBW + 2;                // 16-byte pieces of a tile per thread
     constexpr int KH = (KS + PARTS - 1) / PARTS;
     extern __shared__ __attribute__((aligned(16))) unsigned char smem[];
     const int tid = threadIdx.x, lane = tid & 63, lq = lane & 15, lc = lane >> 4;
     const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
     const int W = KS ? KS * 32 : p.W, pitch = row_pitch(W), R = p.kv_rank, image = KT * pitch;
     unsigned char* ldsQ = smem + 2 * image;
-    float* ldsS = reinterpret_cast<float*>(ldsQ + (KS ? 0 : ROWS * pitch));     // [part][row][key]; behind a row of part 0: its factor
+    // scores [part][row][key]; behind a row of part 0: the row's factor
+    float* ldsS = reinterpret_cast<float*>(ldsQ + (KS ? 0 : ROWS * pitch));
     unsigned char* ldsP = reinterpret_cast<unsigned char*>(ldsS + PARTS * ROWS * kSPitch);   // weights: bf16 parts, then rests
 
     // request fastest: with a multiple of 8 requests one request's workgroups share an XCD (and its L2)
@@ -290,7 +291,7 @@ int launch(const LatentParams& p, hipStream_t st) {
     return MD_OK;
 }
 
-// column blocks per wavefront (a power of two) that cover kv_rank and whose piece count covers W; 0: none
+// column blocks per wavefront (a power of two) that cover kv_rank and whose MAXP pieces cover a tile of rows of W; 0: none
 int blocks_per_wave(int kv_rank, int W, int qt) {
     for (int n = 1; n * qt <= 8; n *= 2)
         if (kv_rank <= 64 * n * qt && W <= 64 * n * qt + 128) return n;

@@ -58,11 +58,10 @@ __global__ __launch_bounds__(NT, 2) void latent_prefill_kernel(const LatentParam
     const int c0 = p.ctx_indptr[b], ctx = min(p.ctx_indptr[b + 1] - c0, cap);
     const int wg_last = min(pos_b + min(qg * kLatentPrefillRows + kLatentPrefillRows, n_b) - 1, ctx - 1);
     if (wg_last < 0) return;
-    const int qi = qg * kLatentPrefillRows + wave * 32 + j;
+    const int w0 = qg * kLatentPrefillRows + wave * 32, qi = w0 + j;            // the wave's first row, this lane's row
     const bool valid = qi < n_b;
     const int pos = pos_b + qi, lim = valid ? min(pos, ctx - 1) : 0;
-    const int lim_lo = min(pos_b + qg * kLatentPrefillRows + wave * 32, ctx - 1);     // the wave's first row
-    const int my_last = qg * kLatentPrefillRows + wave * 32 < n_b ? min(pos_b + min(qg * kLatentPrefillRows + wave * 32 + 32, n_b) - 1, ctx - 1) : -1;
+    const int lim_lo = min(pos_b + w0, ctx - 1), my_last = w0 < n_b ? min(pos_b + min(w0 + 32, n_b) - 1, ctx - 1) : -1;
     const int t1 = wg_last / KT, my1 = my_last >= 0 ? my_last / KT : -1;
     const int dq = p.dim + p.rot_dim;
     const float sl2 = fabsf(p.scale_log2);

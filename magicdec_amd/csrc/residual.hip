@@ -314,12 +314,11 @@ __global__ __launch_bounds__(256) void embed_bigram_kernel(const BigramParams p)
     if (j >= p.qo_indptr[b + 1] - q0) return;
     const int pos = p.pos0[b] + j, pg0 = p.page_indptr[b], cap = (p.page_indptr[b + 1] - pg0) * p.page_size;
     const int64_t tok = clamp_token(p.tokens[q0 + j], p.vocab);
+    auto entry = [&](int at) { return p.history + (int64_t)p.page_indices[pg0 + at / p.page_size] * p.page_size + at % p.page_size; };
     int64_t before = 0;
     if (j > 0) before = clamp_token(p.tokens[q0 + j - 1], p.vocab);
-    else if (pos > 0 && pos - 1 < cap) before = p.history[(int64_t)p.page_indices[pg0 + (pos - 1) / p.page_size] * p.page_size + (pos - 1) % p.page_size];
-    if (threadIdx.x == 0) {
-        if (pos >= 0 && pos < cap) p.history[(int64_t)p.page_indices[pg0 + pos / p.page_size] * p.page_size + pos % p.page_size] = (int32_t)tok;
-    }
+    else if (pos > 0 && pos - 1 < cap) before = *entry(pos - 1);
+    if (threadIdx.x == 0 && pos >= 0 && pos < cap) *entry(pos) = (int32_t)tok;
     int64_t pair = pos <= 0 ? p.buckets : (before * p.mul_before + tok * p.mul_token) % p.buckets;
     if (pair < 0) pair += p.buckets;
     const int nvec = p.width / VEC;

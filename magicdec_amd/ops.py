@@ -623,7 +623,9 @@ def fused_linear(x, weight: "PackedWeight", bias=None, swiglu=False, resid=None,
     SiLU(h1) * h3 (swiglu=True, weight = [w1; w3]) or by the bf16 residual add `resid + linear` (resid [M, N]).
     want_ssq (with resid): also return the per-row partial sums of squares [M, N/32] of the result (the producer half of
     a deferred RMSNorm).  pro (with swiglu): x is pro.h and is normalised on the fly (the consumer half)."""
-    epi = (FL_GEGLU if gelu else FL_SWIGLU) if swiglu else (FL_RESID if resid is not None else (FL_XIELU if xielu is not None else FL_NONE))
+    epi = FL_RESID if resid is not None else (FL_XIELU if xielu is not None else FL_NONE)
+    if swiglu:
+        epi = FL_GEGLU if gelu else FL_SWIGLU
     if xielu is not None and epi != FL_XIELU:
         raise ValueError("fused linear: the xIELU epilogue takes nothing beside it")
     a = _fused_args(x, weight, bias, epi)
@@ -1051,7 +1053,8 @@ def _head_linear(x, w, out, gate=None, tail=None, tail_pad=0, rotary=None, rows=
         if t.stride(-1) != 1 or t.dtype != w.dtype:
             raise ValueError("head_linear: unit inner strides and one dtype expected")
     a = _lib.HeadLinearArgs()
-    a.x, a.w, a.out, a.ldx, a.hx, a.ldo, a.ho = x.data_ptr(), w.data_ptr(), out.data_ptr(), x.stride(0), x.stride(1), out.stride(0), out.stride(1)
+    a.x, a.w, a.out = x.data_ptr(), w.data_ptr(), out.data_ptr()
+    a.ldx, a.hx, a.ldo, a.ho = x.stride(0), x.stride(1), out.stride(0), out.stride(1)
     a.M, a.H, a.N, a.K, a.dtype = M, H, w.shape[1], K, _model_dtype(w)
     if out.shape[2] < a.N + tail_pad:
         raise ValueError("head_linear: out is too narrow")
@@ -1080,7 +1083,8 @@ def latent_attention(q, s: LatentSpec, cache, rows: StepRows, page_indices, page
     lib = _lib.load()
     a = _latent_args(s, cache, rows, page_indices, page_indptr, max_pages, q.dtype)
     a.force_plain = int(plain)
-    if ctx is not None and not plain and ctx.expanded(s) and out.stride(0) % 4 == 0 and lib.md_latent_prefill_supported(ctypes.byref(a)):
+    if (ctx is not None and not plain and ctx.expanded(s) and out.stride(0) % 4 == 0 and out.data_ptr() % 8 == 0
+            and lib.md_latent_prefill_supported(ctypes.byref(a))):
         dense = torch.empty((ctx.total, s.kv_rank), dtype=q.dtype, device=q.device)
         a.ctx_indptr = ctx.indptr.data_ptr()
         check(lib.md_latent_gather(ctypes.byref(a), ctx.longest, _p(dense), _stream()), "md_latent_gather")
@@ -1092,7 +1096,8 @@ def latent_attention(q, s: LatentSpec, cache, rows: StepRows, page_indices, page
         return out
     heads = q.view(M, s.H, s.dim + s.rot_dim)
     qa = torch.empty((M, s.H, s.width), dtype=q.dtype, device=q.device)
-    _head_linear(heads[..., :s.dim], s.absorb, qa, tail=heads[..., s.dim:], tail_pad=s.width - s.kv_rank, rotary=s.rotary, rows=rows)
+    _head_linear(heads[..., :s.dim], s.absorb, qa, tail=heads[..., s.dim:], tail_pad=s.width - s.kv_rank, rotary=s.rotary,
+                 rows=rows)
     lat = torch.empty((M, s.H, s.kv_rank), dtype=q.dtype, device=q.device)
     a.q, a.out = qa.data_ptr(), lat.data_ptr()
     nbytes = lib.md_latent_workspace_bytes(ctypes.byref(a))
@@ -1139,7 +1144,7 @@ def embed_bigram(tokens, table, pairs, norm_weight, eps, mul_before, mul_token, 
     vocab, width = table.shape
     if tokens.dtype != torch.int64 or history.dtype != torch.int32 or history.dim() != 2:
         raise TypeError("embed_bigram: token ids are int64, the token history int32 [pages, page_size]")
-    if pairs.shape[1] != width or pairs.shape[0] < 2 or norm_weight.numel() != width or pairs.dtype != table.dtype or norm_weight.dtype != table.dtype:
+    if pairs.shape[1] != width or pairs.shape[0] < 2 or norm_weight.numel() != width or not (pairs.dtype == norm_weight.dtype == table.dtype):
         raise ValueError("embed_bigram: tables of different widths or dtypes")
     if page_indptr.numel() != rows.B + 1:
         raise ValueError("embed_bigram: page table of another batch")
